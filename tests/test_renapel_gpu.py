@@ -542,11 +542,13 @@ def test_latent_attention_alone(m, dtype, ops):
         got = run_mixer(part, h, cuts, cache, dtype)
         assert float((got - want).abs().max()) <= limit * float(want.abs().max()), f"cuts {cuts[:3]}"
     assert cache.kv.k.shape[1] == 1 and cache.kv.k.shape[3] == m["kv_rank"] + m["rot_dim"] and cache.kv.v.shape[2] == m["kv_rank"]
-    # prompts that start their sequences, nothing else in the step: in bfloat16 their scores are a matrix product of the step's own rows
+    # prompts that start their sequences, nothing else in the step: in bfloat16 the matrix-core kernel takes sizes in whole tiles, and for
+    # others the scores are a matrix product of the step's own rows
+    dense = dtype == torch.bfloat16 and not ops.attention_takes_latent(dtype, m["kv_rank"] + m["rot_dim"], m["kv_rank"])
     if dtype == torch.bfloat16:
         part.DENSE_SCORES = 70 * m["heads"] * length                 # (the prompt's queries in three stretches)
     cache = layer_cache(part.cache_needs(), dtype, length)
-    assert part._prompts_alone(h.cuda(), Step([1], [length], [0]), cache) == (dtype == torch.bfloat16)
+    assert part._prompts_alone(h.cuda(), Step([1], [length], [0]), cache) == dense
     for cuts in ([length], [length - 20] + [1] * 20):
         cache = layer_cache(part.cache_needs(), dtype, length)
         got = run_mixer(part, h, cuts, cache, dtype, padding=0)

@@ -1,5 +1,5 @@
 // Causal attention of every token of a step over its own sequence's cache, float32 math,
-// for any element type, head size (up to 512), head grouping and window.
+// for any element type, head size (keys up to 1024, values up to 768), head grouping and window.
 // It is the attention of the 32-bit path and the fallback of the bfloat16 path.
 //
 // Reference: crates/xrt-models/src/llama.rs:504-574 (online softmax: running maximum m and
@@ -24,6 +24,9 @@ namespace {
 
 constexpr int MAX_HEAD_DIM = 512;
 constexpr int MAX_OWNED = MAX_HEAD_DIM / XRT_WAVE;
+// Larger ones (a latent with a turned part beside it) take an instantiation of their own, with more registers and one head a wavefront.
+constexpr int LARGEST_HEAD_DIM = 1024, LARGEST_VALUE_DIM = 768;
+constexpr int LARGEST_OWNED = LARGEST_HEAD_DIM / XRT_WAVE;
 
 // eight elements from p (aligned to eight elements: a piece of a cache block), as floats, in one or two loads
 template <typename T>
@@ -305,7 +308,8 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
                           int window, const float* distance_slopes, int sink, const float* sink_scores, long q_stride,
                           const float* distance_bias, int bias_span, int stretch, hipStream_t s) {
     XRT_REQUIRE(distance_bias == nullptr || bias_span > 0, "attention: a table of biases by distance needs a distance at least");
-    XRT_REQUIRE(head_dim <= MAX_HEAD_DIM && value_dim > 0 && value_dim <= MAX_HEAD_DIM, "attention: head sizes %d and %d must be at most %d", head_dim, value_dim, MAX_HEAD_DIM);
+    XRT_REQUIRE(head_dim <= LARGEST_HEAD_DIM && value_dim > 0 && value_dim <= LARGEST_VALUE_DIM, "attention: head sizes %d and %d must be at most %d and %d", head_dim,
+                value_dim, LARGEST_HEAD_DIM, LARGEST_VALUE_DIM);
     // Query heads of a key/value head that a wavefront takes together: as many of the group as 4, for head sizes up to 128
     // (what a lane then owns of a head fits two registers a head), where that still leaves two workgroups to a compute
     // unit (a decode step of few sequences would rather have the workgroups). Either way a head's arithmetic is the same.
@@ -313,9 +317,9 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
     // Heads larger than that take two together where the group is even: a key of some hundred dims is a long row of loads,
     // which then serve both (the lanes' registers hold up to eight dims a head either way). (Tried also for steps of few
     // tokens, a decode step of 8 sequences with 16 heads of 448 dims on one key/value head: 125 -> 164 us, the workgroups being half as many.)
-    const bool large = max(head_dim, value_dim) > 2 * XRT_WAVE;
+    const bool large = max(head_dim, value_dim) > 2 * XRT_WAVE, largest = max(head_dim, value_dim) > MAX_HEAD_DIM;
     int together = large ? (group % 2 == 0 ? 2 : 1) : group % 4 == 0 ? 4 : group % 2 == 0 ? 2 : 1;
-    if ((long)tokens * (n_heads / together) < 2L * XRT_COMPUTE_UNITS) together = 1;
+    if (largest || (long)tokens * (n_heads / together) < 2L * XRT_COMPUTE_UNITS) together = 1;
     if (large && (size_t)2 * CHUNK_WAVES * together * value_dim * sizeof(float) > 48 * 1024) together = 1;      // (what the wavefronts' merge needs of LDS)
     const long items = (long)tokens * (n_heads / together);
     XRT_REQUIRE((long)tokens * n_heads < (1L << 31), "attention: too many (token, head) pairs");
@@ -336,7 +340,8 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
 #define XRT_GENERIC_WAVES(T, G_, OWNED_) do { if (side_by_side) XRT_GENERIC(T, CHUNK_WAVES, G_, OWNED_); else XRT_GENERIC(T, 1, G_, OWNED_); } while (0)
 #define XRT_GENERIC_SETS(T)                                                                                               \
     do {                                                                                                                  \
-        if (together == 4) XRT_GENERIC_WAVES(T, 4, 2);                                                                    \
+        if (largest) XRT_GENERIC_WAVES(T, 1, LARGEST_OWNED);                                                               \
+        else if (together == 4) XRT_GENERIC_WAVES(T, 4, 2);                                                                    \
         else if (together == 2 && large) XRT_GENERIC_WAVES(T, 2, MAX_OWNED);                                              \
         else if (together == 2) XRT_GENERIC_WAVES(T, 2, 2);                                                               \
         else XRT_GENERIC_WAVES(T, 1, MAX_OWNED);                                                                          \

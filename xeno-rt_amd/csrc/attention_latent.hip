@@ -1,9 +1,11 @@
 // Attention of many query heads on ONE key/value head with large keys, on the matrix cores: the shape of attention through a
 // cached latent (parts/latent.py), where all heads of a token read the same row [latent | turned key part] and the values are
-// the latents. bfloat16, the queries alone in q; key size a multiple of 32 up to 512, value size a multiple of 32 up to 512
-// (the sizes at which cache blocks lie in the tiles of cache_layout.h).
+// the latents. bfloat16, the queries alone in q; key size a multiple of 32 up to 640, value size a multiple of 32 up to 512
+// (the sizes at which cache blocks lie in the tiles of cache_layout.h). A query sees all keys at or before it, or with a window
+// the `window` newest of them.
 //
-// A wavefront takes a token, sixteen of its heads and a chunk of the sequence's cache blocks. The sixteen heads are the
+// Steps of few tokens (xrt_attention_latent).
+// A wavefront takes a token, sixteen of its heads and a chunk of the keys that it sees, in groups of 32. The sixteen heads are the
 // sixteen columns of v_mfma_f32_16x16x32_bf16: S^T[key][head] = K Q^T with a tile of the cache (16 keys x 32 dims, in the
 // order of the A operand: one load instruction takes a contiguous kilobyte) as A and the heads' queries, kept in registers,
 // as B; after the two tiles of a group of 32 keys a lane holds the scores of eight consecutive keys of one head, which is the
@@ -11,6 +13,14 @@
 // The softmax's weights are float32 and enter that product as two bfloat16 numbers each, the rounded weight and what the
 // rounding left. Every chunk is worked off from empty hands; a second kernel merges a token's chunks in their order, adds the
 // head's sink to the denominator (a learnt score without a value, or none) and writes the result.
+//
+// Steps that bring sequences many tokens (xrt_attention_latent_prompts). All heads of all tokens read the same keys, so the
+// (token, head) pairs of a sequence are simply rows, one after another, and a wavefront takes sixteen of them as the columns of
+// its products: with many heads its rows are one token's or a few tokens', with few heads many tokens'. A workgroup of eight
+// wavefronts (128 rows) walks the groups of 32 keys that some row of it sees; a group's tiles of keys and values (a contiguous
+// stretch each) travel straight into LDS while the group before it is multiplied. The softmax keeps its exponent until a score
+// exceeds it by 8 (in log2), so that the sums are rarely rescaled. (Two sets of sixteen columns a wavefront, which would read every
+// tile from LDS half as often, need more registers than there are: the compiler keeps the sums twice around the rescaling.)
 #include "cache_layout.h"
 #include "xrt_hip.h"
 
@@ -19,11 +29,15 @@ namespace {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float floatx4 __attribute__((ext_vector_type(4)));
 
-constexpr int LATENT_MOST = 512;                 // largest key and value size
-constexpr int KEY_STEPS = LATENT_MOST / 32;      // steps of 32 dims of a score product
+constexpr int KEYS_MOST = 640, LATENT_MOST = 512;       // largest key and value size
+constexpr int KEY_STEPS = KEYS_MOST / 32;        // steps of 32 dims of a score product
 constexpr int VALUE_TILES = LATENT_MOST / 16;    // tiles of 16 dims of the value product
 constexpr int HEADS_A_WAVE = 16;
-constexpr int MOST_CHUNKS = 32;                  // chunks of blocks a sequence is cut into at most
+constexpr int GROUP = 32;                        // keys that are multiplied together (half a cache block)
+constexpr int MOST_CHUNKS = XRT_WAVE;            // chunks of groups that a query's keys are cut into at most (a lane each in the merge)
+
+// the first group of keys that the query at `pos` sees, and the first key
+__device__ __forceinline__ int first_key_of(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
 
 // floats a (token, head group, chunk) leaves for the merge: for each of 16 heads the weighted values, the largest score, the sum
 __host__ __device__ inline int head_floats(int value_dim) { return value_dim + 4; }     // (a multiple of four: a lane stores four at a time)
@@ -32,15 +46,16 @@ __host__ __device__ inline long partial_floats(int value_dim) { return (long)HEA
 __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __restrict__ q, long q_stride, int n_heads, int head_dim, int value_dim,
                                                                 const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache,
                                                                 const int* __restrict__ block_table, int table_stride, int n_blocks,
-                                                                const int* __restrict__ positions, const int* __restrict__ slots, float scale,
-                                                                int chunk_blocks, int chunks, float* __restrict__ partial) {
+                                                                const int* __restrict__ positions, const int* __restrict__ slots, float scale, int window,
+                                                                int chunk_groups, int chunks, float* __restrict__ partial) {
     const int lane = threadIdx.x, column = lane % 16, quarter = lane / 16;
     const int chunk = blockIdx.x, groups = gridDim.z, group = blockIdx.z;
     const long token = blockIdx.y;
     const int slot = slots[token], pos = positions[token];
     if (slot < 0) return;                                      // (the merge writes zeros)
-    const int first_block = chunk * chunk_blocks, last_block = min(pos / XRT_BLOCK_TOKENS, first_block + chunk_blocks - 1);
-    if (first_block > last_block) return;                      // (the merge knows from the position which chunks exist)
+    const int first_key = first_key_of(pos, window);
+    const int first_group = first_key / GROUP + chunk * chunk_groups, last_group = min(pos / GROUP, first_group + chunk_groups - 1);
+    if (first_group > last_group) return;                      // (the merge knows from the position which chunks exist)
     const int head = group * HEADS_A_WAVE + column;
     const int key_steps = head_dim / 32, value_tiles = value_dim / 16;
 
@@ -59,74 +74,71 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __r
     float top = -INFINITY, sum = 0.f;                          // of this lane's head: top is shared by the head's four lanes, sum is this lane's share
 
     const int* table = block_table + (long)slot * table_stride;
-    for (int b = first_block; b <= last_block; ++b) {
-        const int block = min(max(table[b], 0), n_blocks - 1); // the host never hands out anything else
+    for (int g = first_group; g <= last_group; ++g) {
+        const int k0 = g * GROUP, half = g % 2;                // the first or second half of the cache block g / 2
+        const int block = min(max(table[g / 2], 0), n_blocks - 1);     // the host never hands out anything else
         const bf16* keys = k_cache + (long)block * XRT_BLOCK_TOKENS * head_dim;
         const bf16* values = v_cache + (long)block * XRT_BLOCK_TOKENS * value_dim;
-        for (int g = 0; g < 2; ++g) {                          // the block's two groups of 32 keys
-            const int k0 = b * XRT_BLOCK_TOKENS + g * 32;
-            if (k0 > pos) break;
-            // The tiles are asked for four steps at a time, both tiles of a step, before the products that use them (a branch
-            // per step would have every load awaited alone); steps beyond the key's size read the last tile again and multiply
-            // it with queries that are zeros.
-            floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
+        // The tiles are asked for four steps at a time, both tiles of a step, before the products that use them (a branch
+        // per step would have every load awaited alone); steps beyond the key's size read the last tile again and multiply
+        // it with queries that are zeros.
+        floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-            for (int step0 = 0; step0 < KEY_STEPS; step0 += 4) {
-                if (step0 < key_steps) {
-                    bf16x8 tiles[2][4];
+        for (int step0 = 0; step0 < KEY_STEPS; step0 += 4) {
+            if (step0 < key_steps) {
+                bf16x8 tiles[2][4];
 #pragma unroll
-                    for (int t = 0; t < 2; ++t)
-#pragma unroll
-                        for (int i = 0; i < 4; ++i)
-                            tiles[t][i] = *reinterpret_cast<const bf16x8*>(keys + ((long)((g * 2 + t) * key_steps + min(step0 + i, key_steps - 1)) * XRT_WAVE + lane) * 8);
+                for (int t = 0; t < 2; ++t)
 #pragma unroll
                     for (int i = 0; i < 4; ++i)
+                        tiles[t][i] = *reinterpret_cast<const bf16x8*>(keys + ((long)((half * 2 + t) * key_steps + min(step0 + i, key_steps - 1)) * XRT_WAVE + lane) * 8);
 #pragma unroll
-                        for (int t = 0; t < 2; ++t) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[t][i], queries[step0 + i], s[t], 0, 0, 0);
-                }
+                for (int i = 0; i < 4; ++i)
+#pragma unroll
+                    for (int t = 0; t < 2; ++t) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[t][i], queries[step0 + i], s[t], 0, 0, 0);
             }
-            // register i of tile t is the key k0 + 8 quarter + 4 t + i, for this lane's head
-            float scores[8];
-            float here = -INFINITY;
+        }
+        // register i of tile t is the key k0 + 8 quarter + 4 t + i, for this lane's head
+        float scores[8];
+        float here = -INFINITY;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                scores[e] = k0 + quarter * 8 + e <= pos ? s[e / 4][e % 4] * scale : -INFINITY;
-                here = fmaxf(here, scores[e]);
-            }
-            here = fmaxf(here, __shfl_xor(here, 16, XRT_WAVE));
-            here = fmaxf(here, __shfl_xor(here, 32, XRT_WAVE));
-            const float top_new = fmaxf(top, here);            // (finite: the group's first key is at or before the query)
-            const float correction = expf(top - top_new);      // 0 for empty hands
-            top = top_new;
-            sum *= correction;
-            bf16x8 rounded, rest;
+        for (int e = 0; e < 8; ++e) {
+            scores[e] = k0 + quarter * 8 + e <= pos && k0 + quarter * 8 + e >= first_key ? s[e / 4][e % 4] * scale : -INFINITY;
+            here = fmaxf(here, scores[e]);
+        }
+        here = fmaxf(here, __shfl_xor(here, 16, XRT_WAVE));
+        here = fmaxf(here, __shfl_xor(here, 32, XRT_WAVE));
+        const float top_new = fmaxf(top, here);            // (finite: every group of the chunk has a key that the query sees)
+        const float correction = expf(top - top_new);      // 0 for empty hands
+        top = top_new;
+        sum *= correction;
+        bf16x8 rounded, rest;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const float weight = expf(scores[e] - top);     // 0 for a key behind the query
-                sum += weight;
-                rounded[e] = (bf16)weight;
-                rest[e] = (bf16)(weight - (float)rounded[e]);
-            }
-            const bool edge = k0 + 31 > pos;                    // what lies behind the sequence's last key is not ours: kept away from the zeros
+        for (int e = 0; e < 8; ++e) {
+            const float weight = expf(scores[e] - top);     // 0 for a key that is not seen
+            sum += weight;
+            rounded[e] = (bf16)weight;
+            rest[e] = (bf16)(weight - (float)rounded[e]);
+        }
+        const bool edge = k0 + 31 > pos;                    // what lies behind the sequence's last key is not ours: kept away from the zeros
 #pragma unroll
-            for (int u0 = 0; u0 < VALUE_TILES; u0 += 4) {
-                if (u0 < value_tiles) {                        // (tiles beyond the value's size read the last one again into sums that nobody reads)
-                    bf16x8 tiles[4];
+        for (int u0 = 0; u0 < VALUE_TILES; u0 += 4) {
+            if (u0 < value_tiles) {                        // (tiles beyond the value's size read the last one again into sums that nobody reads)
+                bf16x8 tiles[4];
 #pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        tiles[i] = *reinterpret_cast<const bf16x8*>(values + ((long)(g * value_tiles + min(u0 + i, value_tiles - 1)) * XRT_WAVE + lane) * 8);
+                for (int i = 0; i < 4; ++i)
+                    tiles[i] = *reinterpret_cast<const bf16x8*>(values + ((long)(half * value_tiles + min(u0 + i, value_tiles - 1)) * XRT_WAVE + lane) * 8);
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) {
-                        if (edge) {
+                for (int i = 0; i < 4; ++i) {
+                    if (edge) {
 #pragma unroll
-                            for (int e = 0; e < 8; ++e)
-                                if (k0 + quarter * 8 + e > pos) tiles[i][e] = (bf16)0.f;
-                        }
-#pragma unroll
-                        for (int j = 0; j < 4; ++j) o[u0 + i][j] *= correction;
-                        o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[i], rounded, o[u0 + i], 0, 0, 0);
-                        o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[i], rest, o[u0 + i], 0, 0, 0);
+                        for (int e = 0; e < 8; ++e)
+                            if (k0 + quarter * 8 + e > pos) tiles[i][e] = (bf16)0.f;
                     }
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) o[u0 + i][j] *= correction;
+                    o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[i], rounded, o[u0 + i], 0, 0, 0);
+                    o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[i], rest, o[u0 + i], 0, 0, 0);
                 }
             }
         }
@@ -146,8 +158,8 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __r
 }
 
 // A workgroup a (token, head): the chunks' parts in their order, the sink, the quotient.
-__global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __restrict__ partial, int n_heads, int value_dim, int chunk_blocks, int chunks,
-                                                               const int* __restrict__ positions, const int* __restrict__ slots,
+__global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __restrict__ partial, int n_heads, int value_dim, int window,
+                                                               int chunk_groups, int chunks, const int* __restrict__ positions, const int* __restrict__ slots,
                                                                const float* __restrict__ sinks, bf16* __restrict__ out) {
     const long token = blockIdx.x;
     const int head = blockIdx.y, lane = threadIdx.x, groups = (n_heads + HEADS_A_WAVE - 1) / HEADS_A_WAVE;
@@ -156,7 +168,8 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __r
         for (int d = lane; d < value_dim; d += XRT_WAVE) dst[d] = (bf16)0.f;
         return;
     }
-    const int mine = positions[token] / XRT_BLOCK_TOKENS / chunk_blocks + 1;      // this sequence's chunks
+    const int pos = positions[token];
+    const int mine = (pos / GROUP - first_key_of(pos, window) / GROUP) / chunk_groups + 1;      // this query's chunks
     const float* parts = partial + ((token * groups + head / HEADS_A_WAVE) * chunks) * partial_floats(value_dim) + (long)(head % HEADS_A_WAVE) * head_floats(value_dim);
     constexpr int OWNED = LATENT_MOST / XRT_WAVE;
     float acc[OWNED], top = -INFINITY, sum = 0.f;
@@ -201,48 +214,300 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __r
     }
 }
 
-int chunk_blocks_for(int max_context) {
-    const int blocks = (max(max_context, 1) + XRT_BLOCK_TOKENS - 1) / XRT_BLOCK_TOKENS;
-    return (blocks + MOST_CHUNKS - 1) / MOST_CHUNKS;
+// Groups of keys that a query sees at most (a window's keys may begin and end inside a group), and how many of them a chunk has.
+int most_groups(int max_context, int window) {
+    const int all = (max(max_context, 1) + GROUP - 1) / GROUP;
+    return window > 0 ? min(all, (window + GROUP - 2) / GROUP + 1) : all;
+}
+int chunk_groups_for(int max_context, int window) { return (most_groups(max_context, window) + MOST_CHUNKS - 1) / MOST_CHUNKS; }
+int chunks_for(int max_context, int window) {
+    const int groups = chunk_groups_for(max_context, window);
+    return (most_groups(max_context, window) + groups - 1) / groups;
+}
+
+// ---- steps that bring sequences many tokens -------------------------------------------------------------------------------
+
+constexpr int PROMPT_WAVES = 8;
+constexpr int WAVE_ROWS = 16, TILE_ROWS = PROMPT_WAVES * WAVE_ROWS;
+constexpr int AHEAD = 2;                         // pairs of tiles that are read from LDS ahead of their products
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr int TILE_BYTES = 1024;                 // an operand tile of the cache, in the order of the lanes
+
+// KS, VT: the steps of 32 key dims and tiles of 16 value dims that this instantiation multiplies, whatever the sizes leave of them
+template <int KS, int VT>
+__global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel(
+    const bf16* __restrict__ q, int n_heads, int head_dim, int value_dim, const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache,
+    const int* __restrict__ block_table, int table_stride, int n_blocks, const int* __restrict__ seq_offsets, const int* __restrict__ seq_slots,
+    const int* __restrict__ seq_starts, int n_seqs, float scale, int window, const float* __restrict__ sinks, bf16* __restrict__ out) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
+    const int lane = threadIdx.x % XRT_WAVE, column = lane % 16, quarter = lane / 16;
+    const int wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x / XRT_WAVE);
+    const int key_steps = head_dim / 32, value_tiles = value_dim / 16;
+
+    // which sequence, and which of its tiles of rows (the last ones, which see most keys, first)
+    int tile = blockIdx.x, seq = 0, count = 0;
+    bool found = false;
+    for (; seq < n_seqs; ++seq) {
+        count = seq_offsets[seq + 1] - seq_offsets[seq];
+        const int tiles = (int)(((long)count * n_heads + TILE_ROWS - 1) / TILE_ROWS);
+        if (tile < tiles) {
+            tile = tiles - 1 - tile;
+            found = true;
+            break;
+        }
+        tile -= tiles;
+    }
+    if (!found) return;                                        // the whole workgroup leaves
+    const int slot = seq_slots[seq], start = seq_starts[seq];
+    const long first_row = (long)seq_offsets[seq] * n_heads;
+    const int rows = count * n_heads;                          // (below 2^31: checked on the host)
+    if (slot < 0) {                                            // a sequence of padding: zeros, which nobody reads
+        for (int r = tile * TILE_ROWS; r < min(rows, (tile + 1) * TILE_ROWS); ++r)
+            for (int d = threadIdx.x; d < value_dim; d += blockDim.x) out[(first_row + r) * value_dim + d] = (bf16)0.f;
+        return;
+    }
+    // the keys that some row of the workgroup sees
+    const int pos_low = start + tile * TILE_ROWS / n_heads, pos_high = start + (min(rows, (tile + 1) * TILE_ROWS) - 1) / n_heads;
+    const int group_low = first_key_of(pos_low, window) / GROUP, group_high = pos_high / GROUP;
+
+    // this wavefront's rows, a column each
+    const int wave_row = tile * TILE_ROWS + wave * WAVE_ROWS;
+    const bool awake = wave_row < rows;
+    const int wave_low = start + min(wave_row, rows - 1) / n_heads, wave_high = start + min(wave_row + WAVE_ROWS - 1, rows - 1) / n_heads;
+    const int wave_all = first_key_of(wave_high, window);      // the first key that all rows of the wavefront see
+    const int row = wave_row + column, clamped = min(row, rows - 1);
+    const int pos = start + clamped / n_heads, head = clamped % n_heads;
+    const bf16* of_row = q + (first_row + clamped) * head_dim + quarter * 8;
+    bf16x8 queries[KS];
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) queries[s][e] = (bf16)0.f;
+        if (s < key_steps) queries[s] = *reinterpret_cast<const bf16x8*>(of_row + s * 32);
+    }
+    // (awaited here: left to their first use the wait would stand inside the loop and hold up the tiles on their way to LDS)
+#pragma unroll
+    for (int s = 0; s < KS; ++s) asm volatile("" : "+v"(queries[s]));
+    floatx4 o[VT];
+#pragma unroll
+    for (int u = 0; u < VT; ++u) o[u] = floatx4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;                              // m is shared by the row's four lanes, l is this lane's share
+
+    const float scale2 = scale * LOG2E;
+    // A buffer has a place for every tile that this instantiation may have: keys' first tiles, their second ones, values. (The places
+    // are the same whatever the sizes, so that the reads have their offsets in the instructions.)
+    constexpr int PLACES = 2 * KS + VT;
+    const int key_tiles = 2 * key_steps, tiles_a_group = key_tiles + value_tiles;
+    const unsigned lds0 = lds_address(lds_raw);
+    constexpr unsigned buffer_bytes = (unsigned)PLACES * TILE_BYTES;
+    const int* table = block_table + (long)slot * table_stride;
+    // a group's tiles into buffer `buffer`: keys, then values, dealt to the wavefronts in turn
+    auto fetch = [&](int g, int buffer) {
+        const int block = __builtin_amdgcn_readfirstlane(min(max(table[g / 2], 0), n_blocks - 1));       // the host never hands out anything else
+        const char* keys = reinterpret_cast<const char*>(k_cache + (long)block * XRT_BLOCK_TOKENS * head_dim) + (long)(g % 2) * key_tiles * TILE_BYTES;
+        const char* values = reinterpret_cast<const char*>(v_cache + (long)block * XRT_BLOCK_TOKENS * value_dim) + (long)(g % 2) * value_tiles * TILE_BYTES;
+        for (int t = wave; t < tiles_a_group; t += PROMPT_WAVES) {
+            const bool is_key = t < key_tiles;
+            const int place = !is_key ? 2 * KS + t - key_tiles : t < key_steps ? t : KS + t - key_steps;
+            load_to_lds(is_key ? keys : values, (unsigned)((is_key ? t : t - key_tiles) * TILE_BYTES + lane * 16),
+                        lds0 + (unsigned)buffer * buffer_bytes + (unsigned)place * TILE_BYTES);
+        }
+    };
+
+    // places that the sizes at hand leave empty hold zeros (the code multiplies them all, without a branch)
+    for (int t = wave; t < 2 * PLACES; t += PROMPT_WAVES) {
+        const int place = t % PLACES;
+        if (place < 2 * KS ? place % KS >= key_steps : place - 2 * KS >= value_tiles)
+            *reinterpret_cast<uint4*>(lds_raw + (size_t)t * TILE_BYTES + lane * 16) = make_uint4(0u, 0u, 0u, 0u);
+    }
+    fetch(group_low, 0);
+    wait_loads_and_barrier<0>();
+    for (int g = group_low; g <= group_high; ++g) {
+        const int buffer = (g - group_low) & 1;
+        if (g < group_high) fetch(g + 1, buffer ^ 1);      // (read for the last time ahead of the last barrier)
+        const int k0 = g * GROUP;
+        const unsigned char* tiles = lds_raw + (size_t)buffer * buffer_bytes + lane * 16;
+        auto tile_at = [&](int t) { return *reinterpret_cast<const bf16x8*>(tiles + (size_t)t * TILE_BYTES); };
+        floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
+        // A tile is read AHEAD steps before it is multiplied. (The fences between the steps keep the compiler from reading
+        // all of them at once.)
+        bf16x8 ahead[AHEAD][2];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) { ahead[i][0] = tile_at(i); ahead[i][1] = tile_at(KS + i); }
+#pragma unroll
+        for (int step = 0; step < KS; ++step) {
+            __builtin_amdgcn_sched_barrier(0);
+            const bf16x8 first = ahead[step % AHEAD][0], second = ahead[step % AHEAD][1];
+            if (step + AHEAD < KS) { ahead[step % AHEAD][0] = tile_at(step + AHEAD); ahead[step % AHEAD][1] = tile_at(KS + step + AHEAD); }
+            s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(first, queries[step], s[0], 0, 0, 0);
+            s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(second, queries[step], s[1], 0, 0, 0);
+        }
+        // the first values are on their way while the softmax is done
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) { ahead[i][0] = tile_at(2 * KS + 2 * i); ahead[i][1] = tile_at(2 * KS + 2 * i + 1); }
+        __builtin_amdgcn_sched_barrier(0);
+        // register i of tile t is the key k0 + 8 quarter + 4 t + i, for the row of this lane's column
+        const bool masked = k0 + GROUP - 1 > wave_low || k0 < wave_all;
+        if (masked) {
+            const int first = first_key_of(pos, window);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const int key = k0 + quarter * 8 + e;
+                if (key > pos || key < first) s[e / 4][e % 4] = -INFINITY;
+            }
+        }
+        float top = s[0][0];
+#pragma unroll
+        for (int e = 1; e < 8; ++e) top = fmaxf(top, s[e / 4][e % 4]);
+        top *= scale2;                                         // (the scale is positive: checked on the host)
+        // m is the exponent that the sums are relative to; it moves only when some row meets a score more than 8 above it (in
+        // log2), until when the weights stay below 2^8 and the quotient in the end is the same.
+        if (__builtin_amdgcn_ballot_w64(top > m + 8.0f) != 0) {
+            float here = fmaxf(top, __shfl_xor(top, 16, XRT_WAVE));
+            here = fmaxf(here, __shfl_xor(here, 32, XRT_WAVE));
+            const float m_new = fmaxf(m, here);
+            const float correction = __builtin_amdgcn_exp2f(m - (m_new == -INFINITY ? 0.f : m_new));
+            m = m_new;
+            l *= correction;
+#pragma unroll
+            for (int u = 0; u < VT; ++u)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) o[u][j] *= correction;
+        }
+        bf16x8 rounded, rest;
+        const float m_safe = m == -INFINITY ? 0.f : m;       // a row that has seen no key yet
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const float weight = __builtin_amdgcn_exp2f(fmaf(s[e / 4][e % 4], scale2, -m_safe));
+            l += weight;
+            rounded[e] = (bf16)weight;
+            rest[e] = (bf16)(weight - (float)rounded[e]);
+        }
+        const bool edge = k0 + GROUP - 1 > pos_high;       // what lies behind the last key may be anything: kept away from the weights' zeros
+#pragma unroll
+        for (int u0 = 0; u0 < VT; u0 += 2) {
+            __builtin_amdgcn_sched_barrier(0);
+            bf16x8 value[2] = {ahead[u0 / 2 % AHEAD][0], ahead[u0 / 2 % AHEAD][1]};
+            if (u0 + 2 * AHEAD < VT) {
+                ahead[u0 / 2 % AHEAD][0] = tile_at(2 * KS + u0 + 2 * AHEAD);
+                ahead[u0 / 2 % AHEAD][1] = tile_at(2 * KS + u0 + 2 * AHEAD + 1);
+            }
+            if (edge) {
+#pragma unroll
+                for (int i = 0; i < 2; ++i)
+#pragma unroll
+                    for (int e = 0; e < 8; ++e)
+                        if (k0 + quarter * 8 + e > pos_high) value[i][e] = (bf16)0.f;
+            }
+#pragma unroll
+            for (int i = 0; i < 2; ++i)
+                o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rounded, o[u0 + i], 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < 2; ++i)
+                o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rest, o[u0 + i], 0, 0, 0);
+        }
+        wait_loads_and_barrier<0>();                       // the next group has arrived from every wavefront, this one has been read by all
+    }
+    if (!awake) return;
+    float sum = l;
+    sum += __shfl_xor(sum, 16, XRT_WAVE);
+    sum += __shfl_xor(sum, 32, XRT_WAVE);
+    if (sinks != nullptr) sum += __builtin_amdgcn_exp2f(fmaf(sinks[head], LOG2E, -(m == -INFINITY ? 0.f : m)));    // (relative to the same exponent)
+    const float inv = sum > 0.f ? 1.0f / sum : 0.f;
+    if (row < rows) {
+        // register i of tile u is dim 16 u + 4 quarter + i of this lane's row
+        bf16* dst = out + (first_row + row) * value_dim + quarter * 4;
+#pragma unroll
+        for (int u = 0; u < VT; ++u) {
+            if (u < value_tiles) {
+                struct alignas(8) Four { bf16 e[4]; } four;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(o[u][i] * inv);
+                *reinterpret_cast<Four*>(dst + u * 16) = four;
+            }
+        }
+    }
+}
+
+template <int KS, int VT>
+int launch_prompts(const bf16* q, long tokens, int n_heads, int head_dim, int value_dim, const bf16* k_cache, const bf16* v_cache, const int* block_table,
+                   int table_stride, int n_blocks, const int* seq_offsets, const int* seq_slots, const int* seq_starts, int n_seqs, float scale,
+                   int window, const float* sinks, bf16* out, hipStream_t s) {
+    const long tiles = tokens * n_heads / TILE_ROWS + n_seqs;  // every sequence's last tile may be partly filled
+    XRT_REQUIRE(tiles < (1L << 31), "attention (latent, prompts): too many rows");
+    constexpr size_t lds = (size_t)2 * (2 * KS + VT) * TILE_BYTES;
+    static bool configured = false;                            // per instantiation
+    if (!configured) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_prompts_kernel<KS, VT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        XRT_REQUIRE(e == hipSuccess, "attention (latent, prompts): cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(e));
+        configured = true;
+    }
+    latent_prompts_kernel<KS, VT><<<(unsigned)tiles, PROMPT_WAVES * XRT_WAVE, lds, s>>>(q, n_heads, head_dim, value_dim, k_cache, v_cache, block_table, table_stride,
+                                                                                       n_blocks, seq_offsets, seq_slots, seq_starts, n_seqs, scale, window,
+                                                                                       sinks, out);
+    XRT_LAUNCH_CHECK("attention (latent, prompts)");
+    return 0;
 }
 
 }  // namespace
 
 extern "C" int xrt_attention_latent_accepts(int dtype, int n_kv_heads, int head_dim, int value_dim) {
     return dtype == XRT_BF16 && n_kv_heads == 1 && head_dim % 32 == 0 && value_dim % 32 == 0 && head_dim > 0 && value_dim > 0 &&
-           head_dim <= LATENT_MOST && value_dim <= LATENT_MOST;
+           head_dim <= KEYS_MOST && value_dim <= LATENT_MOST;
 }
 
-extern "C" long xrt_attention_latent_workspace(long tokens, int n_heads, int value_dim, int max_context) {
-    const int chunk_blocks = chunk_blocks_for(max_context);
-    const int chunks = ((max(max_context, 1) + XRT_BLOCK_TOKENS - 1) / XRT_BLOCK_TOKENS + chunk_blocks - 1) / chunk_blocks;
-    return tokens * ((n_heads + HEADS_A_WAVE - 1) / HEADS_A_WAVE) * chunks * partial_floats(value_dim);
+extern "C" long xrt_attention_latent_workspace(long tokens, int n_heads, int value_dim, int max_context, int window) {
+    return tokens * ((n_heads + HEADS_A_WAVE - 1) / HEADS_A_WAVE) * chunks_for(max_context, window) * partial_floats(value_dim);
 }
 
 extern "C" int xrt_attention_latent(const void* q, long q_stride, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
                                     const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* positions,
-                                    const int* slots, void* out, float scale, const float* sink_scores, int max_context, float* workspace,
-                                    long workspace_floats, void* stream) {
-    XRT_REQUIRE(xrt_attention_latent_accepts(XRT_BF16, 1, head_dim, value_dim), "attention (latent): key and value sizes %d and %d: multiples of 32 up to %d",
-                head_dim, value_dim, LATENT_MOST);
+                                    const int* slots, void* out, float scale, int window, const float* sink_scores, int max_context,
+                                    float* workspace, long workspace_floats, void* stream) {
+    XRT_REQUIRE(xrt_attention_latent_accepts(XRT_BF16, 1, head_dim, value_dim), "attention (latent): key and value sizes %d and %d: multiples of 32 up to %d and %d",
+                head_dim, value_dim, KEYS_MOST, LATENT_MOST);
     XRT_REQUIRE(q && k_cache && v_cache && block_table && positions && slots && out, "attention (latent): null operand");
-    XRT_REQUIRE(tokens >= 0 && tokens <= 65535 && n_heads > 0 && n_heads <= 65535 * HEADS_A_WAVE && table_stride > 0 && n_blocks > 0 && max_context > 0,
+    XRT_REQUIRE(tokens >= 0 && tokens <= 65535 && n_heads > 0 && n_heads <= 65535 * HEADS_A_WAVE && table_stride > 0 && n_blocks > 0 && max_context > 0 && window >= 0,
                 "attention (latent): bad sizes (%ld tokens, %d heads)", tokens, n_heads);
     XRT_REQUIRE(q_stride >= (long)n_heads * head_dim && q_stride % 8 == 0 && (uintptr_t)q % 16 == 0 && (uintptr_t)k_cache % 16 == 0 && (uintptr_t)v_cache % 16 == 0,
                 "attention (latent): rows of q %ld apart, or operands off their sixteen bytes", q_stride);
     XRT_REQUIRE(max_context <= table_stride * XRT_BLOCK_TOKENS, "attention (latent): a sequence of %d tokens exceeds the block table", max_context);
     if (tokens == 0) return 0;
-    const int chunk_blocks = chunk_blocks_for(max_context);
-    const int chunks = ((max_context + XRT_BLOCK_TOKENS - 1) / XRT_BLOCK_TOKENS + chunk_blocks - 1) / chunk_blocks;
+    const int chunk_groups = chunk_groups_for(max_context, window), chunks = chunks_for(max_context, window);
     const int groups = (n_heads + HEADS_A_WAVE - 1) / HEADS_A_WAVE;
     XRT_REQUIRE(workspace != nullptr && workspace_floats >= tokens * groups * chunks * partial_floats(value_dim) && (uintptr_t)workspace % 16 == 0,
                 "attention (latent): the workspace needs %ld floats", tokens * groups * chunks * partial_floats(value_dim));
     latent_chunks_kernel<<<dim3(chunks, (unsigned)tokens, groups), XRT_WAVE, 0, (hipStream_t)stream>>>(
         (const bf16*)q, q_stride, n_heads, head_dim, value_dim, (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, n_blocks,
-        positions, slots, scale, chunk_blocks, chunks, workspace);
+        positions, slots, scale, window, chunk_groups, chunks, workspace);
     XRT_LAUNCH_CHECK("attention (latent, chunks)");
-    latent_merge_kernel<<<dim3((unsigned)tokens, n_heads), XRT_WAVE, 0, (hipStream_t)stream>>>(workspace, n_heads, value_dim, chunk_blocks, chunks, positions,
-                                                                                              slots, sink_scores, (bf16*)out);
+    latent_merge_kernel<<<dim3((unsigned)tokens, n_heads), XRT_WAVE, 0, (hipStream_t)stream>>>(workspace, n_heads, value_dim, window, chunk_groups, chunks,
+                                                                                              positions, slots, sink_scores, (bf16*)out);
     XRT_LAUNCH_CHECK("attention (latent, merge)");
     return 0;
+}
+
+extern "C" int xrt_attention_latent_prompts(const void* q, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
+                                            const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* seq_offsets,
+                                            const int* seq_slots, const int* seq_starts, int n_seqs, void* out, float scale, int window,
+                                            const float* sink_scores, int max_context, void* stream) {
+    XRT_REQUIRE(xrt_attention_latent_accepts(XRT_BF16, 1, head_dim, value_dim), "attention (latent): key and value sizes %d and %d: multiples of 32 up to %d and %d",
+                head_dim, value_dim, KEYS_MOST, LATENT_MOST);
+    XRT_REQUIRE(q && k_cache && v_cache && block_table && seq_offsets && seq_slots && seq_starts && out, "attention (latent, prompts): null operand");
+    XRT_REQUIRE(tokens >= 0 && n_heads > 0 && tokens * n_heads < (1L << 31) - TILE_ROWS && n_seqs > 0 && n_seqs <= tokens && table_stride > 0 && n_blocks > 0 &&
+                window >= 0 && scale > 0.f, "attention (latent, prompts): bad sizes (%ld tokens, %d heads, %d sequences)", tokens, n_heads, n_seqs);
+    XRT_REQUIRE(((uintptr_t)q | (uintptr_t)k_cache | (uintptr_t)v_cache) % 16 == 0 && (uintptr_t)out % 8 == 0, "attention (latent, prompts): operands off their sixteen bytes");
+    XRT_REQUIRE(max_context > 0 && max_context <= table_stride * XRT_BLOCK_TOKENS, "attention (latent, prompts): a sequence of %d tokens exceeds the block table", max_context);
+    if (tokens == 0) return 0;
+    auto run = [&](auto launcher) {
+        return launcher((const bf16*)q, tokens, n_heads, head_dim, value_dim, (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, n_blocks,
+                        seq_offsets, seq_slots, seq_starts, n_seqs, scale, window, sink_scores, (bf16*)out, (hipStream_t)stream);
+    };
+    // the instantiation that holds the sizes with the least to spare
+    if (head_dim <= 192 && value_dim <= 128) return run(launch_prompts<6, 8>);
+    if (head_dim <= 256 && value_dim <= 192) return run(launch_prompts<8, 12>);
+    if (head_dim <= 320 && value_dim <= 256) return run(launch_prompts<10, 16>);
+    if (head_dim <= 448 && value_dim <= 384) return run(launch_prompts<14, 24>);
+    if (head_dim <= 576) return run(launch_prompts<18, 32>);
+    return run(launch_prompts<20, 32>);
 }

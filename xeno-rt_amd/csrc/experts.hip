@@ -3,15 +3,23 @@
 //                       (softmax != 0); the chosen weights are multiplied by `scale` in the end; the experts stand in `groups`
 //                       equal groups of neighbours, a group's score is the sum of its `group_top` largest scores, only experts
 //                       of the `keep` best groups can be chosen; the `top` largest scores among those are chosen, and their
-//                       weights are their scores divided by the scores' sum (+ floor). Equal scores: the lower index wins.
+//                       weights are their scores divided by the scores' sum (+ floor), or the scores as they are (normalized == 0).
+//                       Equal scores: the lower index wins.
 //                       Out: weights [tokens][experts] (float32, zero for experts not chosen), and, if asked for, the chosen
 //                       experts [tokens][top] (int32) in the order of their scores.
+//   xrt_glu_experts     from the float32 gate and up sums of a token with all experts (and with a shared expert beside them) the
+//                       rows that the down product reads: silu(gate) * up times the token's weight for the expert, or, where the
+//                       weight multiplies what the expert reads, silu(weight * gate) * (weight * up); the shared expert's times
+//                       the sigmoid of the token's number for it
 //   xrt_scale_blocks    act[t][e * width + c] *= weights[t][e]: every expert's stretch of a row times the token's weight for it
 //   xrt_experts_sort    the picks (token, chosen expert) in the order of their experts, every expert's stretch filled up to whole
 //                       tiles of rows, for products in which each expert multiplies only the tokens that chose it
 //   xrt_linear_groups   such a product: every tile of rows with the matrix of its tile's expert (csrc/gemm_mfma.hip)
-//   xrt_gather_rows, xrt_experts_combine   the tokens' rows into that order, and the experts' outputs back, weighted and summed
-// One thread a token for the choice: the experts of a token are few (up to XRT_MOST_EXPERTS).
+//   xrt_gather_rows, xrt_experts_combine   the tokens' rows into that order (times the picks' weights, where those multiply what
+//                       the experts read), and the experts' outputs back, weighted and summed, onto the shared expert's if there is one
+// The choice: one thread a token (the experts of a token are few, up to XRT_MOST_EXPERTS), or, for sigmoid scores without groups, one
+// wavefront a token.
+#include <climits>
 #include "common.h"
 #include "packing.h"
 #include "xrt_hip.h"
@@ -31,9 +39,9 @@ __device__ __forceinline__ void store_from_float(void* p, int dtype, long i, flo
     if (dtype == XRT_F32) ((float*)p)[i] = v; else ((bf16*)p)[i] = from_float<bf16>(v);
 }
 
-__global__ void __launch_bounds__(64) route_experts_kernel(const float* __restrict__ logits, long tokens, int experts, int top, int groups, int keep,
-                                                           int group_top, float floor_, float* __restrict__ weights, int* __restrict__ chosen,
-                                                           int softmax, float scale) {
+__global__ void __launch_bounds__(64) route_experts_kernel(const float* __restrict__ logits, long logits_stride, long tokens, int experts, int top,
+                                                           int groups, int keep, int group_top, float floor_, float* __restrict__ weights,
+                                                           int* __restrict__ chosen, int softmax, float scale, int normalized) {
     const long t = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (t >= tokens) return;
     float s[XRT_MOST_EXPERTS];
@@ -41,11 +49,11 @@ __global__ void __launch_bounds__(64) route_experts_kernel(const float* __restri
     const int per_group = experts / groups;
     float top_logit = -INFINITY, total = 0.f;
     if (softmax) {
-        for (int e = 0; e < experts; ++e) top_logit = fmaxf(top_logit, logits[t * experts + e]);
-        for (int e = 0; e < experts; ++e) total += expf(logits[t * experts + e] - top_logit);
+        for (int e = 0; e < experts; ++e) top_logit = fmaxf(top_logit, logits[t * logits_stride + e]);
+        for (int e = 0; e < experts; ++e) total += expf(logits[t * logits_stride + e] - top_logit);
     }
     for (int e = 0; e < experts; ++e) {
-        s[e] = softmax ? expf(logits[t * experts + e] - top_logit) / total : 1.0f / (1.0f + expf(-logits[t * experts + e]));
+        s[e] = softmax ? expf(logits[t * logits_stride + e] - top_logit) / total : 1.0f / (1.0f + expf(-logits[t * logits_stride + e]));
         open[e] = groups > 1 ? 0 : 1;
     }
     if (groups > 1) {
@@ -85,8 +93,114 @@ __global__ void __launch_bounds__(64) route_experts_kernel(const float* __restri
         sum += s[best];
     }
     for (int round = 0; round < top; ++round) {
-        weights[t * experts + picks[round]] = s[picks[round]] / (sum + floor_) * scale;
+        weights[t * experts + picks[round]] = (normalized ? s[picks[round]] / (sum + floor_) : s[picks[round]]) * scale;
         if (chosen != nullptr) chosen[t * top + round] = picks[round];
+    }
+}
+
+// Sigmoid scores, one group: a wavefront a token, four experts a lane (lane, lane + 64, ...). Every round the largest score that is
+// left wins (the lowest index among equals); the same scores and the same sums, in the same order, as a thread alone.
+constexpr int ROUTE_WAVES = 4, ROUTE_OWNED = XRT_MOST_EXPERTS / XRT_WAVE;
+
+__global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_kernel(const float* __restrict__ logits, long logits_stride, long tokens,
+                                                                                   int experts, int top, float floor_, float* __restrict__ weights,
+                                                                                   int* __restrict__ chosen, float scale, int normalized) {
+    const int lane = threadIdx.x % XRT_WAVE;
+    const long t = (long)blockIdx.x * ROUTE_WAVES + threadIdx.x / XRT_WAVE;
+    if (t >= tokens) return;                                   // (the whole wavefront)
+    float s[ROUTE_OWNED];
+    unsigned picked = 0, open = 0;
+#pragma unroll
+    for (int i = 0; i < ROUTE_OWNED; ++i) {
+        const int e = lane + i * XRT_WAVE;
+        s[i] = -1.f;
+        if (e < experts) {
+            s[i] = 1.0f / (1.0f + expf(-logits[t * logits_stride + e]));
+            open |= 1u << i;
+        }
+    }
+    float sum = 0.f;
+    for (int round = 0; round < top; ++round) {
+        float best = -1.f;
+        int index = INT_MAX;                                   // (a lane whose experts are all taken)
+#pragma unroll
+        for (int i = 0; i < ROUTE_OWNED; ++i)
+            if ((open >> i & 1) && (index == INT_MAX || s[i] > best)) { best = s[i]; index = lane + i * XRT_WAVE; }
+#pragma unroll
+        for (int offset = XRT_WAVE / 2; offset > 0; offset >>= 1) {
+            const float other = __shfl_xor(best, offset, XRT_WAVE);
+            const int other_index = __shfl_xor(index, offset, XRT_WAVE);
+            // (a score that is no number loses to any that is; among such the lowest index wins, so the lanes agree either way)
+            const bool theirs_known = other == other, mine_known = best == best;
+            const bool take = other_index != INT_MAX &&
+                              (index == INT_MAX || (theirs_known && !mine_known) || (theirs_known == mine_known && (other > best || (!(best > other) && other_index < index))));
+            if (take) { best = other; index = other_index; }
+        }
+        sum += best;
+#pragma unroll
+        for (int i = 0; i < ROUTE_OWNED; ++i)
+            if (index == lane + i * XRT_WAVE) { open &= ~(1u << i); picked |= 1u << i; }
+        if (lane == 0 && chosen != nullptr) chosen[t * top + round] = index;
+    }
+#pragma unroll
+    for (int i = 0; i < ROUTE_OWNED; ++i) {
+        const int e = lane + i * XRT_WAVE;
+        if (e < experts) weights[t * experts + e] = !(picked >> i & 1) ? 0.f : (normalized ? s[i] / (sum + floor_) : s[i]) * scale;
+    }
+}
+
+// What the sums of a row mean: gate and up of column c < total at c and total + c, or, from a matrix packed for a gated epilogue
+// (`interleaved`), in groups of sixteen, eight gates and then their eight ups.
+__device__ __forceinline__ long gate_at(int c, int interleaved) { return interleaved ? (long)(c / 8) * 16 + c % 8 : c; }
+
+__global__ void __launch_bounds__(256) glu_experts_kernel(const float* __restrict__ sums, void* __restrict__ out, int out_dtype, long tokens, int experts,
+                                                         int width, int shared_width, const float* __restrict__ weights,
+                                                         const float* __restrict__ shared_logits, long shared_stride, int weigh_input,
+                                                         int interleaved, int step) {
+    const int total = experts * width + shared_width;
+    const long t = blockIdx.y;
+    const float* row = sums + t * 2 * total;
+    const int up_after = interleaved ? 8 : total;
+    const int c = ((int)blockIdx.x * blockDim.x + threadIdx.x) * step;
+    if (c >= total) return;
+    float before = 1.f, after = 1.f;                           // what multiplies the expert's input, and its activations
+    if (c < experts * width) {
+        const float w = weights[t * experts + c / width];
+        if (weigh_input) before = w; else after = w;
+        if (w == 0.f) after = 0.f;                             // (not chosen)
+    } else if (shared_logits != nullptr) {
+        after = 1.0f / (1.0f + expf(-shared_logits[t * shared_stride]));
+    }
+    float gate[4], up[4], made[4];
+    const long at = gate_at(c, interleaved);
+    if (after == 0.f) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) gate[e] = up[e] = 0.f;
+    } else if (step == 4) {
+        const float4 g = *reinterpret_cast<const float4*>(row + at), u = *reinterpret_cast<const float4*>(row + at + up_after);
+        gate[0] = g.x; gate[1] = g.y; gate[2] = g.z; gate[3] = g.w;
+        up[0] = u.x; up[1] = u.y; up[2] = u.z; up[3] = u.w;
+    } else {
+        gate[0] = row[at];
+        up[0] = row[at + up_after];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        if (e < step) {
+            const float g = gate[e] * before;
+            made[e] = g / (1.0f + expf(-g)) * (up[e] * before) * after;
+        }
+    }
+    const long to = t * total + c;
+    if (step == 4 && out_dtype == XRT_F32) {
+        *reinterpret_cast<float4*>((float*)out + to) = make_float4(made[0], made[1], made[2], made[3]);
+    } else if (step == 4) {
+        struct alignas(8) Four { bf16 e[4]; } four;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) four.e[e] = from_float<bf16>(made[e]);
+        *reinterpret_cast<Four*>((bf16*)out + to) = four;
+    } else {
+        store_from_float(out, out_dtype, to, made[0]);
     }
 }
 
@@ -158,27 +272,40 @@ __global__ void __launch_bounds__(1024) experts_sort_kernel(const int* __restric
 }
 
 // out[r] = x[rows[r]] (zeros where rows[r] < 0); a workgroup a row, eight columns a thread
+// (weights [tokens][experts], or null: times the row's weight for the expert of its tile, rounded once more)
 __global__ void __launch_bounds__(256) gather_rows_kernel(const bf16* __restrict__ x, long x_stride, const int* __restrict__ rows, int width,
-                                                          bf16* __restrict__ out) {
+                                                          bf16* __restrict__ out, const float* __restrict__ weights, int experts,
+                                                          const int* __restrict__ tile_group, int tile) {
     const long r = blockIdx.x;
     const int from = rows[r];
+    const bool weighed = weights != nullptr && from >= 0;
+    const float w = weighed ? weights[(long)from * experts + tile_group[r / tile]] : 1.f;      // (a row with a token lies in a tile with an expert)
     for (int c = threadIdx.x * 8; c < width; c += blockDim.x * 8) {
         uint4 piece = make_uint4(0u, 0u, 0u, 0u);
         if (from >= 0) piece = *reinterpret_cast<const uint4*>(x + (long)from * x_stride + c);
+        if (weighed) {
+            bf16* values = reinterpret_cast<bf16*>(&piece);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) values[e] = from_float<bf16>(to_float(values[e]) * w);
+        }
         *reinterpret_cast<uint4*>(out + r * width + c) = piece;
     }
 }
 
 // out[t][c] = sum over a token's picks, in their order, of weights[t][expert of the pick] * sorted[row of the pick][c]
-// (sorted: [tiles][parts][tile][width], the parts' sums of a row added in their order first)
+// (sorted: [tiles][parts][tile][width], the parts' sums of a row added in their order first). weigh 0: the outputs as they are. shared
+// (float32 rows that lie like sorted's in tiles and parts of their own, the tokens in their order, or null) joins the sum, times sigmoid(shared_logits[t]) (null: as it is).
 __global__ void __launch_bounds__(256) experts_combine_kernel(const float* __restrict__ sorted, const int* __restrict__ places,
                                                               const int* __restrict__ chosen, const float* __restrict__ weights, int top,
-                                                              int experts, int width, int tile, int parts, float* __restrict__ out) {
+                                                              int experts, int width, int tile, int parts, float* __restrict__ out, int weigh,
+                                                              const float* __restrict__ shared, int shared_tile, int shared_parts,
+                                                              const float* __restrict__ shared_logits, long shared_stride) {
     const long t = blockIdx.x;
+    const float of_shared = shared != nullptr && shared_logits != nullptr ? 1.0f / (1.0f + expf(-shared_logits[t * shared_stride])) : 1.f;
     for (int c = threadIdx.x * 4; c < width; c += blockDim.x * 4) {
         float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
         for (int k = 0; k < top; ++k) {
-            const float w = weights[t * experts + chosen[t * top + k]];
+            const float w = weigh ? weights[t * experts + chosen[t * top + k]] : 1.f;
             const int place = places[t * top + k];
             const float* row = sorted + (((long)(place / tile) * parts) * tile + place % tile) * width + c;
             float4 v = *reinterpret_cast<const float4*>(row);
@@ -188,23 +315,61 @@ __global__ void __launch_bounds__(256) experts_combine_kernel(const float* __res
             }
             sum.x = fmaf(w, v.x, sum.x); sum.y = fmaf(w, v.y, sum.y); sum.z = fmaf(w, v.z, sum.z); sum.w = fmaf(w, v.w, sum.w);
         }
+        if (shared != nullptr) {
+            const float* row = shared + ((t / shared_tile * shared_parts) * shared_tile + t % shared_tile) * width + c;
+            float4 v = *reinterpret_cast<const float4*>(row);
+            for (int part = 1; part < shared_parts; ++part) {
+                const float4 more = *reinterpret_cast<const float4*>(row + (long)part * shared_tile * width);
+                v.x += more.x; v.y += more.y; v.z += more.z; v.w += more.w;
+            }
+            sum.x = fmaf(of_shared, v.x, sum.x); sum.y = fmaf(of_shared, v.y, sum.y); sum.z = fmaf(of_shared, v.z, sum.z); sum.w = fmaf(of_shared, v.w, sum.w);
+        }
         *reinterpret_cast<float4*>(out + t * width + c) = sum;
     }
 }
 
 }  // namespace
 
-extern "C" int xrt_route_experts(const float* logits, long tokens, int experts, int top, int groups, int keep, int group_top, float floor_,
-                                 float* weights, int* chosen, int softmax, float scale, void* stream) {
-    XRT_REQUIRE(logits && weights && tokens >= 0, "route_experts: null operand");
+extern "C" int xrt_route_experts(const float* logits, long logits_stride, long tokens, int experts, int top, int groups, int keep, int group_top,
+                                 float floor_, float* weights, int* chosen, int softmax, float scale, int normalized, void* stream) {
+    XRT_REQUIRE(logits && weights && tokens >= 0 && logits_stride >= experts, "route_experts: null operand, or rows of logits %ld apart", logits_stride);
     XRT_REQUIRE(experts > 0 && experts <= XRT_MOST_EXPERTS && top > 0 && groups > 0 && experts % groups == 0 && keep > 0 && keep <= groups &&
                 group_top > 0 && (groups == 1 || experts / groups <= 128) && top <= keep * (experts / groups),
                 "route_experts: %d experts in %d groups of which %d are kept, %d chosen: up to %d experts in equal groups, and no more "
                 "chosen than the kept groups hold", experts, groups, keep, top, XRT_MOST_EXPERTS);
     if (tokens == 0) return 0;
-    route_experts_kernel<<<(unsigned)((tokens + 63) / 64), 64, 0, (hipStream_t)stream>>>(logits, tokens, experts, top, groups, keep, group_top,
-                                                                                       floor_, weights, chosen, softmax, scale);
+    if (groups == 1 && !softmax) {
+        const long blocks = (tokens + ROUTE_WAVES - 1) / ROUTE_WAVES;
+        XRT_REQUIRE(blocks < (1L << 31), "route_experts: too many tokens");
+        route_experts_wave_kernel<<<(unsigned)blocks, ROUTE_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>(logits, logits_stride, tokens, experts, top, floor_, weights,
+                                                                                                     chosen, scale, normalized);
+        XRT_LAUNCH_CHECK("route_experts");
+        return 0;
+    }
+    route_experts_kernel<<<(unsigned)((tokens + 63) / 64), 64, 0, (hipStream_t)stream>>>(logits, logits_stride, tokens, experts, top, groups, keep, group_top,
+                                                                                       floor_, weights, chosen, softmax, scale, normalized);
     XRT_LAUNCH_CHECK("route_experts");
+    return 0;
+}
+
+extern "C" int xrt_glu_experts(const float* sums, void* out, int out_dtype, long tokens, int experts, int width, int shared_width, const float* weights,
+                               const float* shared_logits, long shared_stride, int weigh_input, int interleaved, void* stream) {
+    XRT_REQUIRE(sums && out && weights && (out_dtype == XRT_F32 || out_dtype == XRT_BF16) && tokens >= 0, "glu_experts: null operand or unknown dtype");
+    XRT_REQUIRE(experts > 0 && width > 0 && shared_width >= 0 && (long)experts * width + shared_width < (1L << 29) && shared_stride >= 0,
+                "glu_experts: bad sizes (%d experts of %d, a shared one of %d)", experts, width, shared_width);
+    XRT_REQUIRE(!interleaved || ((long)experts * width + shared_width) % 8 == 0, "glu_experts: interleaved sums come in eights");
+    XRT_REQUIRE((uintptr_t)sums % 16 == 0 && (uintptr_t)out % 16 == 0, "glu_experts: operands off their sixteen bytes");
+    const int total = experts * width + shared_width;
+    const int step = width % 4 == 0 && shared_width % 4 == 0 ? 4 : 1;      // columns a thread: four where the experts' widths allow it
+    const int threads = total > 256 * step ? 256 : XRT_WAVE;
+    for (long first = 0; first < tokens; first += 65535) {     // (the grid's second dimension)
+        const long count = tokens - first < 65535 ? tokens - first : 65535;
+        glu_experts_kernel<<<dim3((total + threads * step - 1) / (threads * step), (unsigned)count), threads, 0, (hipStream_t)stream>>>(
+            sums + first * 2 * total, out_dtype == XRT_F32 ? (void*)((float*)out + first * total) : (void*)((bf16*)out + first * total), out_dtype, count, experts,
+            width, shared_width, weights + first * experts, shared_logits == nullptr ? nullptr : shared_logits + first * shared_stride, shared_stride,
+            weigh_input, interleaved, step);
+        XRT_LAUNCH_CHECK("glu_experts");
+    }
     return 0;
 }
 
@@ -270,21 +435,28 @@ extern "C" int xrt_linear_groups(const void* a, int lda, const void* w, long w_s
                                   packing ? *packing : none, parts, (hipStream_t)stream);
 }
 
-extern "C" int xrt_gather_rows(const void* x, long x_stride, const int* rows, long count, int width, void* out, void* stream) {
+extern "C" int xrt_gather_rows(const void* x, long x_stride, const int* rows, long count, int width, void* out, const float* weights, int experts,
+                               const int* tile_group, int tile, void* stream) {
+    XRT_REQUIRE(weights == nullptr || (experts > 0 && tile_group != nullptr && tile > 0 && count % tile == 0), "gather_rows: weights without the tiles' experts");
     XRT_REQUIRE(x && rows && out && count > 0 && count < (1L << 31) && width > 0 && width % 8 == 0 && x_stride >= width && x_stride % 8 == 0 &&
                 (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0, "gather_rows: bfloat16 rows of a multiple of eight columns, aligned to 16 bytes");
-    gather_rows_kernel<<<(unsigned)count, 256, 0, (hipStream_t)stream>>>((const bf16*)x, x_stride, rows, width, (bf16*)out);
+    gather_rows_kernel<<<(unsigned)count, 256, 0, (hipStream_t)stream>>>((const bf16*)x, x_stride, rows, width, (bf16*)out, weights,
+                                                                          experts, tile_group, tile);
     XRT_LAUNCH_CHECK("gather_rows");
     return 0;
 }
 
 extern "C" int xrt_experts_combine(const float* sorted, const int* places, const int* chosen, const float* weights, long tokens, int top,
-                                   int experts, int width, int tile, int parts, float* out, void* stream) {
+                                   int experts, int width, int tile, int parts, float* out, int weigh, const float* shared, int shared_tile,
+                                   int shared_parts, const float* shared_logits, long shared_stride, void* stream) {
+    XRT_REQUIRE(shared == nullptr || (shared_tile > 0 && shared_parts >= 1 && shared_parts <= 2), "experts_combine: %d parts of the shared expert's tiles", shared_parts);
+    XRT_REQUIRE((uintptr_t)shared % 16 == 0 && shared_stride >= 0, "experts_combine: the shared expert's rows lie off their sixteen bytes");
     XRT_REQUIRE(parts >= 1 && parts <= 2 && tile > 0, "experts_combine: %d parts of tiles of %d rows", parts, tile);
     XRT_REQUIRE(sorted && places && chosen && weights && out && tokens > 0 && tokens < (1L << 31) && top > 0 && experts > 0 && width > 0 &&
                 width % 4 == 0 && (uintptr_t)sorted % 16 == 0 && (uintptr_t)out % 16 == 0, "experts_combine: bad operands");
     experts_combine_kernel<<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(sorted, places, chosen, weights, top, experts, width,
-                                                                              tile, parts, out);
+                                                                              tile, parts, out, weigh, shared, shared_tile, shared_parts, shared_logits,
+                                                                              shared_stride);
     XRT_LAUNCH_CHECK("experts_combine");
     return 0;
 }

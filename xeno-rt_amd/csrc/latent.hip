@@ -8,8 +8,10 @@
 //                        position * frequencies[i]; both into the cache
 //   xrt_latent_queries   from the queries' float32 sums, head by head [plain | part to turn]: the plain parts to rows of
 //                        their own, the turned parts to the tail of the rows that the attention kernel reads
+//   xrt_latent_prepare   both of them in one launch, for layers whose queries come straight from the layer's input
 //   xrt_linear_heads     out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k], float32 sums (steps of many rows: on the matrix cores in
-//                        bfloat16 with k in whole steps of 32, else in the order of k; steps of few: the lanes of a wavefront along k)
+//                        bfloat16 with k in whole steps of 32, else in the order of k; steps of few: the lanes of a wavefront along k);
+//                        with gates (float32 [t][h], any stride) times sigmoid(gates[t][h]) before it is rounded
 // A prompt that starts a sequence can have its scores as a matrix product of its own rows (all heads' queries of a stretch of
 // tokens against the prompt's cached rows, which the step has at hand): then
 //   xrt_causal_softmax   turns the float32 scores [queries x heads][keys] into the softmax's weights over the keys at or before
@@ -34,15 +36,14 @@ __device__ __forceinline__ float turned(const float* part, int e, int rot_dims, 
     return e % 2 == 0 ? mine * cosine - other * sine : mine * cosine + other * sine;
 }
 
+// What becomes of a token's float32 row [latent | key part], by the whole workgroup.
 template <typename T>
-__global__ void __launch_bounds__(256) latent_complete_kernel(const float* __restrict__ down, long down_stride, int rank, int rot_dim, int rot_dims,
-                                                             const void* __restrict__ gain, int gain_dtype, float eps,
-                                                             const float* __restrict__ frequencies, const int* __restrict__ positions,
-                                                             const int* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache,
-                                                             const int* __restrict__ block_table, int table_stride, int n_blocks,
-                                                             T* __restrict__ rows_out) {
+__device__ __forceinline__ void complete_row(long t, const float* __restrict__ down, long down_stride, int rank, int rot_dim, int rot_dims,
+                                             const void* __restrict__ gain, int gain_dtype, float eps, const float* __restrict__ frequencies,
+                                             const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ k_cache,
+                                             T* __restrict__ v_cache, const int* __restrict__ block_table, int table_stride, int n_blocks,
+                                             T* __restrict__ rows_out) {
     __shared__ float scratch[32];
-    const long t = blockIdx.x;
     const int slot = slots[t], pos = positions[t];
     if (slot < 0) {                                            // (the whole workgroup)
         if (rows_out != nullptr) for (int e = threadIdx.x; e < rank + rot_dim; e += blockDim.x) rows_out[t * (rank + rot_dim) + e] = from_float<T>(0.f);
@@ -72,17 +73,66 @@ __global__ void __launch_bounds__(256) latent_complete_kernel(const float* __res
 }
 
 template <typename T>
+__global__ void __launch_bounds__(256) latent_complete_kernel(const float* __restrict__ down, long down_stride, int rank, int rot_dim, int rot_dims,
+                                                             const void* __restrict__ gain, int gain_dtype, float eps,
+                                                             const float* __restrict__ frequencies, const int* __restrict__ positions,
+                                                             const int* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache,
+                                                             const int* __restrict__ block_table, int table_stride, int n_blocks,
+                                                             T* __restrict__ rows_out) {
+    complete_row(blockIdx.x, down, down_stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies, positions, slots, k_cache, v_cache,
+                 block_table, table_stride, n_blocks, rows_out);
+}
+
+// A head's query of a token, by one wavefront.
+template <typename T>
+__device__ __forceinline__ void query_row(long t, int head, int lane, const float* __restrict__ q, long q_stride, int heads, int dim, int rot_dim,
+                                          int rot_dims, const float* __restrict__ frequencies, const int* __restrict__ positions,
+                                          T* __restrict__ plain, T* __restrict__ full, long full_stride, int rank) {
+    const int pos = positions[t];
+    const float* mine = q + t * q_stride + (long)head * (dim + rot_dim);
+    for (int e = lane; e < dim; e += XRT_WAVE) plain[(t * heads + head) * dim + e] = from_float<T>(mine[e]);
+    T* tail = full + t * full_stride + (long)head * (rank + rot_dim) + rank;
+    for (int e = lane; e < rot_dim; e += XRT_WAVE) tail[e] = from_float<T>(turned(mine + dim, e, rot_dims, frequencies, pos));
+}
+
+template <typename T>
 __global__ void __launch_bounds__(XRT_WAVE) latent_queries_kernel(const float* __restrict__ q, long q_stride, int heads, int dim, int rot_dim,
                                                                  int rot_dims, const float* __restrict__ frequencies,
                                                                  const int* __restrict__ positions, T* __restrict__ plain, T* __restrict__ full,
                                                                  long full_stride, int rank) {
-    const long t = blockIdx.x / heads;
-    const int head = blockIdx.x % heads, pos = positions[t];
-    const float* mine = q + t * q_stride + (long)head * (dim + rot_dim);
-    for (int e = threadIdx.x; e < dim; e += XRT_WAVE) plain[(t * heads + head) * dim + e] = from_float<T>(mine[e]);
-    T* tail = full + t * full_stride + (long)head * (rank + rot_dim) + rank;
-    for (int e = threadIdx.x; e < rot_dim; e += XRT_WAVE) tail[e] = from_float<T>(turned(mine + dim, e, rot_dims, frequencies, pos));
+    query_row((long)blockIdx.x / heads, (int)(blockIdx.x % heads), (int)threadIdx.x, q, q_stride, heads, dim, rot_dim, rot_dims, frequencies,
+              positions, plain, full, full_stride, rank);
 }
+
+// Workgroup (token, 0) completes the token's row; workgroup (token, 1 + i) makes the queries of heads PREPARE_HEADS i .. + PREPARE_HEADS - 1.
+constexpr int PREPARE_HEADS = 256 / XRT_WAVE;
+
+template <typename T>
+__global__ void __launch_bounds__(256) latent_prepare_kernel(const float* __restrict__ q, const float* __restrict__ down, long stride, int heads,
+                                                            int dim, int rank, int rot_dim, int rot_dims, const void* __restrict__ gain,
+                                                            int gain_dtype, float eps, const float* __restrict__ frequencies,
+                                                            const int* __restrict__ positions, const int* __restrict__ slots,
+                                                            T* __restrict__ k_cache, T* __restrict__ v_cache, const int* __restrict__ block_table,
+                                                            int table_stride, int n_blocks, T* __restrict__ plain, T* __restrict__ full,
+                                                            long full_stride) {
+    if (blockIdx.y == 0) {
+        complete_row<T>(blockIdx.x, down, stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies, positions, slots, k_cache, v_cache,
+                        block_table, table_stride, n_blocks, nullptr);
+        return;
+    }
+    const int head = ((int)blockIdx.y - 1) * PREPARE_HEADS + (int)threadIdx.x / XRT_WAVE;
+    if (head < heads)
+        query_row((long)blockIdx.x, head, (int)threadIdx.x % XRT_WAVE, q, stride, heads, dim, rot_dim, rot_dims, frequencies, positions, plain, full,
+                  full_stride, rank);
+}
+
+// what a head's output is multiplied by: the sigmoid of its gate, or one
+struct HeadGates {
+    const float* logits; long stride;
+    __device__ __forceinline__ float operator()(long row, int head) const {
+        return logits == nullptr ? 1.0f : 1.0f / (1.0f + expf(-logits[row * stride + head]));
+    }
+};
 
 // A tile of 64 rows x 64 outputs of one head a workgroup, k in steps of 16 through LDS, 4 x 4 outputs a thread; every
 // output's sum runs over k in order, whatever the tile it falls into.
@@ -90,7 +140,7 @@ constexpr int HEADS_TILE = 64, HEADS_K = 16;
 
 template <typename T>
 __global__ void __launch_bounds__(256) linear_heads_kernel(const T* __restrict__ a, long a_stride, long a_head, const T* __restrict__ w,
-                                                          T* __restrict__ out, long out_stride, long out_head, long rows, int n, int k) {
+                                                          T* __restrict__ out, long out_stride, long out_head, long rows, int n, int k, const HeadGates gates) {
     __shared__ float as[HEADS_K][HEADS_TILE + 1], ws[HEADS_K][HEADS_TILE + 1];
     const int head = blockIdx.z;
     const long row0 = (long)blockIdx.x * HEADS_TILE;
@@ -128,7 +178,7 @@ __global__ void __launch_bounds__(256) linear_heads_kernel(const T* __restrict__
         for (int j = 0; j < 4; ++j) {
             const long r = row0 + tr * 4 + i;
             const int c = n0 + tc * 4 + j;
-            if (r < rows && c < n) out[r * out_stride + (long)head * out_head + c] = from_float<T>(acc[i][j]);
+            if (r < rows && c < n) out[r * out_stride + (long)head * out_head + c] = from_float<T>(acc[i][j] * gates(r, head));
         }
 }
 
@@ -180,7 +230,7 @@ typedef __bf16 heads_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float heads_floatx4 __attribute__((ext_vector_type(4)));
 
 __global__ void __launch_bounds__(256) linear_heads_mfma_kernel(const bf16* __restrict__ a, long a_stride, long a_head, const bf16* __restrict__ w,
-                                                               bf16* __restrict__ out, long out_stride, long out_head, long rows, int n, int k) {
+                                                               bf16* __restrict__ out, long out_stride, long out_head, long rows, int n, int k, const HeadGates gates) {
     const int head = blockIdx.z, lane = threadIdx.x % XRT_WAVE, wave = threadIdx.x / XRT_WAVE, r = lane % 16, c = lane / 16;
     const long row0 = (long)blockIdx.x * 64 + wave * 16;
     if (row0 >= rows) return;                                  // (the whole wavefront)
@@ -202,13 +252,16 @@ __global__ void __launch_bounds__(256) linear_heads_mfma_kernel(const bf16* __re
         for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(of_rows, of_outputs[j], acc[j], 0, 0, 0);
     }
     // register i of tile j is row row0 + 4 c + i, output n0 + 16 j + r
+    float gate[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) gate[i] = gates(min(row0 + 4 * c + i, rows - 1), head);
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const long row = row0 + 4 * c + i;
             const int column = n0 + 16 * j + r;
-            if (row < rows && column < n) out[row * out_stride + (long)head * out_head + column] = (bf16)acc[j][i];
+            if (row < rows && column < n) out[row * out_stride + (long)head * out_head + column] = (bf16)(acc[j][i] * gate[i]);
         }
 }
 
@@ -220,7 +273,7 @@ constexpr int HEADS_FEW = 16, FEW_WAVES = 4;
 template <typename T>
 __global__ void __launch_bounds__(FEW_WAVES * XRT_WAVE) linear_heads_few_kernel(const T* __restrict__ a, long a_stride, long a_head,
                                                                                const T* __restrict__ w, T* __restrict__ out, long out_stride,
-                                                                               long out_head, int rows, int n, int k) {
+                                                                               long out_head, int rows, int n, int k, const HeadGates gates) {
     const int head = blockIdx.y, lane = threadIdx.x % XRT_WAVE, column = blockIdx.x * FEW_WAVES + threadIdx.x / XRT_WAVE;
     if (column >= n) return;                                   // (the whole wavefront)
     const T* of_w = w + ((long)head * n + column) * k;
@@ -261,7 +314,7 @@ __global__ void __launch_bounds__(FEW_WAVES * XRT_WAVE) linear_heads_few_kernel(
     for (int r = 0; r < HEADS_FEW; ++r) {
         if (r < rows) {
             const float sum = wave_sum(acc[r]);
-            if (lane == 0) out[(long)r * out_stride + (long)head * out_head + column] = from_float<T>(sum);
+            if (lane == 0) out[(long)r * out_stride + (long)head * out_head + column] = from_float<T>(sum * gates(r, head));
         }
     }
 }
@@ -333,8 +386,36 @@ extern "C" int xrt_latent_queries(const float* q, long q_stride, int dtype, long
     return 0;
 }
 
+extern "C" int xrt_latent_prepare(const float* q, const float* down, long stride, int dtype, long tokens, int heads, int dim, int rank, int rot_dim,
+                                  int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions,
+                                  const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
+                                  void* plain, void* full, long full_stride, void* stream) {
+    XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "latent_prepare: unknown dtype %d", dtype);
+    XRT_REQUIRE(gain_dtype == XRT_F32 || gain_dtype == XRT_BF16, "latent_prepare: unknown dtype %d of the gain", gain_dtype);
+    XRT_REQUIRE(q && down && gain && positions && slots && k_cache && v_cache && block_table && plain && full, "latent_prepare: null operand");
+    XRT_REQUIRE(tokens >= 0 && tokens < (1L << 31) && heads > 0 && heads <= 65534 && dim > 0 && rank > 0 && rot_dim >= 0 &&
+                stride >= (long)heads * (dim + rot_dim) && stride >= rank + rot_dim && full_stride >= (long)heads * (rank + rot_dim) &&
+                table_stride > 0 && n_blocks > 0, "latent_prepare: bad sizes");
+    XRT_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= rot_dim && (rot_dims == 0 || frequencies != nullptr),
+                "latent_prepare: %d dims turn in pairs inside a part of %d", rot_dims, rot_dim);
+    if (tokens == 0) return 0;
+    const dim3 grid((unsigned)tokens, 1 + (heads + PREPARE_HEADS - 1) / PREPARE_HEADS);
+    if (dtype == XRT_F32)
+        latent_prepare_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies,
+                                                                            positions, slots, (float*)k_cache, (float*)v_cache, block_table, table_stride,
+                                                                            n_blocks, (float*)plain, (float*)full, full_stride);
+    else
+        latent_prepare_kernel<bf16><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies,
+                                                                           positions, slots, (bf16*)k_cache, (bf16*)v_cache, block_table, table_stride,
+                                                                           n_blocks, (bf16*)plain, (bf16*)full, full_stride);
+    XRT_LAUNCH_CHECK("latent_prepare");
+    return 0;
+}
+
 extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const void* w, int dtype, void* out, long out_stride, long out_head,
-                                long rows, int heads, int n, int k, void* stream) {
+                                long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, void* stream) {
+    XRT_REQUIRE(gate_logits == nullptr || gate_stride >= heads, "linear_heads: rows of gates %ld apart for %d heads", gate_stride, heads);
+    const HeadGates gates{gate_logits, gate_stride};
     XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "linear_heads: unknown dtype %d", dtype);
     XRT_REQUIRE(a && w && out && rows >= 0 && heads > 0 && heads <= 65535 && n > 0 && k > 0, "linear_heads: bad operands");
     XRT_REQUIRE(a_head >= k && a_stride >= (heads - 1) * a_head + k && out_head >= n && out_stride >= (heads - 1) * out_head + n,
@@ -344,10 +425,10 @@ extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const
         const dim3 few((n + FEW_WAVES - 1) / FEW_WAVES, heads);
         if (dtype == XRT_F32)
             linear_heads_few_kernel<float><<<few, FEW_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>((const float*)a, a_stride, a_head, (const float*)w,
-                                                                                               (float*)out, out_stride, out_head, (int)rows, n, k);
+                                                                                               (float*)out, out_stride, out_head, (int)rows, n, k, gates);
         else
             linear_heads_few_kernel<bf16><<<few, FEW_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w,
-                                                                                              (bf16*)out, out_stride, out_head, (int)rows, n, k);
+                                                                                              (bf16*)out, out_stride, out_head, (int)rows, n, k, gates);
         XRT_LAUNCH_CHECK("linear_heads");
         return 0;
     }
@@ -355,7 +436,7 @@ extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const
         (rows + 63) / 64 < (1L << 31) && (n + 63) / 64 <= 65535) {
         const dim3 tiles((unsigned)((rows + 63) / 64), (n + 63) / 64, heads);
         linear_heads_mfma_kernel<<<tiles, 256, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w, (bf16*)out, out_stride, out_head,
-                                                                         rows, n, k);
+                                                                         rows, n, k, gates);
         XRT_LAUNCH_CHECK("linear_heads");
         return 0;
     }
@@ -364,10 +445,10 @@ extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const
     const dim3 grid((unsigned)row_tiles, (n + HEADS_TILE - 1) / HEADS_TILE, heads);
     if (dtype == XRT_F32)
         linear_heads_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>((const float*)a, a_stride, a_head, (const float*)w, (float*)out, out_stride,
-                                                                       out_head, rows, n, k);
+                                                                       out_head, rows, n, k, gates);
     else
         linear_heads_kernel<bf16><<<grid, 256, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w, (bf16*)out, out_stride,
-                                                                      out_head, rows, n, k);
+                                                                      out_head, rows, n, k, gates);
     XRT_LAUNCH_CHECK("linear_heads");
     return 0;
 }

@@ -4,8 +4,9 @@
 //   xrt_linear_recurrence   per head a matrix state S [dim x vdim]: S <- diag(decay) S + k v^T, read with q before or after the
 //                           update; the decay a constant per head, given per token and channel, or worked out here from a
 //                           projection (two forms); then per head an RMS norm, a weight and a gate
-//   xrt_add_normed          residual += scale * sum of RMS-normed rows with their gains
-//   xrt_activation          tanh, silu, and the two-parameter activation xIELU, elementwise
+//   xrt_add_normed          residual += scale * sum of RMS-normed rows with their gains; the updated rows once more in another
+//                           element type, for what reads the stream itself
+//   xrt_activation          tanh, silu, the tanh form of gelu, and the two-parameter activation xIELU, elementwise
 //   xrt_rows_add            out[t] += table[ids[t]]
 //   xrt_kv_store            the step's keys and values into the paged cache, values of a width of their own
 // Everything that is state, a decay, a norm or a sum onto the residual stream is float32 whatever the element type of the
@@ -513,7 +514,7 @@ __global__ void __launch_bounds__(FINISH_THREADS) recurrence_finish_groups_kerne
 
 __global__ void __launch_bounds__(256) add_normed_kernel(float* __restrict__ residual, const float* __restrict__ x0, const void* __restrict__ g0,
                                                          const float* __restrict__ x1, const void* __restrict__ g1, int gain_dtype,
-                                                         int width, float eps, float scale) {
+                                                         int width, float eps, float scale, void* __restrict__ copy, int copy_dtype) {
     __shared__ float scratch[32];
     const long row = blockIdx.x;
     const float* in[2] = {x0, x1};
@@ -529,11 +530,75 @@ __global__ void __launch_bounds__(256) add_normed_kernel(float* __restrict__ res
         float sum = 0.f;
         for (int n = 0; n < 2; ++n)
             if (in[n] != nullptr) sum += in[n][row * width + c] * inv[n] * load_as_float(gains[n], gain_dtype, c);
-        residual[row * width + c] += scale * sum;
+        const float updated = residual[row * width + c] + scale * sum;
+        residual[row * width + c] = updated;
+        if (copy != nullptr) store_from_float(copy, copy_dtype, row * width + c, updated);
+    }
+}
+
+// One part, rows of a multiple of four numbers: every load of a row is asked for at once, four numbers each, and the row stays in
+// registers between the sum and the scaling. copy (or null): the updated rows once more in another element type.
+constexpr int ADD_NORMED_OWNED = 4;
+
+__global__ void __launch_bounds__(1024) add_normed_row_kernel(float* __restrict__ residual, const float* __restrict__ x, const void* __restrict__ gain,
+                                                              int gain_dtype, int width, float eps, float scale, void* __restrict__ copy, int copy_dtype) {
+    __shared__ float scratch[32];
+    const long row = blockIdx.x;
+    const int quads = width / 4;
+    const float4* in = reinterpret_cast<const float4*>(x + row * width);
+    float4* to = reinterpret_cast<float4*>(residual + row * width);
+    float4 kept[ADD_NORMED_OWNED], before[ADD_NORMED_OWNED], gains[ADD_NORMED_OWNED];
+    float squares = 0.f;
+#pragma unroll
+    for (int i = 0; i < ADD_NORMED_OWNED; ++i) {
+        const int q = threadIdx.x + i * blockDim.x;
+        kept[i] = before[i] = gains[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (q < quads) {
+            kept[i] = in[q];
+            before[i] = to[q];
+            gains[i] = make_float4(load_as_float(gain, gain_dtype, 4 * q), load_as_float(gain, gain_dtype, 4 * q + 1),
+                                   load_as_float(gain, gain_dtype, 4 * q + 2), load_as_float(gain, gain_dtype, 4 * q + 3));
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < ADD_NORMED_OWNED; ++i)
+        squares = fmaf(kept[i].x, kept[i].x, fmaf(kept[i].y, kept[i].y, fmaf(kept[i].z, kept[i].z, fmaf(kept[i].w, kept[i].w, squares))));
+    const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / (float)width + eps);
+#pragma unroll
+    for (int i = 0; i < ADD_NORMED_OWNED; ++i) {
+        const int q = threadIdx.x + i * blockDim.x;
+        if (q < quads) {
+            const float4 v = make_float4(before[i].x + scale * (kept[i].x * inv * gains[i].x), before[i].y + scale * (kept[i].y * inv * gains[i].y),
+                                         before[i].z + scale * (kept[i].z * inv * gains[i].z), before[i].w + scale * (kept[i].w * inv * gains[i].w));
+            to[q] = v;
+            if (copy == nullptr) continue;
+            if (copy_dtype == XRT_F32) {
+                reinterpret_cast<float4*>((float*)copy + row * width)[q] = v;
+            } else {
+                struct alignas(8) Four { bf16 e[4]; } four{{from_float<bf16>(v.x), from_float<bf16>(v.y), from_float<bf16>(v.z), from_float<bf16>(v.w)}};
+                reinterpret_cast<Four*>((bf16*)copy + row * width)[q] = four;
+            }
+        }
     }
 }
 
 // ---- activations -------------------------------------------------------------------------------------------------
+
+__device__ __forceinline__ float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
+
+// The tanh form of gelu on float32 sums, four a thread.
+__global__ void __launch_bounds__(256) gelu_tanh_four_kernel(const float* __restrict__ x, void* __restrict__ out, int out_dtype, long count) {
+    const long i = ((long)blockIdx.x * blockDim.x + threadIdx.x) * 4;
+    if (i >= count) return;
+    const float4 z = *reinterpret_cast<const float4*>(x + i);
+    const float y[4] = {gelu_tanh(z.x), gelu_tanh(z.y), gelu_tanh(z.z), gelu_tanh(z.w)};
+    if (out_dtype == XRT_F32) {
+        *reinterpret_cast<float4*>((float*)out + i) = make_float4(y[0], y[1], y[2], y[3]);
+    } else {
+        struct alignas(8) Four { bf16 e[4]; } four{{from_float<bf16>(y[0]), from_float<bf16>(y[1]), from_float<bf16>(y[2]), from_float<bf16>(y[3])}};
+        *reinterpret_cast<Four*>((bf16*)out + i) = four;
+    }
+}
 
 __global__ void activation_kernel(const void* __restrict__ x, int x_dtype, void* __restrict__ out, int out_dtype, long count, int kind,
                                   const void* __restrict__ params, int params_dtype) {
@@ -545,6 +610,8 @@ __global__ void activation_kernel(const void* __restrict__ x, int x_dtype, void*
         y = tanhf(z);
     } else if (kind == XRT_UNARY_SILU) {
         y = silu_exact(z);
+    } else if (kind == XRT_UNARY_GELU_TANH) {
+        y = gelu_tanh(z);
     } else {                                               // xIELU with the numbers (p, q)
         const float p = load_as_float(params, params_dtype, 0), q = load_as_float(params, params_dtype, 1);
         if (z > 0.f) y = fmaf(softplus_exact(p) * z, z, 0.5f * z);
@@ -693,12 +760,20 @@ extern "C" int xrt_linear_recurrence(const xrt_recurrence* args, int dtype, cons
 }
 
 extern "C" int xrt_add_normed(float* residual, const float* x0, const void* gain0, const float* x1, const void* gain1, int gain_dtype,
-                              long rows, int width, float eps, float scale, void* stream) {
+                              long rows, int width, float eps, float scale, void* copy, int copy_dtype, void* stream) {
+    XRT_REQUIRE(copy == nullptr || copy_dtype == XRT_F32 || copy_dtype == XRT_BF16, "add_normed: unknown dtype of the copy");
     XRT_REQUIRE(residual && x0 && gain0 && (x1 == nullptr) == (gain1 == nullptr), "add_normed: null operand");
     XRT_REQUIRE(gain_dtype == XRT_F32 || gain_dtype == XRT_BF16, "add_normed: unknown dtype %d", gain_dtype);
     XRT_REQUIRE(rows >= 0 && rows < (1L << 31) && width > 0, "add_normed: bad sizes");
     if (rows == 0) return 0;
-    add_normed_kernel<<<(unsigned)rows, 256, 0, (hipStream_t)stream>>>(residual, x0, gain0, x1, gain1, gain_dtype, width, eps, scale);
+    const int quads = width / 4;
+    if (x1 == nullptr && width % 4 == 0 && quads <= 1024 * ADD_NORMED_OWNED && ((uintptr_t)residual | (uintptr_t)x0 | (uintptr_t)copy) % 16 == 0) {
+        const int threads = min(1024, (quads + XRT_WAVE - 1) / XRT_WAVE * XRT_WAVE);
+        add_normed_row_kernel<<<(unsigned)rows, threads, 0, (hipStream_t)stream>>>(residual, x0, gain0, gain_dtype, width, eps, scale, copy, copy_dtype);
+        XRT_LAUNCH_CHECK("add_normed");
+        return 0;
+    }
+    add_normed_kernel<<<(unsigned)rows, 256, 0, (hipStream_t)stream>>>(residual, x0, gain0, x1, gain1, gain_dtype, width, eps, scale, copy, copy_dtype);
     XRT_LAUNCH_CHECK("add_normed");
     return 0;
 }
@@ -707,9 +782,16 @@ extern "C" int xrt_activation(const void* x, int x_dtype, void* out, int out_dty
                               int params_dtype, void* stream) {
     XRT_REQUIRE(x && out && count >= 0, "activation: null operand");
     XRT_REQUIRE((x_dtype == XRT_F32 || x_dtype == XRT_BF16) && (out_dtype == XRT_F32 || out_dtype == XRT_BF16), "activation: unknown dtype");
-    XRT_REQUIRE(kind == XRT_UNARY_TANH || kind == XRT_UNARY_SILU || (kind == XRT_UNARY_XIELU && params != nullptr),
+    XRT_REQUIRE(kind == XRT_UNARY_TANH || kind == XRT_UNARY_SILU || kind == XRT_UNARY_GELU_TANH || (kind == XRT_UNARY_XIELU && params != nullptr),
                 "activation: unknown kind %d, or xIELU without its two numbers", kind);
     if (count == 0) return 0;
+    if (kind == XRT_UNARY_GELU_TANH && x_dtype == XRT_F32 && count % 4 == 0 && ((uintptr_t)x | (uintptr_t)out) % 16 == 0) {
+        const long fours = (count / 4 + 255) / 256;
+        XRT_REQUIRE(fours < (1L << 31), "activation: too many elements");
+        gelu_tanh_four_kernel<<<(unsigned)fours, 256, 0, (hipStream_t)stream>>>((const float*)x, out, out_dtype, count);
+        XRT_LAUNCH_CHECK("activation");
+        return 0;
+    }
     const long blocks = (count + 255) / 256;
     XRT_REQUIRE(blocks < (1L << 31), "activation: too many elements");
     activation_kernel<<<(unsigned)blocks, 256, 0, (hipStream_t)stream>>>(x, x_dtype, out, out_dtype, count, kind, params, params_dtype);

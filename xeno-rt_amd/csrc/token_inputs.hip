@@ -6,7 +6,9 @@
 //                       the updated rows may be written once more in another element type, for a product that reads them
 //   xrt_glu_clamped     out = g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit), from
 //                       float32 sums [rows][2 n] that hold g then u; times a weight per row, if given
-//   xrt_softcap         x <- cap * tanh(x / cap), in place on float32
+//   xrt_softcap         x <- cap * tanh(x * scale / cap), in place on float32 (cap 0: x <- x * scale)
+//   xrt_embed_normed    x = v / sqrt(mean(v^2) + eps) * gain with v = table[ids[t]] (+ positions' table[position]), in float32 and, if
+//                       asked for, once more in another element type
 //   xrt_cast            out = x in another element type
 // All arithmetic is float32. Tokens whose slot is negative are padding: they are computed like any other and touch no state.
 #include "common.h"
@@ -133,9 +135,37 @@ __global__ void __launch_bounds__(256) glu_clamped_four_kernel(const float* __re
     }
 }
 
-__global__ void softcap_kernel(float* __restrict__ x, long count, float cap) {
+__global__ void softcap_kernel(float* __restrict__ x, long count, float cap, float scale) {
     const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < count) x[i] = cap * tanhf(x[i] / cap);
+    if (i >= count) return;
+    const float z = x[i] * scale;
+    x[i] = cap > 0.f ? cap * tanhf(z / cap) : z;
+}
+
+// A workgroup a token; the row is made twice (its tables' rows are in the caches the second time).
+__global__ void __launch_bounds__(256) embed_normed_kernel(const void* __restrict__ table, const void* __restrict__ positions_table, int dtype,
+                                                          const int* __restrict__ ids, const int* __restrict__ positions, int position_rows,
+                                                          const void* __restrict__ gain, int gain_dtype, float eps, int width,
+                                                          float* __restrict__ out, void* __restrict__ copy, int copy_dtype) {
+    __shared__ float scratch[32];
+    const long t = blockIdx.x;
+    const long id = ids[t];
+    const int pos = positions_table != nullptr ? positions[t] : 0;
+    const bool placed = positions_table != nullptr && pos >= 0 && pos < position_rows;
+    auto value = [&](int c) {
+        return load_as_float(table, dtype, id * width + c) + (placed ? load_as_float(positions_table, dtype, (long)pos * width + c) : 0.f);
+    };
+    float squares = 0.f;
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+        const float v = value(c);
+        squares = fmaf(v, v, squares);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / (float)width + eps);
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+        const float v = value(c) * inv * load_as_float(gain, gain_dtype, c);
+        out[t * width + c] = v;
+        if (copy != nullptr) store_from_float(copy, copy_dtype, t * width + c, v);
+    }
 }
 
 __global__ void cast_kernel(const void* __restrict__ x, int x_dtype, void* __restrict__ out, int out_dtype, long count) {
@@ -216,13 +246,25 @@ extern "C" int xrt_glu_clamped(const float* sums, void* out, int out_dtype, long
     return 0;
 }
 
-extern "C" int xrt_softcap(float* x, long count, float cap, void* stream) {
-    XRT_REQUIRE(x && count >= 0 && cap > 0.f, "softcap: bad operands");
+extern "C" int xrt_softcap(float* x, long count, float cap, float scale, void* stream) {
+    XRT_REQUIRE(x && count >= 0 && cap >= 0.f, "softcap: bad operands");
     if (count == 0) return 0;
     const long blocks = (count + 255) / 256;
     XRT_REQUIRE(blocks < (1L << 31), "softcap: too many elements");
-    softcap_kernel<<<(unsigned)blocks, 256, 0, (hipStream_t)stream>>>(x, count, cap);
+    softcap_kernel<<<(unsigned)blocks, 256, 0, (hipStream_t)stream>>>(x, count, cap, scale);
     XRT_LAUNCH_CHECK("softcap");
+    return 0;
+}
+
+extern "C" int xrt_embed_normed(const void* table, const void* positions_table, int dtype, const int* ids, const int* positions, long tokens, int width,
+                                int position_rows, const void* gain, int gain_dtype, float eps, float* out, void* copy, int copy_dtype,
+                                void* stream) {
+    XRT_REQUIRE(table && ids && gain && out && known(dtype) && known(gain_dtype) && (copy == nullptr || known(copy_dtype)), "embed_normed: null operand or unknown dtype");
+    XRT_REQUIRE(tokens >= 0 && tokens < (1L << 31) && width > 0 && (positions_table == nullptr || (positions && position_rows > 0)), "embed_normed: bad sizes");
+    if (tokens == 0) return 0;
+    embed_normed_kernel<<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(table, positions_table, dtype, ids, positions, position_rows, gain, gain_dtype, eps,
+                                                                           width, out, copy, copy_dtype);
+    XRT_LAUNCH_CHECK("embed_normed");
     return 0;
 }
 

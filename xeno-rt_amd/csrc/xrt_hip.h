@@ -259,12 +259,13 @@ long xrt_linear_recurrence_workspace(int n_seqs, int max_count, long tokens, int
 int xrt_linear_recurrence(const xrt_recurrence* args, int dtype, const int* seq_offsets, const int* seq_slots, int n_seqs,
                           int max_count, const int* token_slots, long tokens, float* workspace, long workspace_floats, void* stream);
 
-// residual[r] += scale * (x0[r] / rms(x0[r]) * gain0 + x1[r] / rms(x1[r]) * gain1); x float32 [rows][width], x1 may be null
+// residual[r] += scale * (x0[r] / rms(x0[r]) * gain0 + x1[r] / rms(x1[r]) * gain1); x float32 [rows][width], x1 may be null;
+// copy (or null): the updated rows once more, in copy_dtype
 int xrt_add_normed(float* residual, const float* x0, const void* gain0, const float* x1, const void* gain1, int gain_dtype,
-                   long rows, int width, float eps, float scale, void* stream);
+                   long rows, int width, float eps, float scale, void* copy, int copy_dtype, void* stream);
 
-// out[i] = f(x[i]): tanh, silu, or xIELU with params = (p, q): z > 0: softplus(p) z^2 + z / 2, else (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2
-enum { XRT_UNARY_TANH = 0, XRT_UNARY_SILU = 1, XRT_UNARY_XIELU = 2 };
+// out[i] = f(x[i]): tanh, silu, gelu's tanh form z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), or xIELU with params = (p, q): z > 0: softplus(p) z^2 + z / 2, else (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2
+enum { XRT_UNARY_TANH = 0, XRT_UNARY_SILU = 1, XRT_UNARY_XIELU = 2, XRT_UNARY_GELU_TANH = 3 };
 int xrt_activation(const void* x, int x_dtype, void* out, int out_dtype, long count, int kind, const void* params, int params_dtype,
                    void* stream);
 
@@ -391,19 +392,31 @@ int xrt_add_weighted(float* residual, int count, const float* const* y, const vo
 // row_weights[r] (float32 [rows]) unless that is null
 int xrt_glu_clamped(const float* sums, void* out, int out_dtype, long rows, int n, float limit, float alpha, const float* row_weights,
                     void* stream);
-// x <- cap * tanh(x / cap), float32 in place
-int xrt_softcap(float* x, long count, float cap, void* stream);
+// x <- cap * tanh(x * scale / cap), float32 in place; cap 0: x <- x * scale
+int xrt_softcap(float* x, long count, float cap, float scale, void* stream);
+// out[t] = v / sqrt(mean(v^2) + eps) * gain with v = table[ids[t]] + positions_table[positions[t]] (no positions_table: the first alone;
+// positions beyond its rows add nothing), both tables of one dtype, all of it float32; copy (or null): the rows once more in copy_dtype
+int xrt_embed_normed(const void* table, const void* positions_table, int dtype, const int* ids, const int* positions, long tokens, int width,
+                     int position_rows, const void* gain, int gain_dtype, float eps, float* out, void* copy, int copy_dtype, void* stream);
 int xrt_cast(const void* x, int x_dtype, void* out, int out_dtype, long count, void* stream);
 
 // ---- experts (csrc/experts.hip) --------------------------------------------------------------------------------------------
-// The choice of experts for every token from router logits [tokens][experts] (float32): scores sigmoid(z); `groups` equal
+// The choice of experts for every token from router logits [tokens][experts] (float32, rows logits_stride apart): scores sigmoid(z); `groups` equal
 // groups of neighbours, a group's score the sum of its group_top largest scores, experts of the `keep` best groups stay
 // open; the `top` largest open scores are chosen; weights [tokens][experts] (float32) get score / (sum of the chosen scores
 // + floor) for the chosen and 0 for the others; chosen (or null) [tokens][top] the experts in the order of their scores.
-// softmax != 0: the scores are softmax(z) over all experts instead; scale multiplies the chosen experts' weights.
+// softmax != 0: the scores are softmax(z) over all experts instead; scale multiplies the chosen experts' weights; normalized 0: the
+// weights are the chosen scores themselves, times scale.
 #define XRT_MOST_EXPERTS 256
-int xrt_route_experts(const float* logits, long tokens, int experts, int top, int groups, int keep, int group_top, float floor_,
-                      float* weights, int* chosen, int softmax, float scale, void* stream);
+int xrt_route_experts(const float* logits, long logits_stride, long tokens, int experts, int top, int groups, int keep, int group_top,
+                      float floor_, float* weights, int* chosen, int softmax, float scale, int normalized, void* stream);
+// What every expert's down product reads, from float32 gate and up sums of every token with all experts: with total = experts *
+// width + shared_width columns c, sums [tokens][2 total] hold gate c at c and up c at total + c, or (interleaved; total a multiple of
+// eight) in groups of sixteen eight gates and their eight ups. out[t][c] = silu(g) * u * w, or (weigh_input) silu(w g) * (w u), w =
+// weights[t][c / width]; 0 where that is 0. The columns behind the experts' are a shared expert's: silu(g) * u *
+// sigmoid(shared_logits[t * shared_stride]) (null: without the last factor).
+int xrt_glu_experts(const float* sums, void* out, int out_dtype, long tokens, int experts, int width, int shared_width, const float* weights,
+                    const float* shared_logits, long shared_stride, int weigh_input, int interleaved, void* stream);
 // act[t][e * width + c] *= weights[t][e]
 int xrt_scale_blocks(void* act, int dtype, const float* weights, long tokens, int experts, int width, void* stream);
 
@@ -414,11 +427,16 @@ int xrt_scale_blocks(void* act, int dtype, const float* weights, long tokens, in
 // where rows[r] < 0). xrt_linear_groups multiplies every tile of rows of a with the matrix of its tile's group, w + group *
 // w_stride (elements), whose rows lie ldw apart and of which k columns are summed over (coded_mode as in xrt_linear_with: 0,
 // or 2 | activation << 8 with a packed gated matrix of n pairs per group); `accepts` says what it serves.
-// xrt_experts_combine: out[t] = sum over the picks of t, in their order, of weights[t][chosen[t][k]] * sorted[places[t][k]].
+// xrt_gather_rows with weights [tokens][experts] (or null): a row times its token's weight for the expert of its tile of `tile` rows.
+// xrt_experts_combine: out[t] = sum over the picks of t, in their order, of weights[t][chosen[t][k]] * sorted[places[t][k]] (weigh 0:
+// without the weights), and with shared (float32 rows of `width` for all tokens in
+// their order, in tiles of shared_tile rows and shared_parts parts as xrt_linear_groups leaves them, or null)
+// + sigmoid(shared_logits[t * shared_stride]) * shared[t].
 int xrt_linear_groups_tile_rows(long tokens, int top, int experts);
 long xrt_experts_sort_room(long tokens, int top, int experts);
 int xrt_experts_sort(const int* chosen, long tokens, int top, int experts, int* rows, long room, int* places, int* tile_group, void* stream);
-int xrt_gather_rows(const void* x, long x_stride, const int* rows, long count, int width, void* out, void* stream);
+int xrt_gather_rows(const void* x, long x_stride, const int* rows, long count, int width, void* out, const float* weights, int experts,
+                    const int* tile_group, int tile, void* stream);
 int xrt_linear_groups_accepts(const void* a, int lda, const void* w, int ldw, int n, int k, int mode, const xrt_packing* packing);
 // parts: 1, or with plain sums 2: k in two halves whose sums lie tile after tile, [tiles][parts][tile rows][n], for
 // xrt_experts_combine to add (xrt_linear_groups_parts: which of the two pays, from the number of tiles).
@@ -426,7 +444,8 @@ int xrt_linear_groups_parts(long tiles, int n, int k, int coded_mode);
 int xrt_linear_groups(const void* a, int lda, const void* w, long w_stride, int ldw, const xrt_packing* packing, void* out, int out_dtype,
                       int tile, long tiles, int n, int k, int coded_mode, const int* tile_group, int parts, void* stream);
 int xrt_experts_combine(const float* sorted, const int* places, const int* chosen, const float* weights, long tokens, int top, int experts,
-                        int width, int tile, int parts, float* out, void* stream);
+                        int width, int tile, int parts, float* out, int weigh, const float* shared, int shared_tile, int shared_parts,
+                        const float* shared_logits, long shared_stride, void* stream);
 
 // ---- a residual stream in several copies (csrc/streams.hip) ------------------------------------------------------------------
 // streams: float32 [tokens][copies][width]. open: every copy is the token's row of x. read: out[r] = norm(sum over the copies s
@@ -450,7 +469,10 @@ int xrt_streams_write(float* streams, int copies, const float* mix, const float*
 // and the turned parts to full[t][h][rank ..], rows full_stride apart, heads rank + rot_dim apart.
 // linear_heads: out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k]; rows of a and out a_stride and out_stride apart, heads
 // a_head and out_head apart; all three of `dtype`, float32 sums (whose order depends on whether the step has up to 16 rows or more and on
-// the sizes, on nothing else: a row's result never depends on the rows around it).
+// the sizes, on nothing else: a row's result never depends on the rows around it); with gate_logits (float32, rows gate_stride apart, or
+// null) times sigmoid(gate_logits[t][h]) before it is rounded.
+// prepare: complete and queries in one launch, from float32 rows `stride` apart of which q points at the queries and down at the
+// latents (no rows_out).
 int xrt_latent_complete(const float* down, long down_stride, int dtype, long tokens, int rank, int rot_dim, int rot_dims,
                         const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions, const int* slots,
                         void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks, void* rows_out, void* stream);
@@ -463,20 +485,31 @@ int xrt_causal_softmax(const float* scores, long rows, long keys, int heads, int
 int xrt_transpose(const void* src, long src_stride, int dtype, long rows, int cols, void* dst, void* stream);
 int xrt_latent_queries(const float* q, long q_stride, int dtype, long tokens, int heads, int dim, int rot_dim, int rot_dims,
                        const float* frequencies, const int* positions, void* plain, void* full, long full_stride, int rank, void* stream);
+int xrt_latent_prepare(const float* q, const float* down, long stride, int dtype, long tokens, int heads, int dim, int rank, int rot_dim,
+                       int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions,
+                       const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
+                       void* plain, void* full, long full_stride, void* stream);
 int xrt_linear_heads(const void* a, long a_stride, long a_head, const void* w, int dtype, void* out, long out_stride, long out_head,
-                     long rows, int heads, int n, int k, void* stream);
+                     long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, void* stream);
 
 // ---- many heads on one key/value head with large keys, on the matrix cores (csrc/attention_latent.hip) ------------------------
 // Causal attention of the step's tokens (queries alone in q, rows q_stride apart, n_heads x head_dim each) over a cache with one
-// key/value head, keys of head_dim and values of value_dim numbers (multiples of 32 up to 512: `accepts`), bfloat16; with
-// sink_scores (float32 [n_heads], or null) the softmax's denominator also holds exp(sink_scores[head]). out: rows of
-// n_heads x value_dim. max_context: the longest sequence after this step; the workspace holds `xrt_attention_latent_workspace` floats.
+// key/value head, keys of head_dim and values of value_dim numbers (multiples of 32 up to 640 and 512: `accepts`), bfloat16; a
+// query sees the keys at or before it, of those the `window` newest (0: all); with sink_scores (float32 [n_heads], or null) the
+// softmax's denominator also holds exp(sink_scores[head]). out: rows of n_heads x value_dim. max_context: the longest sequence
+// after this step; the workspace holds `xrt_attention_latent_workspace` floats.
+// prompts: the same for steps that bring sequences many tokens (the step's sequences as in xrt_attention; rows of q lie
+// n_heads * head_dim apart; rows of no sequence are left as they are), scale > 0.
 int xrt_attention_latent_accepts(int dtype, int n_kv_heads, int head_dim, int value_dim);
-long xrt_attention_latent_workspace(long tokens, int n_heads, int value_dim, int max_context);
+long xrt_attention_latent_workspace(long tokens, int n_heads, int value_dim, int max_context, int window);
 int xrt_attention_latent(const void* q, long q_stride, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
                          const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* positions,
-                         const int* slots, void* out, float scale, const float* sink_scores, int max_context, float* workspace,
+                         const int* slots, void* out, float scale, int window, const float* sink_scores, int max_context, float* workspace,
                          long workspace_floats, void* stream);
+int xrt_attention_latent_prompts(const void* q, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
+                                 const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* seq_offsets,
+                                 const int* seq_slots, const int* seq_starts, int n_seqs, void* out, float scale, int window,
+                                 const float* sink_scores, int max_context, void* stream);
 
 #ifdef __cplusplus
 }

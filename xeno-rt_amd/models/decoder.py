@@ -100,16 +100,27 @@ class DecoderModel:
         for part in spec.parts():
             part.bind(tensors, runtime)
 
+    def _first_reads_stream(self) -> bool:
+        """Whether the first block reads the stream itself in the compute dtype and the embedding can hand it that beside the stream."""
+        spec = self.spec
+        first = spec.layers[spec.schedule[0].layer]
+        reads = first.first_norm() if getattr(first, "passes_norms", False) else None
+        return (getattr(reads, "reads_stream", False) and spec.streams is None and self.runtime.dtype != torch.float32
+                and getattr(spec.embedding, "norm_name", None) is not None)
+
     def forward(self, batch, cache) -> torch.Tensor:
         """Logits [len(batch.logit_rows), vocab] in float32 for the tokens of `batch`."""
         spec = self.spec
+        h = None            # what the next block reads first (its first norm of x), where the part before it has made it already
         if getattr(spec.embedding, "keeps_state", False):       # its cache entry follows the schedule's
             x = spec.embedding.forward_step(batch, cache.layer_cache(len(spec.schedule)))
+        elif self._first_reads_stream():
+            h = self.runtime.empty((batch.n_tokens, spec.embedding.hidden))
+            x = spec.embedding.forward_copied(batch.token_ids, batch.positions, h)
         else:
             x = spec.embedding.forward(batch.token_ids, batch.positions)
         if spec.streams is not None:                             # the blocks then work on the copies [tokens, copies, hidden]
             x = spec.streams.open(x)
-        h = None            # the next block's first norm of x, where the block before it has made it already
         for index, call in enumerate(spec.schedule):
             block = spec.layers[call.layer]
             if not getattr(block, "passes_norms", False):

@@ -72,6 +72,11 @@ class PackedMatrix:
     def dim(self) -> int:
         return 2
 
+    def rows_as_they_lie(self) -> "PackedMatrix":
+        """The same data as plain tiles: its products come out in the order in which the rows lie, not in that of the outputs (a gated
+        matrix: eight gates and their eight ups, in turn). For a reader that knows the order and wants the sums themselves."""
+        return PackedMatrix(self.data, self.shape[0], self.shape[1], _Packing(PACK_TILES, 0, 0, 0))
+
     def unpacked(self) -> torch.Tensor:
         """The matrix [rows, k] with rows contiguous along k again (for inspection and tests; products never need it)."""
         rows, cols = self.shape
@@ -153,7 +158,7 @@ CONV_MODES = {"plain": 0, "plus_input": 1, "towards_last": 2}          # XRT_CON
 DECAY_MODES = {"per_head": 0, "given": 1, "exp_neg_exp": 2, "sigmoid_power": 3, "step": 4}      # XRT_DECAY_*
 CONV_ACTIVATIONS = {None: 0, "silu": 1}                                # XRT_CONV_ACT_*
 MOST_EXPERTS = 256                                                     # XRT_MOST_EXPERTS
-UNARY = {"tanh": 0, "silu": 1, "xielu": 2}                             # XRT_UNARY_*
+UNARY = {"tanh": 0, "silu": 1, "xielu": 2, "gelu_tanh": 3}                             # XRT_UNARY_*
 
 
 class HipOps:
@@ -203,7 +208,7 @@ class HipOps:
                      "xrt_experts_sort", "xrt_gather_rows", "xrt_linear_groups", "xrt_linear_groups_accepts", "xrt_experts_combine",
                      "xrt_linear_groups_tile_rows", "xrt_linear_groups_parts", "xrt_streams_open", "xrt_streams_read", "xrt_streams_write",
                      "xrt_latent_complete", "xrt_latent_queries", "xrt_linear_heads", "xrt_causal_softmax", "xrt_transpose", "xrt_attention_latent",
-                     "xrt_attention_latent_accepts"):
+                     "xrt_attention_latent_accepts", "xrt_attention_latent_prompts", "xrt_latent_prepare", "xrt_glu_experts", "xrt_embed_normed"):
             getattr(self.lib, name).restype = ctypes.c_int
         from ..cache.allocator import BLOCK_TOKENS
         if int(self.lib.xrt_block_tokens()) != BLOCK_TOKENS:
@@ -506,8 +511,8 @@ class HipOps:
                 and self._attention_stretches(qkv, n_heads, n_kv_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, chunk,
                                               distance_bias, sink if isinstance(sink, torch.Tensor) else None)):
             return None
-        if (queries_alone and n_kv_heads == 1 and sink is not True and distance_bias is None and distance_slopes is None and not window and not chunk
-                and self._attention_one_kv_head(qkv, n_heads, head_dim, value_dim or head_dim, kv, batch, out, scale,
+        if (queries_alone and n_kv_heads == 1 and sink is not True and distance_bias is None and distance_slopes is None and not chunk
+                and self._attention_one_kv_head(qkv, n_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, window,
                                                 sink if isinstance(sink, torch.Tensor) else None)):
             return None
         if sink is not False or (value_dim is not None and value_dim != head_dim) or distance_bias is not None or queries_alone or chunk:
@@ -546,28 +551,53 @@ class HipOps:
             ctypes.c_float(scale), int(window or 0), _ptr(distance_slopes), _ptr(offsets), _ptr(seq_slots), _ptr(starts), n_seqs,
             max_count, max_context, _ptr(workspace), ctypes.c_long(workspace_floats), self._stream(qkv)))
 
-    def _attention_one_kv_head(self, q, n_heads, head_dim, value_dim, kv, batch, out, scale, sink_scores) -> bool:
-        """The matrix-core kernel for many query heads on one key/value head (the queries alone in `q`; bfloat16, key and value
-        sizes that are multiples of 32 up to 512). False: not served here, and nothing was done."""
+    def attention_takes_latent(self, dtype, head_dim, value_dim) -> bool:
+        """Whether `attention` has matrix-core kernels for many query heads on one key/value head of these sizes."""
+        return dtype in _CODES and bool(self.lib.xrt_attention_latent_accepts(_CODES[dtype], 1, int(head_dim), int(value_dim)))
+
+    PROMPTS_FROM = 16           # new tokens of some sequence from which a step takes the kernel for prompts
+
+    def _attention_one_kv_head(self, q, n_heads, head_dim, value_dim, kv, batch, out, scale, window, sink_scores) -> bool:
+        """The matrix-core kernels for many query heads on one key/value head (the queries alone in `q`; bfloat16, key and value
+        sizes that are multiples of 32 up to 640 and 512): one for steps of few tokens a sequence, one for prompts. False: not
+        served here, and nothing was done."""
         tokens = q.shape[0]
         max_context = int(getattr(batch, "max_context", 0) or 0)
-        if tokens > 65535 or max_context <= 0 or not self.lib.xrt_attention_latent_accepts(_code(q), 1, head_dim, value_dim):
+        if max_context <= 0 or not self.lib.xrt_attention_latent_accepts(_code(q), 1, head_dim, value_dim):
+            return False
+        offsets, seq_slots = getattr(batch, "sequence_offsets", None), getattr(batch, "sequence_slots", None)
+        starts, counts = getattr(batch, "sequence_starts", None), getattr(batch, "host_counts", None)
+        prompts = (int(getattr(batch, "max_count", 0) or 0) >= self.PROMPTS_FROM and scale > 0 and offsets is not None and seq_slots is not None
+                   and starts is not None and 0 < int(batch.n_sequences) <= tokens and q.is_contiguous() and tokens * n_heads < 2 ** 30)
+        if not prompts and tokens > 65535:
             return False
         q_stride = self._rows(q, "attention q", n_heads * head_dim)
         if q_stride % 8 != 0 or q.data_ptr() % 16 != 0:
             return False
         self._require(out, "attention out", q.dtype, (tokens, n_heads * value_dim), q)
-        self._require(batch.positions, "positions", torch.int32, (tokens,), q)
-        self._require(batch.slots, "slots", torch.int32, (tokens,), q)
         k_cache, v_cache, table, stride, n_blocks = self._kv(kv, q, 1, head_dim, value_dim)
         if sink_scores is not None:
             self._require(sink_scores, "attention sink", torch.float32, (n_heads,), q)
-        need = int(self.lib.xrt_attention_latent_workspace(ctypes.c_long(tokens), n_heads, value_dim, max_context))
+        if prompts:
+            n_seqs = int(batch.n_sequences)
+            self._require(offsets, "sequence offsets", torch.int32, (n_seqs + 1,), q)
+            self._require(seq_slots, "sequence slots", torch.int32, (n_seqs,), q)
+            self._require(starts, "sequence starts", torch.int32, (n_seqs,), q)
+            if counts is None or sum(counts) < tokens:
+                out.zero_()                       # padding rows: written by no one, read by the product that follows
+            self._check(self.lib.xrt_attention_latent_prompts(
+                _ptr(q), ctypes.c_long(tokens), n_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride, n_blocks, _ptr(offsets),
+                _ptr(seq_slots), _ptr(starts), n_seqs, _ptr(out), ctypes.c_float(scale), int(window or 0), _ptr(sink_scores), max_context,
+                self._stream(q)))
+            return True
+        self._require(batch.positions, "positions", torch.int32, (tokens,), q)
+        self._require(batch.slots, "slots", torch.int32, (tokens,), q)
+        need = int(self.lib.xrt_attention_latent_workspace(ctypes.c_long(tokens), n_heads, value_dim, max_context, int(window or 0)))
         workspace = self._empty(need, torch.float32, q.device)
         self._check(self.lib.xrt_attention_latent(
             _ptr(q), ctypes.c_long(q_stride), ctypes.c_long(tokens), n_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride,
-            n_blocks, _ptr(batch.positions), _ptr(batch.slots), _ptr(out), ctypes.c_float(scale), _ptr(sink_scores), max_context, _ptr(workspace),
-            ctypes.c_long(need), self._stream(q)))
+            n_blocks, _ptr(batch.positions), _ptr(batch.slots), _ptr(out), ctypes.c_float(scale), int(window or 0), _ptr(sink_scores), max_context,
+            _ptr(workspace), ctypes.c_long(need), self._stream(q)))
         return True
 
     def _attention_stretches(self, q, n_heads, n_kv_heads, head_dim, value_dim, kv, batch, out, scale, chunk, distance_bias=None,
@@ -1018,10 +1048,31 @@ class HipOps:
         self._check(self.lib.xrt_glu_clamped(_ptr(sums), _ptr(out), _code(out), ctypes.c_long(rows), n, ctypes.c_float(limit),
                                              ctypes.c_float(alpha), _ptr(row_weights), self._stream(sums)))
 
-    def softcap(self, x, cap):
-        """x <- cap * tanh(x / cap), in place; x float32."""
+    def softcap(self, x, cap, scale=1.0):
+        """x <- cap * tanh(x * scale / cap), in place; x float32. cap None: x <- x * scale."""
         self._require(x, "softcap x", torch.float32)
-        self._check(self.lib.xrt_softcap(_ptr(x), ctypes.c_long(x.numel()), ctypes.c_float(cap), self._stream(x)))
+        if cap is not None and not cap > 0:
+            raise KernelError(f"softcap: the cap must be positive, found {cap}")
+        self._check(self.lib.xrt_softcap(_ptr(x), ctypes.c_long(x.numel()), ctypes.c_float(0.0 if cap is None else cap), ctypes.c_float(scale),
+                                         self._stream(x)))
+
+    def embed_normed(self, table, ids, gain, eps, out, positions_table=None, positions=None, copy=None):
+        """out[t] (float32) = v / sqrt(mean(v^2) + eps) * gain with v = table[ids[t]] (+ positions_table[positions[t]]); copy: a tensor
+        shaped like out that takes the rows once more in its own element type."""
+        vocab, width = table.shape
+        tokens = ids.shape[0]
+        self._require(table, "embed_normed table")
+        self._require(ids, "embed_normed ids", torch.int32, (tokens,), table)
+        self._require(gain, "embed_normed gain", None, (width,), table)
+        self._require(out, "embed_normed out", torch.float32, (tokens, width), table)
+        if positions_table is not None:
+            self._require(positions_table, "embed_normed positions_table", table.dtype, (positions_table.shape[0], width), table)
+            self._require(positions, "embed_normed positions", torch.int32, (tokens,), table)
+        if copy is not None:
+            self._require(copy, "embed_normed copy", None, (tokens, width), table)
+        self._check(self.lib.xrt_embed_normed(_ptr(table), _ptr(positions_table), _code(table), _ptr(ids), _ptr(positions), ctypes.c_long(tokens), width,
+                                              0 if positions_table is None else positions_table.shape[0], _ptr(gain), _code(gain),
+                                              ctypes.c_float(eps), _ptr(out), _ptr(copy), 0 if copy is None else _code(copy), self._stream(out)))
 
     def cast(self, x, out):
         """out = x in out's element type."""
@@ -1029,21 +1080,47 @@ class HipOps:
         self._require(out, "cast out", None, x.shape, x)
         self._check(self.lib.xrt_cast(_ptr(x), _code(x), _ptr(out), _code(out), ctypes.c_long(x.numel()), self._stream(x)))
 
-    def route_experts(self, logits, weights, top, groups=1, keep=1, group_top=2, floor=1e-20, chosen=None, scores="sigmoid", scale=1.0):
-        """From router logits [tokens, experts] (float32) the weights [tokens, experts] (float32; zero for experts not chosen):
-        scores sigmoid(z) or, scores="softmax", softmax(z) over all experts; the chosen weights times `scale` in the end; experts in `groups` equal groups of neighbours, a group's score the sum of its group_top largest,
-        experts of the `keep` best groups stay open; the `top` largest open scores are chosen and divided by their sum + floor.
+    def route_experts(self, logits, weights, top, groups=1, keep=1, group_top=2, floor=1e-20, chosen=None, scores="sigmoid", scale=1.0,
+                      normalized=True):
+        """From router logits [tokens, experts] (float32, columns of a wider matrix will do) the weights [tokens, experts] (float32; zero
+        for experts not chosen): scores sigmoid(z) or, scores="softmax", softmax(z) over all experts; experts in `groups` equal groups of
+        neighbours, a group's score the sum of its group_top largest, experts of the `keep` best groups stay open; the `top` largest open
+        scores are chosen and divided by their sum + floor (normalized False: left as they are), times `scale`.
         chosen (int32 [tokens, top], or None) takes the chosen experts in the order of their scores."""
         tokens, experts = logits.shape
-        self._require(logits, "route_experts logits", torch.float32)
+        stride = self._rows(logits, "route_experts logits", experts, torch.float32)
         self._require(weights, "route_experts weights", torch.float32, (tokens, experts), logits)
         if chosen is not None:
             self._require(chosen, "route_experts chosen", torch.int32, (tokens, top), logits)
         if scores not in ("sigmoid", "softmax"):
             raise KernelError(f"route_experts: scores are 'sigmoid' or 'softmax', found {scores!r}")
-        self._check(self.lib.xrt_route_experts(_ptr(logits), ctypes.c_long(tokens), experts, int(top), int(groups), int(keep), int(group_top),
-                                               ctypes.c_float(floor), _ptr(weights), _ptr(chosen), int(scores == "softmax"),
-                                               ctypes.c_float(scale), self._stream(logits)))
+        self._check(self.lib.xrt_route_experts(_ptr(logits), ctypes.c_long(stride), ctypes.c_long(tokens), experts, int(top), int(groups), int(keep),
+                                               int(group_top), ctypes.c_float(floor), _ptr(weights), _ptr(chosen), int(scores == "softmax"),
+                                               ctypes.c_float(scale), int(bool(normalized)), self._stream(logits)))
+
+    def _shared_logits(self, shared_logits, tokens, like):
+        """(pointer argument, distance of two tokens' numbers) of a column of float32 logits, or of None."""
+        if shared_logits is None:
+            return _ptr(None), 0
+        if (not shared_logits.is_cuda or shared_logits.dtype != torch.float32 or shared_logits.dim() != 1 or shared_logits.shape[0] != tokens
+                or shared_logits.device != like.device):
+            raise KernelError(f"a shared expert's logits: float32 [{tokens}] on the GPU, found {tuple(shared_logits.shape)} {shared_logits.dtype}")
+        return _ptr(shared_logits), int(shared_logits.stride(0)) if tokens > 1 else 1
+
+    def glu_experts(self, sums, out, weights, width, shared_width=0, shared_logits=None, weigh_input=False, interleaved=False):
+        """The rows that the experts' down product reads, from the float32 sums of every token with all experts: sums [tokens, 2 * total],
+        total = experts * width + shared_width columns, gates then ups (interleaved: as products with a matrix packed for a gated
+        epilogue leave them, in groups of eight gates and their eight ups). out[t, c] = silu(g) * u * w with w = weights[t, c // width],
+        or, weigh_input, silu(w g) * (w u); the last shared_width columns are a shared expert's, times sigmoid(shared_logits[t])
+        (float32 [tokens], may be a column of a wider matrix) if given."""
+        tokens, experts = weights.shape
+        total = experts * int(width) + int(shared_width)
+        self._require(sums, "glu_experts sums", torch.float32, (tokens, 2 * total))
+        self._require(out, "glu_experts out", None, (tokens, total), sums)
+        self._require(weights, "glu_experts weights", torch.float32, (tokens, experts), sums)
+        logits, stride = self._shared_logits(shared_logits, tokens, sums)
+        self._check(self.lib.xrt_glu_experts(_ptr(sums), _ptr(out), _code(out), ctypes.c_long(tokens), experts, int(width), int(shared_width), _ptr(weights),
+                                             logits, ctypes.c_long(stride), int(bool(weigh_input)), int(bool(interleaved)), self._stream(sums)))
 
     # -- a residual stream in several copies -----------------------------------------------------------
     def streams_open(self, x, streams):
@@ -1145,31 +1222,64 @@ class HipOps:
                                                 int(rot_dims), _ptr(frequencies), _ptr(batch.positions), _ptr(plain), _ptr(full),
                                                 ctypes.c_long(heads * (rank + rot_dim)), rank, self._stream(q)))
 
-    def linear_heads(self, a, w, out, out_head=None):
+    def latent_prepare(self, q, down, heads, dim, rank, rot_dim, gain, eps, frequencies, rot_dims, kv, batch, plain, full):
+        """`latent_complete` of `down` and `latent_queries` of `q` in one launch: both float32 columns of one matrix, or of two whose
+        rows lie equally far apart."""
+        tokens = q.shape[0]
+        stride = self._rows(q, "latent_prepare q", heads * (dim + rot_dim), torch.float32)
+        down_stride = self._rows(down, "latent_prepare down", rank + rot_dim, torch.float32, q)
+        if tokens == 1:
+            stride = down_stride = max(stride, down_stride)          # (a single row lies nowhere apart)
+        if down_stride != stride:
+            raise KernelError("latent_prepare: the rows of q and down lie unequally far apart")
+        self._require(plain, "latent_prepare plain", None, (tokens, heads * dim), q)
+        self._require(full, "latent_prepare full", plain.dtype, (tokens, heads * (rank + rot_dim)), q)
+        self._require(gain, "latent_prepare gain", None, (rank,), q)
+        if rot_dims:
+            self._require(frequencies, "latent_prepare frequencies", torch.float32, (rot_dims // 2,), q)
+        self._require(batch.positions, "positions", torch.int32, (tokens,), q)
+        self._require(batch.slots, "slots", torch.int32, (tokens,), q)
+        k_cache, v_cache, table, table_stride, n_blocks = self._kv(kv, plain, 1, rank + rot_dim, rank)
+        self._check(self.lib.xrt_latent_prepare(_ptr(q), _ptr(down), ctypes.c_long(stride), _code(plain), ctypes.c_long(tokens), heads, dim, rank, rot_dim,
+                                                int(rot_dims), _ptr(gain), _code(gain), ctypes.c_float(eps), _ptr(frequencies), _ptr(batch.positions),
+                                                _ptr(batch.slots), _ptr(k_cache), _ptr(v_cache), _ptr(table), table_stride, n_blocks, _ptr(plain),
+                                                _ptr(full), ctypes.c_long(heads * (rank + rot_dim)), self._stream(q)))
+
+    def linear_heads(self, a, w, out, out_head=None, gate_logits=None):
         """out[t, h, :n] = w[h] a[t, h]: a [tokens, heads * k], w [heads, n, k], out [tokens, heads * out_head] with the head's
-        n outputs at the beginning of its out_head columns (out_head None: n). One element type, float32 sums in the order of k."""
+        n outputs at the beginning of its out_head columns (out_head None: n). One element type, float32 sums in the order of k.
+        gate_logits (float32 [tokens, heads], columns of a wider matrix will do): times sigmoid(gate_logits[t, h]) before the rounding."""
         heads, n, k = w.shape
         tokens = a.shape[0]
         out_head = n if out_head is None else int(out_head)
         self._require(a, "linear_heads a", None, (tokens, heads * k))
         self._require(w, "linear_heads w", a.dtype, None, a)
         self._require(out, "linear_heads out", a.dtype, (tokens, heads * out_head), a)
+        gate_stride = 0
+        if gate_logits is not None:
+            gate_stride = self._rows(gate_logits, "linear_heads gate_logits", heads, torch.float32, a)
+            if gate_logits.shape[0] != tokens:
+                raise KernelError(f"linear_heads gate_logits: {gate_logits.shape[0]} rows for {tokens} tokens")
         self._check(self.lib.xrt_linear_heads(_ptr(a), ctypes.c_long(heads * k), ctypes.c_long(k), _ptr(w), _code(a), _ptr(out),
                                               ctypes.c_long(heads * out_head), ctypes.c_long(out_head), ctypes.c_long(tokens), heads, n, k,
-                                              self._stream(a)))
+                                              _ptr(gate_logits), ctypes.c_long(gate_stride), self._stream(a)))
 
     # -- experts that multiply only the tokens that chose them
-    def _expert_matrices(self, w_gate_up, w_down, experts, width, stacked=False):
+    def _expert_matrices(self, w_gate_up, w_down, experts, width, stacked=False, shared_width=0):
         """(data, packing, elements between two experts' matrices, row distance) of the gate/up matrix and of the down matrix, as
         `xrt_linear_groups` wants them, or None: [all gates | all ups] packed for a gated epilogue lies expert after expert
         already (a group of sixteen packed rows holds eight outputs' gate and up rows); an expert's down matrix is `width`
         columns of the wide one. stacked: the gate/up matrix is a plain one that holds every expert's [gate rows | up rows] one
-        below the other (for experts whose activation reads float32 sums of both)."""
-        if width % 64 != 0:
+        below the other (for experts whose activation reads float32 sums of both). shared_width: the rows and columns of a
+        shared expert of that width, behind all others' in both matrices."""
+        if width % 64 != 0 or shared_width % 64 != 0:
             return None
         hidden = w_gate_up.shape[1]
+        total = experts * width + shared_width
+        if tuple(w_down.shape) != (hidden, total):
+            return None
         if stacked:
-            if tuple(w_gate_up.shape) != (2 * experts * width, hidden) or tuple(w_down.shape) != (hidden, experts * width):
+            if tuple(w_gate_up.shape) != (2 * total, hidden) or shared_width:
                 return None
             if isinstance(w_gate_up, PackedMatrix):            # in tiles of 16 rows, an expert's rows (a multiple of 128) begin where they would unpacked
                 if w_gate_up.packing.kind != PACK_TILES:
@@ -1178,23 +1288,21 @@ class HipOps:
             else:
                 up = (w_gate_up, None, 2 * width * hidden, hidden)
         else:
-            if not isinstance(w_gate_up, PackedMatrix) or w_gate_up.packing.kind != PACK_GATED:
-                return None
-            if w_gate_up.packing.gated_n != experts * width or tuple(w_down.shape) != (hidden, experts * width):
+            if not isinstance(w_gate_up, PackedMatrix) or w_gate_up.packing.kind != PACK_GATED or w_gate_up.packing.gated_n != total:
                 return None
             up = (w_gate_up.data, _Packing(PACK_GATED, width, 0, 0), 2 * width * hidden, hidden)
         if isinstance(w_down, PackedMatrix):
             if w_down.packing.kind != PACK_TILES:
                 return None
-            down = (w_down.data, w_down.packing, width * 16, experts * width)
+            down = (w_down.data, w_down.packing, width * 16, total)
         else:
-            down = (w_down, None, width, experts * width)
+            down = (w_down, None, width, total)
         return up, down
 
-    def experts_sorted_takes(self, h, w_gate_up, w_down, experts, width, top, stacked=False) -> bool:
+    def experts_sorted_takes(self, h, w_gate_up, w_down, experts, width, top, stacked=False, shared_width=0) -> bool:
         """Whether `experts_sorted` serves these operands, and pays: it multiplies every pick once, in tiles that are filled up
-        per expert, where the plain way multiplies every token with every expert. stacked: see `_expert_matrices`."""
-        matrices = self._expert_matrices(w_gate_up, w_down, experts, width, stacked)
+        per expert, where the plain way multiplies every token with every expert. stacked, shared_width: see `_expert_matrices`."""
+        matrices = self._expert_matrices(w_gate_up, w_down, experts, width, stacked, shared_width)
         if matrices is None or h.dtype != torch.bfloat16 or h.dim() != 2 or h.shape[1] % 64 != 0 or experts > 256:
             return False
         tokens, hidden = h.shape
@@ -1205,22 +1313,50 @@ class HipOps:
         takes_up = (self.lib.xrt_linear_groups_accepts(_ptr(h), hidden, _ptr(up), up_rows, 2 * width, hidden, 0,
                                                        None if up_packing is None else ctypes.byref(up_packing)) if stacked else
                     self.lib.xrt_linear_groups_accepts(_ptr(h), hidden, _ptr(up), up_rows, width, hidden, 2, ctypes.byref(up_packing)))
-        return bool(takes_up and self.lib.xrt_linear_groups_accepts(_ptr(h), width, _ptr(down), down_rows, hidden, width, 0,
-                                                           None if down_packing is None else ctypes.byref(down_packing)))
+        return bool(takes_up and all(self.lib.xrt_linear_groups_accepts(_ptr(h), k, _ptr(down), down_rows, hidden, k, 0,
+                                                                        None if down_packing is None else ctypes.byref(down_packing))
+                                     for k in ((width, shared_width) if shared_width else (width,))))
 
     def group_tile(self, tokens: int, top: int, experts: int) -> int:
         """Rows of a tile of sorted picks for a step of that many tokens."""
         return int(self.lib.xrt_linear_groups_tile_rows(ctypes.c_long(tokens), int(top), int(experts)))
 
-    def experts_sorted(self, h, w_gate_up, w_down, weights, chosen, width, out, activation: str = "silu", clamp=None):
+    SHARED_TILE = 128
+
+    def _shared_expert(self, h, w_gate_up, down, first, width, activation):
+        """A shared expert's outputs (float32, tokens filled up to tiles of SHARED_TILE rows; [tiles, parts, SHARED_TILE, hidden]) and the
+        parts they come in: its gate and up rows are the last `width` of each in the packed matrix, its down matrix the `width`
+        columns from `first` on of the wide one."""
+        tokens, hidden = h.shape
+        data, packing, _, down_rows = down
+        mine = PackedMatrix(w_gate_up.data[2 * first * hidden:2 * (first + width) * hidden], 2 * width, hidden, _Packing(PACK_GATED, width, 0, 0))
+        tile = self.SHARED_TILE
+        tiles = (tokens + tile - 1) // tile
+        parts = int(self.lib.xrt_linear_groups_parts(ctypes.c_long(tiles), hidden, width, 0))
+        act = self._empty((tiles * tile, width), torch.bfloat16, h.device)
+        self.linear_glu(h, mine, act[:tokens], activation=activation)
+        out = self._empty((tiles * parts * tile, hidden), torch.float32, h.device)
+        of_mine = data.data_ptr() + data.element_size() * first * (16 if packing is not None else 1)
+        groups = self._empty((tiles,), torch.int32, h.device)
+        groups.zero_()                                          # every tile multiplies the one matrix
+        self._check(self.lib.xrt_linear_groups(_ptr(act), width, ctypes.c_void_p(of_mine), ctypes.c_long(0), down_rows,
+                                               None if packing is None else ctypes.byref(packing), _ptr(out), _code(out), tile, ctypes.c_long(tiles),
+                                               hidden, width, 0, _ptr(groups), parts, self._stream(h)))
+        return out, parts
+
+    def experts_sorted(self, h, w_gate_up, w_down, weights, chosen, width, out, activation: str = "silu", clamp=None, weigh_input=False,
+                       shared_width=0, shared_logits=None):
         """out[t] (float32) = sum over the experts e that token t chose, in the order of `chosen`, of weights[t, e] *
         W_down_e (act(W_gate_e h_t) * (W_up_e h_t)): the picks are sorted by expert, every expert multiplies its own rows, and
         the outputs go back to their tokens. A token's result does not depend on what else the step holds.
         clamp = (limit, alpha): the experts are clamped ones (`glu_clamped`) whose gate and up rows lie stacked expert after
-        expert in a plain matrix; their product keeps float32 sums, and the clamps and the activation are a pass of their own."""
+        expert in a plain matrix; their product keeps float32 sums, and the clamps and the activation are a pass of their own.
+        weigh_input: the weight multiplies the row that the expert reads instead of its output. shared_width: both matrices hold a
+        shared expert's rows and columns behind the others'; it runs for every token and is added, times sigmoid(shared_logits[t])
+        if those are given."""
         tokens, hidden = h.shape
         experts, top = weights.shape[1], chosen.shape[1]
-        matrices = self._expert_matrices(w_gate_up, w_down, experts, width, stacked=clamp is not None)
+        matrices = self._expert_matrices(w_gate_up, w_down, experts, width, stacked=clamp is not None, shared_width=shared_width)
         if matrices is None:
             raise KernelError("experts_sorted: the experts' matrices do not lie expert after expert")
         (up, up_packing, up_stride, up_rows), (down, down_packing, down_stride, down_rows) = matrices
@@ -1228,6 +1364,7 @@ class HipOps:
         self._require(weights, "experts_sorted weights", torch.float32, (tokens, experts), h)
         self._require(chosen, "experts_sorted chosen", torch.int32, (tokens, top), h)
         self._require(out, "experts_sorted out", torch.float32, (tokens, hidden), h)
+        logits, logits_stride = self._shared_logits(shared_logits, tokens, h)
         h_stride = self._rows(h, "experts_sorted h", hidden)
         stream, tile = self._stream(h), self.group_tile(tokens, top, experts)
         room = int(self.lib.xrt_experts_sort_room(ctypes.c_long(tokens), top, experts))
@@ -1236,7 +1373,8 @@ class HipOps:
         self._check(self.lib.xrt_experts_sort(_ptr(chosen), ctypes.c_long(tokens), top, experts, _ptr(rows), ctypes.c_long(room), _ptr(places),
                                               _ptr(tile_group), stream))
         gathered = self._empty((room, hidden), torch.bfloat16, h.device)
-        self._check(self.lib.xrt_gather_rows(_ptr(h), ctypes.c_long(h_stride), _ptr(rows), ctypes.c_long(room), hidden, _ptr(gathered), stream))
+        self._check(self.lib.xrt_gather_rows(_ptr(h), ctypes.c_long(h_stride), _ptr(rows), ctypes.c_long(room), hidden, _ptr(gathered),
+                                             _ptr(weights if weigh_input else None), experts, _ptr(tile_group), tile, stream))
         act = self._empty((room, width), torch.bfloat16, h.device)
         if clamp is not None:
             sums = self._empty((room, 2 * width), torch.float32, h.device)
@@ -1254,8 +1392,12 @@ class HipOps:
         self._check(self.lib.xrt_linear_groups(_ptr(act), width, _ptr(down), ctypes.c_long(down_stride), down_rows,
                                                None if down_packing is None else ctypes.byref(down_packing), _ptr(sorted_out),
                                                _code(sorted_out), tile, ctypes.c_long(room // tile), hidden, width, 0, _ptr(tile_group), parts, stream))
+        shared, shared_parts = None, 1
+        if shared_width:
+            shared, shared_parts = self._shared_expert(h, w_gate_up, matrices[1], experts * width, shared_width, activation)
         self._check(self.lib.xrt_experts_combine(_ptr(sorted_out), _ptr(places), _ptr(chosen), _ptr(weights), ctypes.c_long(tokens), top, experts,
-                                                 hidden, tile, parts, _ptr(out), stream))
+                                                 hidden, tile, parts, _ptr(out), int(not weigh_input), _ptr(shared), self.SHARED_TILE, shared_parts,
+                                                 logits, ctypes.c_long(logits_stride), stream))
 
     def scale_blocks(self, act, weights, width):
         """act[t, e * width + c] *= weights[t, e], in place."""
@@ -1265,8 +1407,9 @@ class HipOps:
         self._check(self.lib.xrt_scale_blocks(_ptr(act), _code(act), _ptr(weights), ctypes.c_long(tokens), experts, int(width),
                                               self._stream(act)))
 
-    def add_normed(self, residual, parts, eps, scale=1.0):
-        """residual += scale * sum over (x, gain) in parts of x / sqrt(mean(x^2) + eps) * gain; x float32 like residual; one or two parts."""
+    def add_normed(self, residual, parts, eps, scale=1.0, copy=None):
+        """residual += scale * sum over (x, gain) in parts of x / sqrt(mean(x^2) + eps) * gain; x float32 like residual; one or two parts.
+        copy: a tensor shaped like residual that takes the updated rows in its own element type."""
         self._require(residual, "add_normed residual", torch.float32)
         if residual.dim() != 2 or not 1 <= len(parts) <= 2:
             raise KernelError("add_normed: a residual [rows, width] and one or two parts")
@@ -1274,12 +1417,15 @@ class HipOps:
         for x, gain in parts:
             self._require(x, "add_normed x", torch.float32, (rows, width), residual)
             self._require(gain, "add_normed gain", parts[0][1].dtype, (width,), residual)
+        if copy is not None:
+            self._require(copy, "add_normed copy", None, (rows, width), residual)
         (x0, g0), (x1, g1) = parts[0], (parts[1] if len(parts) == 2 else (None, None))
         self._check(self.lib.xrt_add_normed(_ptr(residual), _ptr(x0), _ptr(g0), _ptr(x1), _ptr(g1), _code(g0), ctypes.c_long(rows), width,
-                                            ctypes.c_float(eps), ctypes.c_float(scale), self._stream(residual)))
+                                            ctypes.c_float(eps), ctypes.c_float(scale), _ptr(copy), 0 if copy is None else _code(copy),
+                                            self._stream(residual)))
 
     def activation(self, x, out, kind, params=None):
-        """out = f(x) elementwise in float32: "tanh", "silu", or "xielu" with params = (p, q) on the device."""
+        """out = f(x) elementwise in float32: "tanh", "silu", "gelu_tanh", or "xielu" with params = (p, q) on the device."""
         if kind not in UNARY:
             raise KernelError(f"activation: kind must be one of {sorted(UNARY)}")
         self._require(x, "activation x")

@@ -159,6 +159,77 @@ class SandwichBlock(Block):
         self.feed_forward_post_norm.add_to(x, y, self.residual_scale)
 
 
+class _StreamItself:
+    """What a block whose sublayers read the stream itself asks of the block before it: the stream's rows in the compute dtype."""
+    reads_stream = True
+
+    def row_scale(self):
+        return None                 # (for a block before it that could do a norm's work: there is none)
+
+
+class PostNormBlock(Block):
+    """A norm on what a sublayer adds and none before it: x += norm1(mixer(x)), then, if the block has a feed-forward,
+    x += norm2(feed_forward(x)). The sublayers read the stream itself, rounded to the compute dtype, and write their float32 output
+    aside (`forward_into`); the norm takes it from there onto the stream and writes the updated rows once more in the compute
+    dtype for whatever reads them next, across blocks too. The norms are RMS norms (`add_to(..., copy=)`). `unread`: tensors that a
+    checkpoint may carry for the block and that it does not read."""
+    passes_norms = True
+
+    def __init__(self, mixer, mixer_norm, feed_forward=None, feed_forward_norm=None, unread=()):
+        if (feed_forward is None) != (feed_forward_norm is None):
+            raise ValueError("a feed-forward and its norm come together")
+        self.mixer, self.mixer_norm, self.feed_forward, self.feed_forward_norm = mixer, mixer_norm, feed_forward, feed_forward_norm
+        self.unread = list(unread)
+
+    def parts(self):
+        return tuple(part for part in (self.mixer, self.mixer_norm, self.feed_forward, self.feed_forward_norm) if part is not None)
+
+    @property
+    def capturable(self) -> bool:
+        return all(part.capturable for part in self.parts())
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        specs: Dict[str, WeightSpec] = {}
+        for part in self.parts():
+            specs.update(part.weight_specs())
+        return specs
+
+    def ignored_names(self):
+        return self.unread + [name for part in self.parts() for name in getattr(part, "ignored_names", lambda: [])()]
+
+    def cache_needs(self) -> CacheNeeds:
+        return self.mixer.cache_needs()
+
+    def bind(self, tensors, runtime: Runtime) -> None:
+        super().bind(tensors, runtime)
+        for part in self.parts():
+            part.bind(tensors, runtime)
+
+    def first_norm(self):
+        return _StreamItself()
+
+    def forward(self, x, batch, cache, h=None, then=None):
+        """h: x in the compute dtype, if the part before has made it; then: the next block's `first_norm()`. Returns x in the compute
+        dtype if the next block reads that (None where the stream's own type is the compute dtype: the stream is read as it is)."""
+        rt = self.runtime
+        rounds = rt.dtype != torch.float32
+        if not rounds:
+            h = x
+        elif h is None:
+            h = rt.empty(x.shape)
+            rt.ops.cast(x, h)
+        wanted = rounds and getattr(then, "reads_stream", False)
+        y = rt.empty(x.shape, torch.float32)
+        self.mixer.forward_into(h, batch, cache, y)
+        after = rt.empty(x.shape) if rounds and (self.feed_forward is not None or wanted) else None
+        self.mixer_norm.add_to(x, y, copy=after)
+        if self.feed_forward is not None:
+            h, after = (after if rounds else x), (rt.empty(x.shape) if wanted else None)
+            self.feed_forward.forward_into(h, batch, y)
+            self.feed_forward_norm.add_to(x, y, copy=after)
+        return after
+
+
 class ParallelBlock(Block):
     """One norm, and both sublayers read its output: with h = norm(x), x += a * mixer(h) + b * feed_forward(h), where a and b
     are vectors over the model width (`mixer_scale`, `feed_forward_scale`: tensor names, or None for ones). The sublayers
@@ -351,5 +422,6 @@ class HyperConnectionBlock(Block):
 
 register_part("block", "hyper_connection", HyperConnectionBlock)
 register_part("block", "parallel", ParallelBlock)
+register_part("block", "post_norm", PostNormBlock)
 register_part("block", "pre_norm", PreNormBlock)
 register_part("block", "sandwich", SandwichBlock)

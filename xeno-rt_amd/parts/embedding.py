@@ -6,7 +6,7 @@ the model ties them (llama.rs:299-305, 604-613).
 """
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict, Optional, Tuple
 
 import torch
 
@@ -42,11 +42,14 @@ class Embedding(Part):
 
 
 class PositionedEmbedding(Embedding):
-    """x = E[token] + P[position]: a learnt vector for every position from 0 to max_positions - 1, added unscaled."""
+    """x = E[token] + P[position]: a learnt vector for every position from 0 to max_positions - 1, added unscaled. With `norm` =
+    (tensor name, eps) the sum goes through an RMS norm of its own: x = s / sqrt(mean(s^2) + eps) * w."""
 
     def __init__(self, prefix: str, vocab: int, hidden: int, max_positions: int, name: Optional[str] = None,
-                 positions_name: Optional[str] = None):
+                 positions_name: Optional[str] = None, norm: Optional[Tuple[str, float]] = None):
         super().__init__(prefix, vocab, hidden, name)
+        self.norm_name, self.norm_eps = (None, 0.0) if norm is None else (norm[0], float(norm[1]))
+        self.norm_weight = None
         self.max_positions = int(max_positions)
         self.positions_name = positions_name if positions_name is not None else prefix + "positions"
         self.position_table = None
@@ -54,15 +57,28 @@ class PositionedEmbedding(Embedding):
     def weight_specs(self) -> Dict[str, WeightSpec]:
         specs = super().weight_specs()
         specs[self.positions_name] = WeightSpec((self.max_positions, self.hidden))
+        if self.norm_name is not None:
+            specs[self.norm_name] = WeightSpec((self.hidden,), init="ones", kind="vector")
         return specs
 
     def bind(self, tensors, runtime: Runtime) -> None:
         super().bind(tensors, runtime)
         self.position_table = runtime.matrix(tensors[self.positions_name])
+        if self.norm_name is not None:
+            self.norm_weight = runtime.vector(tensors[self.norm_name])
+
+    def forward_copied(self, token_ids: torch.Tensor, positions: torch.Tensor, copy: Optional[torch.Tensor]) -> torch.Tensor:
+        """`forward` of an embedding with a norm; `copy`, if given, takes the same rows in its own element type."""
+        x = self.runtime.empty((token_ids.shape[0], self.hidden), torch.float32)
+        self.runtime.ops.embed_normed(self.table, token_ids, self.norm_weight, self.norm_eps, x, positions_table=self.position_table,
+                                      positions=positions, copy=copy)
+        return x
 
     def forward(self, token_ids: torch.Tensor, positions: Optional[torch.Tensor] = None) -> torch.Tensor:
         if positions is None:
             raise ValueError("an embedding with learnt positions needs the tokens' positions")
+        if self.norm_name is not None:
+            return self.forward_copied(token_ids, positions, None)
         x = super().forward(token_ids)
         self.runtime.ops.rows_add(self.position_table, positions, x)
         return x
@@ -178,8 +194,9 @@ class OutputHead(Part):
     capturable = True
 
     def __init__(self, prefix: str, vocab: int, hidden: int, tied_to: Optional[Embedding] = None, name: Optional[str] = None,
-                 softcap: Optional[float] = None):
-        """softcap: logits <- softcap * tanh(logits / softcap)."""
+                 softcap: Optional[float] = None, scale: float = 1.0):
+        """scale, softcap: logits <- logits * scale, then logits <- softcap * tanh(logits / softcap)."""
+        self.scale = float(scale)
         self.softcap = None if softcap is None else float(softcap)
         self.prefix = prefix
         self.name = name if name is not None else prefix + "weight"
@@ -209,6 +226,8 @@ class OutputHead(Part):
     def forward(self, y: torch.Tensor) -> torch.Tensor:
         logits = self.runtime.empty((y.shape[0], self.vocab), torch.float32, outlives_the_step=True)
         self.runtime.ops.linear(y, self.weight, logits)
-        if self.softcap is not None:
+        if self.scale != 1.0:
+            self.runtime.ops.softcap(logits, self.softcap, scale=self.scale)
+        elif self.softcap is not None:
             self.runtime.ops.softcap(logits, self.softcap)
         return logits

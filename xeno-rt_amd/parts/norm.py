@@ -44,9 +44,9 @@ class RMSNorm(Norm):
         self.runtime.ops.rmsnorm(x, self.weight, self.eps, out, rows=rows)
         return out
 
-    def add_to(self, residual: torch.Tensor, y: torch.Tensor, scale: float = 1.0) -> None:
-        """residual += scale * norm(y); y float32 like the residual."""
-        self.runtime.ops.add_normed(residual, [(y, self.weight)], self.eps, scale)
+    def add_to(self, residual: torch.Tensor, y: torch.Tensor, scale: float = 1.0, copy: Optional[torch.Tensor] = None) -> None:
+        """residual += scale * norm(y); y float32 like the residual. copy, if given, takes the updated rows in its own element type."""
+        self.runtime.ops.add_normed(residual, [(y, self.weight)], self.eps, scale, **({} if copy is None else {"copy": copy}))
 
 
 class LayerNorm(Norm):
