@@ -44,6 +44,13 @@ the same for the Renapel decoder (a residual stream in four copies; layers of li
 cached latent, and of softmax attention with a learnt sink and biases by distance, of which every second reads the keys and
 values of the one before it; eight clamped experts of which a token uses two after every mixer), beside the Depunex decoder,
 the library's closest (a matrix state per head, attention on the general kernel, experts), and Llama.
+
+    python bench.py --design mitunex [--size small|medium|large] [--layers N]
+
+the same for the Mitunex decoder (attention through a cached latent under a window of 512 keys in every layer, norms behind the
+sublayers; the first layer's feed-forward dense, behind the others eight experts of which a token uses two and a shared one;
+every fourth layer runs the weights of the one before it once more), beside the Renapel decoder, the library's closest
+(attention through a latent, experts), and Llama.
 """
 import argparse
 import json
@@ -193,8 +200,23 @@ def renapel_config(size, layers, max_positions):
     return {"architecture": "Renapel", "vocab": size["vocab"], "width": w, "norm": {"eps": 1e-6}, "streams": 4, "layers": out}
 
 
-DESIGN_CONFIGS = {"sozopel": sozopel_config, "ledudra": ledudra_config, "depunex": depunex_config, "renapel": renapel_config}
-DESIGN_BESIDE = {"depunex": ("sozopel", "llama"), "renapel": ("depunex", "llama")}          # the models a design is measured beside (Llama alone unless named)
+def mitunex_config(size, layers, max_positions):
+    w, d, ff = size["width"], size["head"], size["ff"]
+    latent = {"heads": w // d, "dim": d, "rot_dim": d // 2, "vdim": d, "kv_rank": 3 * d, "scale": (3 * d // 2) ** -0.5, "mask": {"size": 512},
+              "rot": {"dims": d // 2, "base": 500000.0}}
+    experts = {"kind": "moe", "expert": {"ff": ff // 2}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 2}}
+    out = []
+    for i in range(layers):
+        out.append({"type": "latent_attention", "mixer": latent, "mlp": {"kind": "dense", "ff": ff} if i == 0 else experts})
+        if i % 4 == 3:
+            out[-1]["weights_of"] = i - 1
+    return {"architecture": "Mitunex", "vocab": size["vocab"], "width": w, "max_positions": max_positions, "norm": {"eps": 1e-6},
+            "logit_scale": 2.0, "logit_softcap": 30.0, "layers": out}
+
+
+DESIGN_CONFIGS = {"sozopel": sozopel_config, "ledudra": ledudra_config, "depunex": depunex_config, "renapel": renapel_config,
+                  "mitunex": mitunex_config}
+DESIGN_BESIDE = {"depunex": ("sozopel", "llama"), "renapel": ("depunex", "llama"), "mitunex": ("renapel", "llama")}          # the models a design is measured beside (Llama alone unless named)
 
 
 def llama_config(size, layers, max_positions):

@@ -172,3 +172,21 @@ def load_folder(folder):
             begin, end = entry["data_offsets"]
             tensors[name] = torch.frombuffer(bytearray(data[begin:end]), dtype=kinds[entry["dtype"]]).reshape(entry["shape"])
     return config, tensors
+
+
+class PlainModel:
+    def __init__(self, folder):
+        self.config, self.tensors = load_folder(folder)
+
+    def logits(self, ids):
+        with torch.no_grad():
+            return logits(self.config, self.tensors, list(ids)).to(torch.float32)
+
+
+def generate_greedy(model, prompt, count):
+    ids, out = list(prompt), []
+    for _ in range(count):
+        token = int(model.logits(ids)[-1].argmax())
+        out.append(token)
+        ids.append(token)
+    return out

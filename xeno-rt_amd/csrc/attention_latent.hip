@@ -34,6 +34,8 @@ constexpr int KEY_STEPS = KEYS_MOST / 32;        // steps of 32 dims of a score 
 constexpr int VALUE_TILES = LATENT_MOST / 16;    // tiles of 16 dims of the value product
 constexpr int HEADS_A_WAVE = 16;
 constexpr int GROUP = 32;                        // keys that are multiplied together (half a cache block)
+constexpr int BATCH = 8;                         // tiles (or pairs of them) that a decode step's wavefront asks for at a time
+static_assert(VALUE_TILES % BATCH == 0, "values come in whole batches");
 constexpr int MOST_CHUNKS = XRT_WAVE;            // chunks of groups that a query's keys are cut into at most (a lane each in the merge)
 
 // the first group of keys that the query at `pos` sees, and the first key
@@ -79,25 +81,33 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __r
         const int block = min(max(table[g / 2], 0), n_blocks - 1);     // the host never hands out anything else
         const bf16* keys = k_cache + (long)block * XRT_BLOCK_TOKENS * head_dim;
         const bf16* values = v_cache + (long)block * XRT_BLOCK_TOKENS * value_dim;
-        // The tiles are asked for four steps at a time, both tiles of a step, before the products that use them (a branch
-        // per step would have every load awaited alone); steps beyond the key's size read the last tile again and multiply
-        // it with queries that are zeros.
+        // The tiles are asked for BATCH steps at a time, both tiles of a step, before the products that use them (a branch per step
+        // would have every load awaited alone; a decode step's wavefronts are few, and what they wait for is memory); steps
+        // beyond the key's size read the last tile again and multiply it with queries that are zeros.
         floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-        for (int step0 = 0; step0 < KEY_STEPS; step0 += 4) {
+        for (int step0 = 0; step0 < KEY_STEPS; step0 += BATCH) {
             if (step0 < key_steps) {
-                bf16x8 tiles[2][4];
+                bf16x8 tiles[2][BATCH];
 #pragma unroll
                 for (int t = 0; t < 2; ++t)
 #pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        tiles[t][i] = *reinterpret_cast<const bf16x8*>(keys + ((long)((half * 2 + t) * key_steps + min(step0 + i, key_steps - 1)) * XRT_WAVE + lane) * 8);
+                    for (int i = 0; i < BATCH; ++i)
+                        if (step0 + i < KEY_STEPS)
+                            tiles[t][i] = *reinterpret_cast<const bf16x8*>(keys + ((long)((half * 2 + t) * key_steps + min(step0 + i, key_steps - 1)) * XRT_WAVE + lane) * 8);
 #pragma unroll
-                for (int i = 0; i < 4; ++i)
+                for (int i = 0; i < BATCH; ++i)
 #pragma unroll
-                    for (int t = 0; t < 2; ++t) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[t][i], queries[step0 + i], s[t], 0, 0, 0);
+                    for (int t = 0; t < 2; ++t)
+                        if (step0 + i < KEY_STEPS) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tiles[t][i], queries[step0 + i], s[t], 0, 0, 0);
             }
         }
+        // the first values are on their way while the softmax is done, and later ones while those before them are multiplied
+        // (tiles beyond the value's size: the last one again, into sums that nobody reads)
+        auto value_at = [&](int u) { return *reinterpret_cast<const bf16x8*>(values + ((long)(half * value_tiles + min(u, value_tiles - 1)) * XRT_WAVE + lane) * 8); };
+        bf16x8 coming[BATCH];
+#pragma unroll
+        for (int i = 0; i < BATCH; ++i) coming[i] = value_at(i);
         // register i of tile t is the key k0 + 8 quarter + 4 t + i, for this lane's head
         float scores[8];
         float here = -INFINITY;
@@ -122,14 +132,16 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __r
         }
         const bool edge = k0 + 31 > pos;                    // what lies behind the sequence's last key is not ours: kept away from the zeros
 #pragma unroll
-        for (int u0 = 0; u0 < VALUE_TILES; u0 += 4) {
-            if (u0 < value_tiles) {                        // (tiles beyond the value's size read the last one again into sums that nobody reads)
-                bf16x8 tiles[4];
+        for (int u0 = 0; u0 < VALUE_TILES; u0 += BATCH) {
+            if (u0 < value_tiles) {
+                bf16x8 tiles[BATCH];
 #pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    tiles[i] = *reinterpret_cast<const bf16x8*>(values + ((long)(half * value_tiles + min(u0 + i, value_tiles - 1)) * XRT_WAVE + lane) * 8);
+                for (int i = 0; i < BATCH; ++i) {
+                    tiles[i] = coming[i];
+                    if (u0 + BATCH < VALUE_TILES) coming[i] = value_at(u0 + BATCH + i);
+                }
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
+                for (int i = 0; i < BATCH; ++i) {
                     if (edge) {
 #pragma unroll
                         for (int e = 0; e < 8; ++e)
@@ -171,30 +183,30 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __r
     const int pos = positions[token];
     const int mine = (pos / GROUP - first_key_of(pos, window) / GROUP) / chunk_groups + 1;      // this query's chunks
     const float* parts = partial + ((token * groups + head / HEADS_A_WAVE) * chunks) * partial_floats(value_dim) + (long)(head % HEADS_A_WAVE) * head_floats(value_dim);
-    constexpr int OWNED = LATENT_MOST / XRT_WAVE;
+    constexpr int OWNED = LATENT_MOST / XRT_WAVE, MERGED = 8;
     float acc[OWNED], top = -INFINITY, sum = 0.f;
 #pragma unroll
     for (int i = 0; i < OWNED; ++i) acc[i] = 0.f;
     // First the largest score of all chunks (lane c reads chunk c's), then every chunk's share relative to it, in the chunks'
-    // order, four chunks' loads on their way at a time (chunks beyond the sequence's read the last one again with a share of nothing).
+    // order, MERGED chunks' loads on their way at a time (chunks beyond the sequence's read the last one again with a share of nothing).
     const long stride = partial_floats(value_dim);
     const float my_top = lane < mine ? parts[(long)lane * stride + value_dim] : -INFINITY;
     top = wave_max(my_top);
     const float my_take = lane < mine ? expf(my_top - top) : 0.f;
     sum = wave_sum(lane < mine ? parts[(long)lane * stride + value_dim + 1] * my_take : 0.f);
 #pragma unroll
-    for (int c0 = 0; c0 < MOST_CHUNKS; c0 += 4) {
+    for (int c0 = 0; c0 < MOST_CHUNKS; c0 += MERGED) {
         if (c0 < mine) {
-            float loaded[4][OWNED], take[4];
+            float loaded[MERGED][OWNED], take[MERGED];
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
+            for (int j = 0; j < MERGED; ++j) {
                 const float* part = parts + (long)min(c0 + j, mine - 1) * stride;
                 take[j] = __shfl(my_take, c0 + j, XRT_WAVE);       // (0 from a lane beyond the sequence's chunks)
 #pragma unroll
                 for (int i = 0; i < OWNED; ++i) loaded[j][i] = lane + i * XRT_WAVE < value_dim ? part[lane + i * XRT_WAVE] : 0.f;
             }
 #pragma unroll
-            for (int j = 0; j < 4; ++j)
+            for (int j = 0; j < MERGED; ++j)
 #pragma unroll
                 for (int i = 0; i < OWNED; ++i) acc[i] = fmaf(loaded[j][i], take[j], acc[i]);
         }

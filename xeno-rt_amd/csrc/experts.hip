@@ -98,8 +98,9 @@ __global__ void __launch_bounds__(64) route_experts_kernel(const float* __restri
     }
 }
 
-// Sigmoid scores, one group: a wavefront a token, four experts a lane (lane, lane + 64, ...). Every round the largest score that is
-// left wins (the lowest index among equals); the same scores and the same sums, in the same order, as a thread alone.
+// Sigmoid scores, one group: a wavefront a token, four experts a lane (lane, lane + 64, ...). Every round the largest logit that is
+// left wins (the lowest index among equals): the order of the scores, which in float32 are all one from a logit of 17 on and could
+// no longer be told apart. The scores and their sums are those of a thread alone.
 constexpr int ROUTE_WAVES = 4, ROUTE_OWNED = XRT_MOST_EXPERTS / XRT_WAVE;
 
 __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_kernel(const float* __restrict__ logits, long logits_stride, long tokens,
@@ -108,35 +109,36 @@ __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_ker
     const int lane = threadIdx.x % XRT_WAVE;
     const long t = (long)blockIdx.x * ROUTE_WAVES + threadIdx.x / XRT_WAVE;
     if (t >= tokens) return;                                   // (the whole wavefront)
-    float s[ROUTE_OWNED];
+    float z[ROUTE_OWNED];
     unsigned picked = 0, open = 0;
 #pragma unroll
     for (int i = 0; i < ROUTE_OWNED; ++i) {
         const int e = lane + i * XRT_WAVE;
-        s[i] = -1.f;
+        z[i] = 0.f;
         if (e < experts) {
-            s[i] = 1.0f / (1.0f + expf(-logits[t * logits_stride + e]));
+            z[i] = logits[t * logits_stride + e];
             open |= 1u << i;
         }
     }
+    auto score = [](float logit) { return 1.0f / (1.0f + expf(-logit)); };
     float sum = 0.f;
     for (int round = 0; round < top; ++round) {
-        float best = -1.f;
+        float best = 0.f;
         int index = INT_MAX;                                   // (a lane whose experts are all taken)
 #pragma unroll
         for (int i = 0; i < ROUTE_OWNED; ++i)
-            if ((open >> i & 1) && (index == INT_MAX || s[i] > best)) { best = s[i]; index = lane + i * XRT_WAVE; }
+            if ((open >> i & 1) && (index == INT_MAX || z[i] > best)) { best = z[i]; index = lane + i * XRT_WAVE; }
 #pragma unroll
         for (int offset = XRT_WAVE / 2; offset > 0; offset >>= 1) {
             const float other = __shfl_xor(best, offset, XRT_WAVE);
             const int other_index = __shfl_xor(index, offset, XRT_WAVE);
-            // (a score that is no number loses to any that is; among such the lowest index wins, so the lanes agree either way)
+            // (a logit that is no number loses to any that is; among such the lowest index wins, so the lanes agree either way)
             const bool theirs_known = other == other, mine_known = best == best;
             const bool take = other_index != INT_MAX &&
                               (index == INT_MAX || (theirs_known && !mine_known) || (theirs_known == mine_known && (other > best || (!(best > other) && other_index < index))));
             if (take) { best = other; index = other_index; }
         }
-        sum += best;
+        sum += score(best);
 #pragma unroll
         for (int i = 0; i < ROUTE_OWNED; ++i)
             if (index == lane + i * XRT_WAVE) { open &= ~(1u << i); picked |= 1u << i; }
@@ -145,7 +147,7 @@ __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_ker
 #pragma unroll
     for (int i = 0; i < ROUTE_OWNED; ++i) {
         const int e = lane + i * XRT_WAVE;
-        if (e < experts) weights[t * experts + e] = !(picked >> i & 1) ? 0.f : (normalized ? s[i] / (sum + floor_) : s[i]) * scale;
+        if (e < experts) weights[t * experts + e] = !(picked >> i & 1) ? 0.f : (normalized ? score(z[i]) / (sum + floor_) : score(z[i])) * scale;
     }
 }
 
@@ -416,7 +418,7 @@ extern "C" int xrt_linear_groups_accepts(const void* a, int lda, const void* w, 
 }
 
 // out (rows of n, bfloat16 or float32) = for every tile t of `tile` rows (128 or 256) of a (bfloat16, rows lda apart)
-// with tile_group[t] >= 0: its rows times the matrix at w + tile_group[t] * w_stride (rows ldw apart, k of their columns
+// with tile_group[t] >= 0 (tile_group null: every tile, group 0): its rows times the matrix at w + tile_group[t] * w_stride (rows ldw apart, k of their columns
 // summed over; packed or not), mode 0, or mode 2 with an activation: act(gate) * up of a packed gated matrix of n pairs.
 // parts: 1, or (mode 0) 2: k is split in two and out holds, tile after tile, the tile's rows of the first half's sums and then
 // those of the second half's, for a reader that adds them (xrt_linear_groups_parts says which pays).
@@ -426,7 +428,7 @@ extern "C" int xrt_linear_groups(const void* a, int lda, const void* w, long w_s
                                  int tile, long tiles, int n, int k, int coded_mode, const int* tile_group, int parts, void* stream) {
     const Packing none = {};
     const int mode = coded_mode & 255, activation = coded_mode >> 8;
-    XRT_REQUIRE(a && w && out && tile_group && tiles > 0 && tiles <= 65535 && n > 0 && w_stride >= 0, "linear_groups: bad operands");
+    XRT_REQUIRE(a && w && out && tiles > 0 && tiles <= 65535 && n > 0 && w_stride >= 0, "linear_groups: bad operands");
     XRT_REQUIRE(out_dtype == XRT_F32 || out_dtype == XRT_BF16, "linear_groups: unknown dtype %d", out_dtype);
     XRT_REQUIRE(xrt_linear_groups_mfma_accepts(a, lda, w, ldw, n, k, mode, packing ? *packing : none),
                 "linear_groups: not served (n %d, k %d, rows %d and %d apart, mode %d): k in whole tiles of 64, a gated matrix packed", n, k, lda, ldw, mode);

@@ -496,7 +496,7 @@ __global__ void __launch_bounds__(8 * XRT_WAVE) gemm_grouped_kernel(
     const bf16* __restrict__ a, const bf16* __restrict__ w, long w_stride, TO* __restrict__ out, int N, int K, int lda, int ldw,
     int tiles_n, const int* __restrict__ tile_group, const Packing packing, const RowScale scale) {
     const int tile = blockIdx.z;
-    const int group = tile_group[tile];
+    const int group = tile_group == nullptr ? 0 : tile_group[tile];      // (no table: one matrix for all tiles)
     if (group < 0) return;
     // (grid rows split k among them, and gemm_tile puts row y's sums BM * N elements further on: a tile's parts lie one
     // after the other, tile after tile)

@@ -9,8 +9,8 @@
 //   xrt_latent_queries   from the queries' float32 sums, head by head [plain | part to turn]: the plain parts to rows of
 //                        their own, the turned parts to the tail of the rows that the attention kernel reads
 //   xrt_latent_prepare   both of them in one launch, for layers whose queries come straight from the layer's input
-//   xrt_linear_heads     out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k], float32 sums (steps of many rows: on the matrix cores in
-//                        bfloat16 with k in whole steps of 32, else in the order of k; steps of few: the lanes of a wavefront along k);
+//   xrt_linear_heads     out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k], float32 sums (bfloat16 with k in whole steps of 32: on the
+//                        matrix cores; else steps of many rows in the order of k, steps of few with the lanes of a wavefront along k);
 //                        with gates (float32 [t][h], any stride) times sigmoid(gates[t][h]) before it is rounded
 // A prompt that starts a sequence can have its scores as a matrix product of its own rows (all heads' queries of a stretch of
 // tokens against the prompt's cached rows, which the step has at hand): then
@@ -223,52 +223,77 @@ __global__ void __launch_bounds__(256) transpose_kernel(const T* __restrict__ sr
         if (c0 + i < cols && r0 + tx < rows) dst[(long)(c0 + i) * rows + r0 + tx] = tile[tx][i];
 }
 
-// The same product on the matrix cores, for bfloat16 steps of many rows with k in whole steps of 32: a wavefront takes 16 rows
-// and 64 outputs of one head; both operands of v_mfma_f32_16x16x32_bf16 come straight from memory, sixteen bytes a lane (a row
-// of a: 8 consecutive k of one token; a row of w: 8 consecutive k of one output), nothing passes LDS.
+// The same product on the matrix cores, for bfloat16 with k in whole steps of 32: a wavefront takes RT x 16 rows and NT x 16
+// outputs of one head; both operands of v_mfma_f32_16x16x32_bf16 come straight from memory, sixteen bytes a lane (a row of w:
+// 8 consecutive k of one output; a row of a: 8 consecutive k of one token), nothing passes LDS. The outputs are the rows of
+// the products, dealt to the tiles such that a lane ends up with 4 NT consecutive outputs of one token. A token's sums run
+// over k in one order whatever RT and NT are.
 typedef __bf16 heads_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float heads_floatx4 __attribute__((ext_vector_type(4)));
+constexpr int MFMA_WAVES = 4;
 
-__global__ void __launch_bounds__(256) linear_heads_mfma_kernel(const bf16* __restrict__ a, long a_stride, long a_head, const bf16* __restrict__ w,
-                                                               bf16* __restrict__ out, long out_stride, long out_head, long rows, int n, int k, const HeadGates gates) {
-    const int head = blockIdx.z, lane = threadIdx.x % XRT_WAVE, wave = threadIdx.x / XRT_WAVE, r = lane % 16, c = lane / 16;
-    const long row0 = (long)blockIdx.x * 64 + wave * 16;
-    if (row0 >= rows) return;                                  // (the whole wavefront)
-    const int n0 = blockIdx.y * 64;
-    const bf16* of_a = a + min(row0 + r, rows - 1) * a_stride + (long)head * a_head + c * 8;
-    const bf16* of_w[4];
+template <int RT, int NT>
+__global__ void __launch_bounds__(MFMA_WAVES * XRT_WAVE) linear_heads_mfma_kernel(const bf16* __restrict__ a, long a_stride, long a_head,
+                                                                                 const bf16* __restrict__ w, bf16* __restrict__ out, long out_stride,
+                                                                                 long out_head, long rows, int n, int k, long row_blocks, int n_blocks,
+                                                                                 bool fours, const HeadGates gates) {
+    const int head = blockIdx.y, lane = threadIdx.x % XRT_WAVE, r = lane % 16, c = lane / 16;
+    const long unit = (long)blockIdx.x * MFMA_WAVES + threadIdx.x / XRT_WAVE;
+    if (unit >= row_blocks * n_blocks) return;                 // (the whole wavefront)
+    const long row0 = unit % row_blocks * (16 * RT);           // (a workgroup's wavefronts share their outputs' rows of w)
+    const int n0 = (int)(unit / row_blocks) * (16 * NT);
+    const bf16* of_a[RT];
+    const bf16* of_w[NT];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) of_w[j] = w + ((long)head * n + min(n0 + 16 * j + r, n - 1)) * k + c * 8;
-    heads_floatx4 acc[4];
+    for (int t = 0; t < RT; ++t) of_a[t] = a + min(row0 + 16 * t + r, rows - 1) * a_stride + (long)head * a_head + c * 8;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = heads_floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+    for (int j = 0; j < NT; ++j) of_w[j] = w + ((long)head * n + min(n0 + r / 4 * (4 * NT) + 4 * j + r % 4, n - 1)) * k + c * 8;
+    heads_floatx4 acc[RT][NT];
+#pragma unroll
+    for (int t = 0; t < RT; ++t)
+#pragma unroll
+        for (int j = 0; j < NT; ++j) acc[t][j] = heads_floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll(RT * NT == 1 ? 4 : 2)
     for (int k0 = 0; k0 < k; k0 += 32) {
-        const heads_bf16x8 of_rows = *reinterpret_cast<const heads_bf16x8*>(of_a + k0);
-        heads_bf16x8 of_outputs[4];
+        heads_bf16x8 of_rows[RT], of_outputs[NT];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) of_outputs[j] = *reinterpret_cast<const heads_bf16x8*>(of_w[j] + k0);
+        for (int t = 0; t < RT; ++t) of_rows[t] = *reinterpret_cast<const heads_bf16x8*>(of_a[t] + k0);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(of_rows, of_outputs[j], acc[j], 0, 0, 0);
+        for (int j = 0; j < NT; ++j) of_outputs[j] = *reinterpret_cast<const heads_bf16x8*>(of_w[j] + k0);
+#pragma unroll
+        for (int t = 0; t < RT; ++t)
+#pragma unroll
+            for (int j = 0; j < NT; ++j) acc[t][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(of_outputs[j], of_rows[t], acc[t][j], 0, 0, 0);
     }
-    // register i of tile j is row row0 + 4 c + i, output n0 + 16 j + r
-    float gate[4];
+    // register i of tile (t, j) is output n0 + 4 NT c + 4 j + i of row row0 + 16 t + r
 #pragma unroll
-    for (int i = 0; i < 4; ++i) gate[i] = gates(min(row0 + 4 * c + i, rows - 1), head);
+    for (int t = 0; t < RT; ++t) {
+        const long row = row0 + 16 * t + r;
+        if (row >= rows) continue;
+        const float gate = gates(row, head);
+        bf16* dst = out + row * out_stride + (long)head * out_head;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+        for (int j = 0; j < NT; ++j) {
+            const int column = n0 + c * (4 * NT) + 4 * j;
+            if (fours && column + 3 < n) {
+                struct alignas(8) Four { bf16 e[4]; } four;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const long row = row0 + 4 * c + i;
-            const int column = n0 + 16 * j + r;
-            if (row < rows && column < n) out[row * out_stride + (long)head * out_head + column] = (bf16)(acc[j][i] * gate[i]);
+                for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(acc[t][j][i] * gate);
+                *reinterpret_cast<Four*>(dst + column) = four;
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (column + i < n) dst[column + i] = (bf16)(acc[t][j][i] * gate);
+            }
         }
+    }
 }
 
-// The same product for a step of few rows (a decode step): a wavefront an output column of one head, its lanes along k (a lane
+// The same product for a step of few rows (a decode step) in float32 or with other sizes: a wavefront an output column of one head, its lanes along k (a lane
 // takes sixteen bytes of the column's row of w at a time, and the same stretch of every row of a), the lanes' sums added in
 // the fixed order of the wavefront's butterfly. A row's result does not depend on the rows around it.
 constexpr int HEADS_FEW = 16, FEW_WAVES = 4;
+constexpr int HEADS_MANY = 512;                  // rows from which a wavefront takes 64 of them
 
 template <typename T>
 __global__ void __launch_bounds__(FEW_WAVES * XRT_WAVE) linear_heads_few_kernel(const T* __restrict__ a, long a_stride, long a_head,
@@ -421,6 +446,25 @@ extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const
     XRT_REQUIRE(a_head >= k && a_stride >= (heads - 1) * a_head + k && out_head >= n && out_stride >= (heads - 1) * out_head + n,
                 "linear_heads: rows %ld and %ld apart do not hold %d heads %ld and %ld apart", a_stride, out_stride, heads, a_head, out_head);
     if (rows == 0) return 0;
+    if (dtype == XRT_BF16 && k % 32 == 0 && a_stride % 8 == 0 && a_head % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0) {
+        const bool fours = out_stride % 4 == 0 && out_head % 4 == 0 && (uintptr_t)out % 8 == 0;
+        // a tile a wavefront for a step of few rows, whose wavefronts would else be few; more as the rows are more
+        const int rt = rows >= HEADS_MANY ? 4 : 1, nt = rows > HEADS_FEW ? 4 : 1;
+        const long row_blocks = (rows + 16 * rt - 1) / (16 * rt);
+        const int n_blocks = (n + 16 * nt - 1) / (16 * nt);
+        const long groups = (row_blocks * n_blocks + MFMA_WAVES - 1) / MFMA_WAVES;
+        XRT_REQUIRE(groups < (1L << 31), "linear_heads: too many tiles");
+        const dim3 grid((unsigned)groups, heads);
+#define XRT_HEADS_MFMA(RT_, NT_)                                                                                                                          \
+    linear_heads_mfma_kernel<RT_, NT_><<<grid, MFMA_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w, (bf16*)out, \
+                                                                                              out_stride, out_head, rows, n, k, row_blocks, n_blocks, fours, gates)
+        if (rt == 4) XRT_HEADS_MFMA(4, 4);
+        else if (nt == 4) XRT_HEADS_MFMA(1, 4);
+        else XRT_HEADS_MFMA(1, 1);
+#undef XRT_HEADS_MFMA
+        XRT_LAUNCH_CHECK("linear_heads");
+        return 0;
+    }
     if (rows <= HEADS_FEW) {
         const dim3 few((n + FEW_WAVES - 1) / FEW_WAVES, heads);
         if (dtype == XRT_F32)
@@ -429,14 +473,6 @@ extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const
         else
             linear_heads_few_kernel<bf16><<<few, FEW_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w,
                                                                                               (bf16*)out, out_stride, out_head, (int)rows, n, k, gates);
-        XRT_LAUNCH_CHECK("linear_heads");
-        return 0;
-    }
-    if (dtype == XRT_BF16 && k % 32 == 0 && a_stride % 8 == 0 && a_head % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0 &&
-        (rows + 63) / 64 < (1L << 31) && (n + 63) / 64 <= 65535) {
-        const dim3 tiles((unsigned)((rows + 63) / 64), (n + 63) / 64, heads);
-        linear_heads_mfma_kernel<<<tiles, 256, 0, (hipStream_t)stream>>>((const bf16*)a, a_stride, a_head, (const bf16*)w, (bf16*)out, out_stride, out_head,
-                                                                         rows, n, k, gates);
         XRT_LAUNCH_CHECK("linear_heads");
         return 0;
     }

@@ -441,6 +441,7 @@ int xrt_linear_groups_accepts(const void* a, int lda, const void* w, int ldw, in
 // parts: 1, or with plain sums 2: k in two halves whose sums lie tile after tile, [tiles][parts][tile rows][n], for
 // xrt_experts_combine to add (xrt_linear_groups_parts: which of the two pays, from the number of tiles).
 int xrt_linear_groups_parts(long tiles, int n, int k, int coded_mode);
+// tile_group null: all tiles are group 0's.
 int xrt_linear_groups(const void* a, int lda, const void* w, long w_stride, int ldw, const xrt_packing* packing, void* out, int out_dtype,
                       int tile, long tiles, int n, int k, int coded_mode, const int* tile_group, int parts, void* stream);
 int xrt_experts_combine(const float* sorted, const int* places, const int* chosen, const float* weights, long tokens, int top, int experts,
@@ -468,8 +469,8 @@ int xrt_streams_write(float* streams, int copies, const float* mix, const float*
 // queries: from float32 rows of heads x [plain (dim) | part to turn (rot_dim)] the plain parts to `plain` [tokens][heads][dim]
 // and the turned parts to full[t][h][rank ..], rows full_stride apart, heads rank + rot_dim apart.
 // linear_heads: out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k]; rows of a and out a_stride and out_stride apart, heads
-// a_head and out_head apart; all three of `dtype`, float32 sums (whose order depends on whether the step has up to 16 rows or more and on
-// the sizes, on nothing else: a row's result never depends on the rows around it); with gate_logits (float32, rows gate_stride apart, or
+// a_head and out_head apart; all three of `dtype`, float32 sums (whose order depends on the sizes and, in float32 or with k off the
+// steps of 32, on whether the step has up to 16 rows or more; on nothing else: a row's result never depends on the rows around it); with gate_logits (float32, rows gate_stride apart, or
 // null) times sigmoid(gate_logits[t][h]) before it is rounded.
 // prepare: complete and queries in one launch, from float32 rows `stride` apart of which q points at the queries and down at the
 // latents (no rows_out).

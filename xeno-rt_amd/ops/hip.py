@@ -1337,11 +1337,9 @@ class HipOps:
         self.linear_glu(h, mine, act[:tokens], activation=activation)
         out = self._empty((tiles * parts * tile, hidden), torch.float32, h.device)
         of_mine = data.data_ptr() + data.element_size() * first * (16 if packing is not None else 1)
-        groups = self._empty((tiles,), torch.int32, h.device)
-        groups.zero_()                                          # every tile multiplies the one matrix
         self._check(self.lib.xrt_linear_groups(_ptr(act), width, ctypes.c_void_p(of_mine), ctypes.c_long(0), down_rows,
                                                None if packing is None else ctypes.byref(packing), _ptr(out), _code(out), tile, ctypes.c_long(tiles),
-                                               hidden, width, 0, _ptr(groups), parts, self._stream(h)))
+                                               hidden, width, 0, None, parts, self._stream(h)))          # (no table of groups: one matrix for all tiles)
         return out, parts
 
     def experts_sorted(self, h, w_gate_up, w_down, weights, chosen, width, out, activation: str = "silu", clamp=None, weigh_input=False,
