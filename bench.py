@@ -211,7 +211,7 @@ def mitunex_config(size, layers, max_positions):
         if i % 4 == 3:
             out[-1]["weights_of"] = i - 1
     return {"architecture": "Mitunex", "vocab": size["vocab"], "width": w, "max_positions": max_positions, "norm": {"eps": 1e-6},
-            "logit_scale": 2.0, "logit_softcap": 30.0, "layers": out}
+            "logit_scale": 0.5, "logit_softcap": 50.0, "layers": out}
 
 
 DESIGN_CONFIGS = {"sozopel": sozopel_config, "ledudra": ledudra_config, "depunex": depunex_config, "renapel": renapel_config,

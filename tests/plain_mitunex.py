@@ -55,7 +55,7 @@ def turn_neighbours(part, dims, base):
 
 
 def window_mask(tokens, size):
-    """[queries, keys]: a query sees itself and the size - 1 tokens before it (size None: all before it)."""
+    """[queries, keys]: what a query sees are the `size` newest tokens up to its own, its own among them (size None: all of them)."""
     behind = torch.arange(tokens)[:, None] - torch.arange(tokens)[None, :]
     seen = behind >= 0
     return seen if size is None else seen & (behind < size)

@@ -327,7 +327,7 @@ def attend(ops, q, k, v, cuts, dtype, n_heads, dim, vdim, ahead=0, **options):
     return torch.cat(rows).double().cpu()
 
 
-MATRIX_CORE_SIZES = [(16, 128, 96), (6, 160, 128), (20, 64, 32), (5, 448, 384), (33, 96, 64), (1, 32, 32), (3, 192, 192), (7, 320, 256), (2, 576, 512), (4, 640, 512)]
+MATRIX_CORE_SIZES = [(16, 128, 96), (9, 224, 160), (20, 64, 32), (5, 448, 384), (33, 96, 64), (1, 32, 32), (3, 192, 192), (7, 320, 256), (2, 576, 512), (4, 640, 512)]
 
 
 @pytest.mark.parametrize("n_heads,dim,vdim", MATRIX_CORE_SIZES)
@@ -373,7 +373,7 @@ def test_a_prompts_scores_that_grow_along_the_keys_move_the_exponent(ops):
 
 
 @pytest.mark.parametrize("dtype,n_heads,dim,vdim", [(torch.float32, 2, 32, 16), (torch.bfloat16, 2, 128, 96), (torch.bfloat16, 18, 96, 64), (torch.bfloat16, 3, 40, 24)])
-@pytest.mark.parametrize("window", [40, 64, 65, 300])
+@pytest.mark.parametrize("window", [41, 64, 65, 300])
 def test_a_key_just_inside_a_window_is_found_and_one_just_outside_is_not(window, dtype, n_heads, dim, vdim, ops):
     """One key towers over all others: the query for which it is the window's last key reads its value, the next query does not, wherever
     the key lies in its block, in a prompt, in a portion and decoded."""
@@ -417,7 +417,7 @@ def test_heads_larger_than_the_matrix_core_kernels_take(dim, vdim, dtype, ops):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("heads,dim,rot_dim,rank", [(3, 16, 8, 24), (6, 32, 32, 128), (5, 7, 2, 9), (1, 40, 64, 96)])
+@pytest.mark.parametrize("heads,dim,rot_dim,rank", [(3, 16, 8, 24), (7, 32, 32, 96), (5, 7, 2, 9), (1, 40, 64, 96)])
 def test_one_launch_prepares_what_two_would(heads, dim, rot_dim, rank, dtype, ops):
     from xeno_rt_amd.parts.base import CacheNeeds, KVSpec
     tokens, q_width = 70, heads * (dim + rot_dim)
@@ -446,7 +446,7 @@ def test_one_launch_prepares_what_two_would(heads, dim, rot_dim, rank, dtype, op
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("tokens,heads,n,k", [(1, 3, 24, 16), (5, 6, 80, 128), (16, 2, 33, 64), (17, 2, 33, 64), (70, 5, 40, 8), (200, 1, 80, 72), (600, 3, 70, 96), (512, 2, 64, 32)])
+@pytest.mark.parametrize("tokens,heads,n,k", [(1, 3, 24, 16), (5, 7, 72, 96), (16, 2, 33, 64), (17, 2, 33, 64), (70, 5, 40, 8), (200, 1, 80, 72), (600, 3, 70, 96), (512, 2, 64, 32)])
 def test_a_heads_outputs_times_the_sigmoid_of_its_gate(tokens, heads, n, k, dtype, ops):
     generator = torch.Generator().manual_seed(n + k)
     a, w = torch.randn(tokens, heads * k, generator=generator).to(dtype), torch.randn(heads, n, k, generator=generator).to(dtype)
@@ -486,7 +486,7 @@ def test_latent_attention_alone(m, dtype, ops):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("window,sink,gate,q_rank", [(40, "sink", None, None), (None, "sink", "g", 24), (33, None, "g", 20), (None, None, None, 16), (20, "sink", "g", 12)])
+@pytest.mark.parametrize("window,sink,gate,q_rank", [(44, "sink", None, None), (None, "sink", "g", 24), (33, None, "g", 20), (None, None, None, 16), (20, "sink", "g", 12)])
 def test_the_latent_attentions_options_in_other_combinations(window, sink, gate, q_rank, dtype, ops):
     """A low rank for the queries with a window and a gate, a sink under a window, neither: the part serves other designs too."""
     from xeno_rt_amd.parts import LatentAttention
@@ -685,10 +685,10 @@ def random_configuration(seed):
         elif r.random() < 0.85:
             experts = r.randint(1, 9)
             mlp = _moe(r.choice([6, 20, 64, 128]), experts, r.randint(1, experts), r.choice([None, 7, 32, 64, 192]))
-        layers.append(_layer(r.randint(1, 20), r.choice([4, 12, 32]), r.choice([2, 16, 32, 64]), r.choice([6, 16, 36, 80]), r.choice([8, 30, 64, 96, 160]),
-                             r.choice([0.1, 0.25]), r.choice([10.0, 1e4, 1e6]), r.choice([None, 1, 5, 32, 50, 64, 90]), mlp))
+        layers.append(_layer(r.randint(1, 20), r.choice([4, 12, 32]), r.choice([2, 16, 32, 64]), r.choice([6, 16, 36, 72]), r.choice([8, 30, 64, 96, 160]),
+                             r.choice([0.1, 0.25]), r.choice([10.0, 1e4, 3e5]), r.choice([None, 1, 5, 32, 50, 64, 90]), mlp))
     return _model(r.choice([50, 97, 200]), r.choice([24, 40, 64, 96, 128]), r.choice([100, 512]), r.choice([1e-6, 1e-4]), r.choice([0.5, 1.0, 3.0]),
-                  r.choice([5.0, 30.0]), layers)
+                  r.choice([5.0, 20.0]), layers)
 
 
 @pytest.mark.parametrize("seed", range(12))

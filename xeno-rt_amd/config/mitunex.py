@@ -1,7 +1,7 @@
 """Configuration of the Mitunex decoder: layers of windowed attention through a latent, each before a feed-forward, a mixture of
 experts or nothing, some of which run another layer's weights.
 
-config.json names the design under `architecture` and lists the layers; each entry gives `type` (`latent_attention`), the mixer's
+config.json names the design under `architecture`; every entry of its `layers` has a `type` (`latent_attention`), the mixer's
 sizes under `mixer` (`heads`, `dim`, `rot_dim`, `vdim`, `kv_rank`, `scale`, `rot.dims|base`, `mask.size`: the window, which may be
 absent for none), and `mlp`: `kind` "dense" with `ff`, `kind` "moe" with `expert.ff`, `router.experts|top` and `shared.ff` (absent: no
 shared expert), or null. An entry with `weights_of`: j has the same sizes as layer j and runs on its tensors. Beside the layers:

@@ -1350,7 +1350,7 @@ class HipOps:
         clamp = (limit, alpha): the experts are clamped ones (`glu_clamped`) whose gate and up rows lie stacked expert after
         expert in a plain matrix; their product keeps float32 sums, and the clamps and the activation are a pass of their own.
         weigh_input: the weight multiplies the row that the expert reads instead of its output. shared_width: both matrices hold a
-        shared expert's rows and columns behind the others'; it runs for every token and is added, times sigmoid(shared_logits[t])
+        shared expert's rows and columns behind the others'; every token's output of it joins the sum, times sigmoid(shared_logits[t])
         if those are given."""
         tokens, hidden = h.shape
         experts, top = weights.shape[1], chosen.shape[1]

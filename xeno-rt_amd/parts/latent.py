@@ -10,7 +10,7 @@ With h the mixer's input, H heads, per head d plain and r turned query/key dims 
   output    W_o on the heads' outputs side by side
 
 Options: `q_rank=None` makes the queries straight from the input, q = W_q h (no c_q); `sink=None` leaves the denominator to the keys
-alone; `window=W` lets a query see the W newest of the keys at or before it only (itself and W - 1 before it), and the cache
+alone; `window=W` lets a query see only the W newest of the keys up to its own, which is one of them, and the cache
 then keeps what a window still sees; `output_gate="g"` multiplies head i's output by sigmoid(W_g h)_i before W_o.
 
 What is cached per token is one row [c | turned key part] as the key of a single key/value head, and c as its value. The
