@@ -65,7 +65,7 @@ class KVGroup:
         self.table = torch.from_numpy(self._table)
         self.device_table = self.table.to(device)
         self._lib = load_host()
-        self._handle = self._lib.xrt_tables_new(n_blocks, max_slots, max_blocks_per_sequence, int(spec.window or 0),
+        self._handle = self._lib.xrt_tables_new(n_blocks, max_slots, max_blocks_per_sequence, int(spec.window or 0), int(spec.keep_first),
                                                 BLOCK_TOKENS, self._table.ctypes.data)
         if not self._handle:
             raise CacheError(last_error())
@@ -82,11 +82,11 @@ class KVGroup:
             self._handle = None
 
     def first_needed_block(self, length: int) -> int:
-        """Lowest logical block that a query at position >= length can still see."""
+        """Lowest logical block that a query at position >= length can still see beside the first ones that are kept."""
         return int(self._lib.xrt_tables_first_needed_block(self._handle, int(length)))
 
     def floor(self, slot: int) -> int:
-        """Lowest logical block that the sequence may still hold (a window lets go of those below)."""
+        """Lowest logical block that the sequence may still hold beside the first ones that are kept (a window lets go of those below)."""
         return int(self._lib.xrt_tables_floor(self._handle, int(slot)))
 
     def held(self, slot: int) -> List[int]:
@@ -240,9 +240,10 @@ class SequenceCache:
             raise CacheError("a cache with per-sequence state cannot be truncated")
         for group in self.groups:
             # a window has let go of the blocks below its floor: a shorter sequence that would look there again cannot be had
-            if group.spec.window is not None and group.first_needed_block(length) < group.floor(slot):
+            kept = blocks_for(group.spec.keep_first)
+            if group.spec.window is not None and max(group.first_needed_block(length), kept) < group.floor(slot):
                 raise CacheError(f"slot {slot}: cannot truncate to {length} tokens: a window of {group.spec.window} has "
-                                 f"released the keys before {group.floor(slot) * BLOCK_TOKENS}, which a query there would see")
+                                 f"released keys before {group.floor(slot) * BLOCK_TOKENS} that a query there would see")
         self.lengths[slot] = length
         for group in self.groups:
             group.shrink_to(slot, length)

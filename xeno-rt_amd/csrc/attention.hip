@@ -9,7 +9,7 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
                           const void* k_cache, const void* v_cache, const int* block_table, int table_stride,
                           int n_blocks, const int* positions, const int* slots, void* out, float scale,
                           int window, const float* distance_slopes, int sink, const float* sink_scores, long q_stride,
-                          const float* distance_bias, int bias_span, int chunk, hipStream_t s);
+                          const float* distance_bias, int bias_span, int chunk, int keep_first, float softcap, hipStream_t s);
 bool xrt_attention_decode_accepts(int head_dim);
 long xrt_attention_decode_workspace(int tokens, int n_heads, int n_kv_heads, int head_dim, int max_context);
 int xrt_attention_decode(const void* qkv, int tokens, int n_heads, int n_kv_heads, int head_dim, const void* k_cache,
@@ -66,7 +66,7 @@ extern "C" int xrt_attention(const void* qkv, int dtype, int tokens, int n_heads
         }
     }
     return xrt_attention_generic(qkv, dtype, tokens, n_heads, n_kv_heads, head_dim, head_dim, k_cache, v_cache, block_table,
-                                 table_stride, n_blocks, positions, slots, out, scale, window, distance_slopes, 0, nullptr, 0, nullptr, 0, 0, s);
+                                 table_stride, n_blocks, positions, slots, out, scale, window, distance_slopes, 0, nullptr, 0, nullptr, 0, 0, 0, 0.f, s);
 }
 
 // The general kernel asked for by name, with what only it serves: values of another width than the keys (qkv rows are
@@ -76,12 +76,13 @@ extern "C" int xrt_attention(const void* qkv, int dtype, int tokens, int n_heads
 // beside them (the kernel reads keys and values from the cache alone). distance_bias: null, or float32
 // [n_heads][bias_span]: a key d tokens behind the query adds distance_bias[h][min(d, bias_span - 1)] to the scaled score.
 // chunk: 0, or the size of the stretches that the positions are cut into, counted from a sequence's first token: a query sees
-// the keys of its own stretch only (those at or before it).
+// the keys of its own stretch only (those at or before it). keep_first: beside those a query sees the sequence's first keep_first keys
+// (at or before it). softcap: 0, or c > 0: a scaled score s becomes c * tanh(s / c), ahead of every bias.
 extern "C" int xrt_attention_general(const void* qkv, int dtype, int tokens, int n_heads, int n_kv_heads, int head_dim, int value_dim,
                                      const void* k_cache, const void* v_cache, const int* block_table, int table_stride, int n_blocks,
                                      const int* positions, const int* slots, void* out, float scale, int window,
                                      const float* distance_slopes, int sink, const float* sink_scores, long q_stride,
-                                     const float* distance_bias, int bias_span, int chunk, void* stream) {
+                                     const float* distance_bias, int bias_span, int chunk, int keep_first, float softcap, void* stream) {
     XRT_REQUIRE(tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0,
                 "attention: head counts %d/%d: the first must be a multiple of the second", n_heads, n_kv_heads);
     XRT_REQUIRE(head_dim > 0 && value_dim > 0, "attention: head sizes %d and %d must be positive", head_dim, value_dim);
@@ -89,10 +90,11 @@ extern "C" int xrt_attention_general(const void* qkv, int dtype, int tokens, int
     XRT_REQUIRE(qkv && k_cache && v_cache && block_table && positions && slots && out, "attention: null operand");
     XRT_REQUIRE(table_stride > 0 && n_blocks > 0 && window >= 0 && chunk >= 0, "attention: empty cache, or negative window or chunk");
     XRT_REQUIRE(sink || sink_scores == nullptr, "attention: the sink's scores without a sink");
+    XRT_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attention: %d first keys kept, a softcap of %g", keep_first, (double)softcap);
     if (tokens == 0) return 0;
     return xrt_attention_generic(qkv, dtype, tokens, n_heads, n_kv_heads, head_dim, value_dim, k_cache, v_cache, block_table,
                                  table_stride, n_blocks, positions, slots, out, scale, window, distance_slopes, sink, sink_scores, q_stride,
-                                 distance_bias, bias_span, chunk, (hipStream_t)stream);
+                                 distance_bias, bias_span, chunk, keep_first, softcap, (hipStream_t)stream);
 }
 
 // ---- the matrix-core kernel for a step of many tokens whose queries see their own stretch of positions only (xrt_hip.h)

@@ -17,6 +17,9 @@
 // A position encoding that acts on the scores instead of on q and k is served here too: with
 // distance_slopes (one float per query head) a key at position j adds slope * (j - P) to the
 // score of the query at position P, after the scale. Not in the reference's model.
+//
+// A window may keep a sequence's first keys: a query then sees its window and the keys before keep_first (of those at or before
+// it). The blocks between the two are passed over. With a softcap c a scaled score s becomes c * tanh(s / c).
 #include "cache_layout.h"
 #include "xrt_hip.h"
 
@@ -85,19 +88,22 @@ __device__ __forceinline__ void merge(Seen<OWNED>& into, const Seen<OWNED>& from
 
 // The blocks b_begin .. b_end of the sequence in `slot`, for the G queries (heads of one key/value head) whose dims lie in
 // qs[g * head_dim ..]: online softmax as in llama.rs:514-574, block by block (64 keys, lane j takes key j).
-// ps: G x 64 floats of LDS of this wavefront. slopes: of the G heads (biased).
+// ps: G x 64 floats of LDS of this wavefront. slopes: of the G heads (biased). Blocks that neither the window (keys from `first` on) nor
+// the first `kept` keys reach into are passed over.
 template <typename T, int G, int OWNED>
-__device__ __forceinline__ void attend_blocks(Seen<OWNED> (&seen)[G], int b_begin, int b_end, int first, int pos, const float* qs, float* ps,
+__device__ __forceinline__ void attend_blocks(Seen<OWNED> (&seen)[G], int b_begin, int b_end, int first, int kept, int pos, const float* qs, float* ps,
                                               const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                                               const int* __restrict__ table, int n_blocks, int n_kv_heads, int kv_head, int head_dim, int value_dim,
                                               float scale, bool biased, const float (&slopes)[G], bool whole_pieces,
-                                              const float* __restrict__ distance_bias, int bias_span, int head0) {
+                                              const float* __restrict__ distance_bias, int bias_span, int head0, float softcap) {
     const int lane = threadIdx.x % XRT_WAVE;
     for (int b = b_begin; b <= b_end; ++b) {
+        const bool in_window = b >= first / XRT_BLOCK_TOKENS, in_kept = b * XRT_BLOCK_TOKENS < kept;
+        if (!in_window && !in_kept) continue;                  // (its keys are seen by no later query either: the block may be gone)
         const int block = table[b];
         if (block < 0 || block >= n_blocks) continue;          // the host never lets this happen
         const int j = b * XRT_BLOCK_TOKENS + lane;
-        const bool valid = j >= first && j <= pos;
+        const bool valid = j <= pos && (j >= first || j < kept);
         const long head_base = ((long)block * n_kv_heads + kv_head) * XRT_BLOCK_TOKENS * head_dim;
         const long value_base = ((long)block * n_kv_heads + kv_head) * XRT_BLOCK_TOKENS * value_dim;
         float s[G];
@@ -137,6 +143,7 @@ __device__ __forceinline__ void attend_blocks(Seen<OWNED> (&seen)[G], int b_begi
 #pragma unroll
             for (int g = 0; g < G; ++g) {
                 s[g] = dot[g] * scale;
+                if (softcap > 0.f) s[g] = softcap * tanhf(s[g] / softcap);
                 if (biased) s[g] = fmaf(slopes[g], (float)(j - pos), s[g]);
                 if (distance_bias != nullptr) s[g] += distance_bias[(long)(head0 + g) * bias_span + min(pos - j, bias_span - 1)];
             }
@@ -152,8 +159,9 @@ __device__ __forceinline__ void attend_blocks(Seen<OWNED> (&seen)[G], int b_begi
             ps[g * XRT_WAVE + lane] = p;
         }
         wave_sync();
-        const int j_begin = max(0, first - b * XRT_BLOCK_TOKENS);
-        const int j_end = min(XRT_BLOCK_TOKENS - 1, pos - b * XRT_BLOCK_TOKENS);
+        // (a block that both reach into may hold keys between the two: they have a weight of nothing)
+        const int j_begin = in_kept ? 0 : max(0, first - b * XRT_BLOCK_TOKENS);
+        const int j_end = min(XRT_BLOCK_TOKENS - 1, (in_window ? pos : min(pos, kept - 1)) - b * XRT_BLOCK_TOKENS);
 #pragma unroll
         for (int i = 0; i < OWNED; ++i) {
             const int d = lane + i * XRT_WAVE;
@@ -198,7 +206,7 @@ __global__ void __launch_bounds__(WAVES * XRT_WAVE) attention_generic_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int* __restrict__ block_table,
     int table_stride, int n_blocks, const int* __restrict__ positions, const int* __restrict__ slots,
     T* __restrict__ out, float scale, int window, const float* __restrict__ distance_slopes, int sink,
-    const float* __restrict__ sink_scores, int chunk_blocks, const float* __restrict__ distance_bias, int bias_span, int stretch) {
+    const float* __restrict__ sink_scores, int chunk_blocks, const float* __restrict__ distance_bias, int bias_span, int stretch, int keep_first, float softcap) {
     __shared__ float qs[G * OWNED * XRT_WAVE];                 // [G][head_dim]
     __shared__ float ps[WAVES][G * XRT_WAVE];
     // what the wavefronts found in the chunks of a round, for the merge: two sets, used in turn (WAVES > 1)
@@ -228,19 +236,27 @@ __global__ void __launch_bounds__(WAVES * XRT_WAVE) attention_generic_kernel(
     if constexpr (WAVES > 1) __syncthreads(); else wave_sync();
     const int* table = block_table + (long)slot * table_stride;
     const int first_block = first / XRT_BLOCK_TOKENS, last_block = pos / XRT_BLOCK_TOKENS;
-    const int first_chunk = first_block / chunk_blocks, last_chunk = last_block / chunk_blocks;
+    const int window_chunk = first_block / chunk_blocks, last_chunk = last_block / chunk_blocks;
+    // The first keys that are kept come before the window's: chunks 0 .. kept_chunks - 1 (those that lie before the window's first chunk),
+    // then the window's, counted through from first_chunk on.
+    const int kept = min(keep_first, first);                   // (what the window holds itself needs no keeping)
+    const int kept_blocks = (kept + XRT_BLOCK_TOKENS - 1) / XRT_BLOCK_TOKENS;
+    const int kept_chunks = min((kept_blocks + chunk_blocks - 1) / chunk_blocks, window_chunk);
+    const int first_chunk = window_chunk - kept_chunks;
+    auto chunk_at = [&](int counted) { return counted < window_chunk ? counted - first_chunk : counted; };
 
     Seen<OWNED> all[G];
 #pragma unroll
     for (int g = 0; g < G; ++g) all[g].clear();
     if constexpr (WAVES == 1) {
-        for (int chunk = first_chunk; chunk <= last_chunk; ++chunk) {
+        for (int counted = first_chunk; counted <= last_chunk; ++counted) {
+            const int chunk = chunk_at(counted);
             Seen<OWNED> here[G];
 #pragma unroll
             for (int g = 0; g < G; ++g) here[g].clear();
-            attend_blocks<T, G, OWNED>(here, max(first_block, chunk * chunk_blocks), min(last_block, chunk * chunk_blocks + chunk_blocks - 1),
-                                       first, pos, qs, ps[0], k_cache, v_cache, table, n_blocks, n_kv_heads, kv_head, head_dim, value_dim, scale,
-                                       biased, slopes, whole_pieces, distance_bias, bias_span, head0);
+            attend_blocks<T, G, OWNED>(here, chunk * chunk_blocks, min(last_block, chunk * chunk_blocks + chunk_blocks - 1),
+                                       first, kept, pos, qs, ps[0], k_cache, v_cache, table, n_blocks, n_kv_heads, kv_head, head_dim, value_dim, scale,
+                                       biased, slopes, whole_pieces, distance_bias, bias_span, head0, softcap);
 #pragma unroll
             for (int g = 0; g < G; ++g) merge(all[g], here[g]);
         }
@@ -249,15 +265,15 @@ __global__ void __launch_bounds__(WAVES * XRT_WAVE) attention_generic_kernel(
         // round's chunks in order (each for itself: they all hold the same sums, and the first writes them in the end)
         int set = 0;
         for (int round = first_chunk; round <= last_chunk; round += WAVES, set ^= 1) {
-            const int chunk = round + wave;
+            const int counted = round + wave, chunk = chunk_at(counted);
             float* mine = round_acc + ((long)set * WAVES + wave) * G * value_dim;
-            if (chunk <= last_chunk) {
+            if (counted <= last_chunk) {
                 Seen<OWNED> here[G];
 #pragma unroll
                 for (int g = 0; g < G; ++g) here[g].clear();
-                attend_blocks<T, G, OWNED>(here, max(first_block, chunk * chunk_blocks), min(last_block, chunk * chunk_blocks + chunk_blocks - 1),
-                                           first, pos, qs, ps[wave], k_cache, v_cache, table, n_blocks, n_kv_heads, kv_head, head_dim, value_dim, scale,
-                                           biased, slopes, whole_pieces, distance_bias, bias_span, head0);
+                attend_blocks<T, G, OWNED>(here, chunk * chunk_blocks, min(last_block, chunk * chunk_blocks + chunk_blocks - 1),
+                                           first, kept, pos, qs, ps[wave], k_cache, v_cache, table, n_blocks, n_kv_heads, kv_head, head_dim, value_dim, scale,
+                                           biased, slopes, whole_pieces, distance_bias, bias_span, head0, softcap);
 #pragma unroll
                 for (int g = 0; g < G; ++g) {
 #pragma unroll
@@ -306,7 +322,7 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
                           const void* k_cache, const void* v_cache, const int* block_table, int table_stride,
                           int n_blocks, const int* positions, const int* slots, void* out, float scale,
                           int window, const float* distance_slopes, int sink, const float* sink_scores, long q_stride,
-                          const float* distance_bias, int bias_span, int stretch, hipStream_t s) {
+                          const float* distance_bias, int bias_span, int stretch, int keep_first, float softcap, hipStream_t s) {
     XRT_REQUIRE(distance_bias == nullptr || bias_span > 0, "attention: a table of biases by distance needs a distance at least");
     XRT_REQUIRE(head_dim <= LARGEST_HEAD_DIM && value_dim > 0 && value_dim <= LARGEST_VALUE_DIM, "attention: head sizes %d and %d must be at most %d and %d", head_dim,
                 value_dim, LARGEST_HEAD_DIM, LARGEST_VALUE_DIM);
@@ -336,7 +352,7 @@ int xrt_attention_generic(const void* qkv, int dtype, int tokens, int n_heads, i
 #define XRT_GENERIC(T, WAVES_, G_, OWNED_)                                                                                \
     attention_generic_kernel<T, WAVES_, G_, OWNED_><<<(unsigned)items, WAVES_ * XRT_WAVE, WAVES_ > 1 ? round_bytes : 0, s>>>( \
         (const T*)qkv, row_width, n_heads, n_kv_heads, head_dim, value_dim, (const T*)k_cache, (const T*)v_cache, block_table,       \
-        table_stride, n_blocks, positions, slots, (T*)out, scale, window, distance_slopes, sink, sink_scores, chunk_blocks, distance_bias, bias_span, stretch)
+        table_stride, n_blocks, positions, slots, (T*)out, scale, window, distance_slopes, sink, sink_scores, chunk_blocks, distance_bias, bias_span, stretch, keep_first, softcap)
 #define XRT_GENERIC_WAVES(T, G_, OWNED_) do { if (side_by_side) XRT_GENERIC(T, CHUNK_WAVES, G_, OWNED_); else XRT_GENERIC(T, 1, G_, OWNED_); } while (0)
 #define XRT_GENERIC_SETS(T)                                                                                               \
     do {                                                                                                                  \

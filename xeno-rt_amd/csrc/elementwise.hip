@@ -12,7 +12,7 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ ids,
-                             float* __restrict__ out, int hidden) {
+                             float* __restrict__ out, int hidden, float scale) {
     const long token = blockIdx.x;
     const T* row = table + (long)ids[token] * hidden;
     float* dst = out + token * hidden;
@@ -21,24 +21,24 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
             for (int i = threadIdx.x * 8; i < hidden; i += blockDim.x * 8) {
                 const bf16x8 eight = *reinterpret_cast<const bf16x8*>(row + i);
                 float4 low, high;
-                low.x = (float)eight[0]; low.y = (float)eight[1]; low.z = (float)eight[2]; low.w = (float)eight[3];
-                high.x = (float)eight[4]; high.y = (float)eight[5]; high.z = (float)eight[6]; high.w = (float)eight[7];
+                low.x = (float)eight[0] * scale; low.y = (float)eight[1] * scale; low.z = (float)eight[2] * scale; low.w = (float)eight[3] * scale;
+                high.x = (float)eight[4] * scale; high.y = (float)eight[5] * scale; high.z = (float)eight[6] * scale; high.w = (float)eight[7] * scale;
                 *reinterpret_cast<float4*>(dst + i) = low;
                 *reinterpret_cast<float4*>(dst + i + 4) = high;
             }
             return;
         }
     }
-    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(row[i]);
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(row[i]) * scale;
 }
 
 // the same from a table kept in tiles (a table that is also the output head's weight)
 __global__ void embed_packed_kernel(const bf16* __restrict__ table, const int* __restrict__ ids,
-                                    float* __restrict__ out, int hidden, const Packing packing) {
+                                    float* __restrict__ out, int hidden, const Packing packing, float scale) {
     const long token = blockIdx.x;
     const long row = packed_row(packing, ids[token]);
     float* dst = out + token * hidden;
-    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(table[packed_offset(row, i / 8 * 8, hidden) + i % 8]);
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(table[packed_offset(row, i / 8 * 8, hidden) + i % 8]) * scale;
 }
 
 template <typename T>
@@ -194,8 +194,110 @@ __global__ void __launch_bounds__(256) rmsnorm_kernel(const float* __restrict__ 
         dst[i] = finished((row[i] * inv_rms) * to_float(weight[i]), i);
 }
 
+// Two norms of the same rows that differ in their gains, a workgroup a row (the arithmetic and the order of rmsnorm_kernel's sums).
+template <typename TW, typename TO>
+__global__ void __launch_bounds__(256) rmsnorm_two_kernel(const float* __restrict__ x, const TW* __restrict__ weight_a, const TW* __restrict__ weight_b,
+                                                          float eps, TO* __restrict__ out_a, TO* __restrict__ out_b, int hidden) {
+    constexpr int CACHED = 8;
+    __shared__ float scratch[32];
+    const float* row = x + (long)blockIdx.x * hidden;
+    TO* dst_a = out_a + (long)blockIdx.x * hidden;
+    TO* dst_b = out_b + (long)blockIdx.x * hidden;
+    float sum = 0.f;
+    if (hidden % 4 == 0) {
+        const int quads = hidden / 4;
+        const float4* row4 = reinterpret_cast<const float4*>(row);
+        float4 kept[CACHED];
+#pragma unroll
+        for (int i = 0; i < CACHED; ++i) {
+            const int q = threadIdx.x + i * 256;
+            kept[i] = q < quads ? row4[q] : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+#pragma unroll
+        for (int i = 0; i < CACHED; ++i)
+            sum = fmaf(kept[i].x, kept[i].x, fmaf(kept[i].y, kept[i].y, fmaf(kept[i].z, kept[i].z, fmaf(kept[i].w, kept[i].w, sum))));
+        for (int q = threadIdx.x + CACHED * 256; q < quads; q += 256) {
+            const float4 v = row4[q];
+            sum = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, sum))));
+        }
+        const float inv_rms = 1.0f / sqrtf(block_sum(sum, scratch) / (float)hidden + eps);
+        auto emit = [&](int q, const float4& v) {
+            const Vec4<TW> a = *reinterpret_cast<const Vec4<TW>*>(weight_a + 4 * q), b = *reinterpret_cast<const Vec4<TW>*>(weight_b + 4 * q);
+            const float four[4] = {v.x * inv_rms, v.y * inv_rms, v.z * inv_rms, v.w * inv_rms};
+            Vec4<TO> of_a, of_b;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                of_a.e[e] = from_float<TO>(four[e] * to_float(a.e[e]));
+                of_b.e[e] = from_float<TO>(four[e] * to_float(b.e[e]));
+            }
+            *reinterpret_cast<Vec4<TO>*>(dst_a + 4 * q) = of_a;
+            *reinterpret_cast<Vec4<TO>*>(dst_b + 4 * q) = of_b;
+        };
+#pragma unroll
+        for (int i = 0; i < CACHED; ++i) {
+            const int q = threadIdx.x + i * 256;
+            if (q < quads) emit(q, kept[i]);
+        }
+        for (int q = threadIdx.x + CACHED * 256; q < quads; q += 256) emit(q, row4[q]);
+        return;
+    }
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) sum = fmaf(row[i], row[i], sum);
+    const float inv_rms = 1.0f / sqrtf(block_sum(sum, scratch) / (float)hidden + eps);
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+        const float v = row[i] * inv_rms;
+        dst_a[i] = from_float<TO>(v * to_float(weight_a[i]));
+        dst_b[i] = from_float<TO>(v * to_float(weight_b[i]));
+    }
+}
+
+// copy = x in another element type, then x = base; four numbers a thread where the count allows it
+template <typename TO>
+__global__ void __launch_bounds__(256) replace_rows_kernel(float* __restrict__ x, const float* __restrict__ base, TO* __restrict__ copy, long count, int step) {
+    const long i = ((long)blockIdx.x * blockDim.x + threadIdx.x) * step;
+    if (i >= count) return;
+    if (step == 4) {
+        const float4 old = *reinterpret_cast<const float4*>(x + i);
+        Vec4<TO> rounded;
+        rounded.e[0] = from_float<TO>(old.x); rounded.e[1] = from_float<TO>(old.y); rounded.e[2] = from_float<TO>(old.z); rounded.e[3] = from_float<TO>(old.w);
+        *reinterpret_cast<Vec4<TO>*>(copy + i) = rounded;
+        *reinterpret_cast<float4*>(x + i) = *reinterpret_cast<const float4*>(base + i);
+        return;
+    }
+    copy[i] = from_float<TO>(x[i]);
+    x[i] = base[i];
+}
+
+extern "C" int xrt_rmsnorm_two(const float* x, const void* weight_a, const void* weight_b, int weight_dtype, float eps, void* out_a, void* out_b,
+                               int out_dtype, int n_rows, int hidden, void* stream) {
+    XRT_REQUIRE(x && weight_a && weight_b && out_a && out_b && n_rows >= 0 && hidden > 0, "rmsnorm_two: bad operands rows=%d hidden=%d", n_rows, hidden);
+    XRT_REQUIRE((weight_dtype == XRT_F32 || weight_dtype == XRT_BF16) && (out_dtype == XRT_F32 || out_dtype == XRT_BF16),
+                "rmsnorm_two: unknown dtype weight=%d out=%d", weight_dtype, out_dtype);
+    if (n_rows == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+#define XRT_RMS(TW, TO) rmsnorm_two_kernel<TW, TO><<<n_rows, 256, 0, s>>>(x, (const TW*)weight_a, (const TW*)weight_b, eps, (TO*)out_a, (TO*)out_b, hidden)
+    if (weight_dtype == XRT_F32 && out_dtype == XRT_F32) XRT_RMS(float, float);
+    else if (weight_dtype == XRT_F32) XRT_RMS(float, bf16);
+    else if (out_dtype == XRT_F32) XRT_RMS(bf16, float);
+    else XRT_RMS(bf16, bf16);
+#undef XRT_RMS
+    XRT_LAUNCH_CHECK("rmsnorm_two");
+    return 0;
+}
+
+extern "C" int xrt_replace_rows(float* x, const float* base, void* copy, int copy_dtype, long count, void* stream) {
+    XRT_REQUIRE(x && base && copy && count >= 0 && (copy_dtype == XRT_F32 || copy_dtype == XRT_BF16), "replace_rows: bad operands");
+    if (count == 0) return 0;
+    const int step = count % 4 == 0 && ((uintptr_t)x | (uintptr_t)base | (uintptr_t)copy) % 16 == 0 ? 4 : 1;
+    const long blocks = (count / step + 255) / 256;
+    XRT_REQUIRE(blocks < (1L << 31), "replace_rows: too many elements");
+    if (copy_dtype == XRT_F32) replace_rows_kernel<float><<<(unsigned)blocks, 256, 0, (hipStream_t)stream>>>(x, base, (float*)copy, count, step);
+    else replace_rows_kernel<bf16><<<(unsigned)blocks, 256, 0, (hipStream_t)stream>>>(x, base, (bf16*)copy, count, step);
+    XRT_LAUNCH_CHECK("replace_rows");
+    return 0;
+}
+
 extern "C" int xrt_embed(const void* table, int table_dtype, const xrt_packing* packing, const int* ids, float* out, int tokens,
-                         int hidden, int vocab, void* stream) {
+                         int hidden, int vocab, float scale, void* stream) {
     XRT_REQUIRE(tokens >= 0 && hidden > 0 && vocab > 0, "embed: bad sizes tokens=%d hidden=%d vocab=%d", tokens, hidden, vocab);
     XRT_REQUIRE(table_dtype == XRT_F32 || table_dtype == XRT_BF16, "embed: unknown dtype %d", table_dtype);
     if (tokens == 0) return 0;
@@ -203,14 +305,14 @@ extern "C" int xrt_embed(const void* table, int table_dtype, const xrt_packing* 
     if (packing && is_packed(*packing)) {
         XRT_REQUIRE(packing->kind == XRT_PACK_TILES && table_dtype == XRT_BF16 && hidden % 32 == 0,
                     "embed: a packed table is bfloat16 in plain tiles with a width that is a multiple of 32");
-        embed_packed_kernel<<<tokens, 256, 0, s>>>((const bf16*)table, ids, out, hidden, *packing);
+        embed_packed_kernel<<<tokens, 256, 0, s>>>((const bf16*)table, ids, out, hidden, *packing, scale);
         XRT_LAUNCH_CHECK("embed (packed)");
         return 0;
     }
     if (table_dtype == XRT_F32)
-        embed_kernel<float><<<tokens, 256, 0, s>>>((const float*)table, ids, out, hidden);
+        embed_kernel<float><<<tokens, 256, 0, s>>>((const float*)table, ids, out, hidden, scale);
     else
-        embed_kernel<bf16><<<tokens, 256, 0, s>>>((const bf16*)table, ids, out, hidden);
+        embed_kernel<bf16><<<tokens, 256, 0, s>>>((const bf16*)table, ids, out, hidden, scale);
     XRT_LAUNCH_CHECK("embed");
     return 0;
 }

@@ -17,8 +17,8 @@
 //   xrt_linear_groups   such a product: every tile of rows with the matrix of its tile's expert (csrc/gemm_mfma.hip)
 //   xrt_gather_rows, xrt_experts_combine   the tokens' rows into that order (times the picks' weights, where those multiply what
 //                       the experts read), and the experts' outputs back, weighted and summed, onto the shared expert's if there is one
-// The choice: one thread a token (the experts of a token are few, up to XRT_MOST_EXPERTS), or, for sigmoid scores without groups, one
-// wavefront a token.
+// The choice: one wavefront a token, or, among groups of experts, one thread a token (the experts of a token are few, up to
+// XRT_MOST_EXPERTS).
 #include <climits>
 #include "common.h"
 #include "packing.h"
@@ -98,14 +98,15 @@ __global__ void __launch_bounds__(64) route_experts_kernel(const float* __restri
     }
 }
 
-// Sigmoid scores, one group: a wavefront a token, four experts a lane (lane, lane + 64, ...). Every round the largest logit that is
+// One group: a wavefront a token, four experts a lane (lane, lane + 64, ...). Every round the largest logit that is
 // left wins (the lowest index among equals): the order of the scores, which in float32 are all one from a logit of 17 on and could
-// no longer be told apart. The scores and their sums are those of a thread alone.
+// no longer be told apart. Sigmoid scores and their sums are those of a thread alone; softmax scores are relative to the first
+// winner's logit, the largest.
 constexpr int ROUTE_WAVES = 4, ROUTE_OWNED = XRT_MOST_EXPERTS / XRT_WAVE;
 
 __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_kernel(const float* __restrict__ logits, long logits_stride, long tokens,
                                                                                    int experts, int top, float floor_, float* __restrict__ weights,
-                                                                                   int* __restrict__ chosen, float scale, int normalized) {
+                                                                                   int* __restrict__ chosen, int softmax, float scale, int normalized) {
     const int lane = threadIdx.x % XRT_WAVE;
     const long t = (long)blockIdx.x * ROUTE_WAVES + threadIdx.x / XRT_WAVE;
     if (t >= tokens) return;                                   // (the whole wavefront)
@@ -120,7 +121,8 @@ __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_ker
             open |= 1u << i;
         }
     }
-    auto score = [](float logit) { return 1.0f / (1.0f + expf(-logit)); };
+    float largest = 0.f, total = 1.f;                          // (softmax: the largest logit, and the sum over all experts)
+    auto score = [&](float logit) { return softmax ? expf(logit - largest) / total : 1.0f / (1.0f + expf(-logit)); };
     float sum = 0.f;
     for (int round = 0; round < top; ++round) {
         float best = 0.f;
@@ -137,6 +139,14 @@ __global__ void __launch_bounds__(ROUTE_WAVES * XRT_WAVE) route_experts_wave_ker
             const bool take = other_index != INT_MAX &&
                               (index == INT_MAX || (theirs_known && !mine_known) || (theirs_known == mine_known && (other > best || (!(best > other) && other_index < index))));
             if (take) { best = other; index = other_index; }
+        }
+        if (softmax && round == 0) {
+            largest = best;
+            float mine = 0.f;
+#pragma unroll
+            for (int i = 0; i < ROUTE_OWNED; ++i)
+                if (lane + i * XRT_WAVE < experts) mine += expf(z[i] - largest);
+            total = wave_sum(mine);
         }
         sum += score(best);
 #pragma unroll
@@ -297,11 +307,12 @@ __global__ void __launch_bounds__(256) gather_rows_kernel(const bf16* __restrict
 // out[t][c] = sum over a token's picks, in their order, of weights[t][expert of the pick] * sorted[row of the pick][c]
 // (sorted: [tiles][parts][tile][width], the parts' sums of a row added in their order first). weigh 0: the outputs as they are. shared
 // (float32 rows that lie like sorted's in tiles and parts of their own, the tokens in their order, or null) joins the sum, times sigmoid(shared_logits[t]) (null: as it is).
+// accumulate: onto what out holds.
 __global__ void __launch_bounds__(256) experts_combine_kernel(const float* __restrict__ sorted, const int* __restrict__ places,
                                                               const int* __restrict__ chosen, const float* __restrict__ weights, int top,
                                                               int experts, int width, int tile, int parts, float* __restrict__ out, int weigh,
                                                               const float* __restrict__ shared, int shared_tile, int shared_parts,
-                                                              const float* __restrict__ shared_logits, long shared_stride) {
+                                                              const float* __restrict__ shared_logits, long shared_stride, int accumulate) {
     const long t = blockIdx.x;
     const float of_shared = shared != nullptr && shared_logits != nullptr ? 1.0f / (1.0f + expf(-shared_logits[t * shared_stride])) : 1.f;
     for (int c = threadIdx.x * 4; c < width; c += blockDim.x * 4) {
@@ -326,7 +337,12 @@ __global__ void __launch_bounds__(256) experts_combine_kernel(const float* __res
             }
             sum.x = fmaf(of_shared, v.x, sum.x); sum.y = fmaf(of_shared, v.y, sum.y); sum.z = fmaf(of_shared, v.z, sum.z); sum.w = fmaf(of_shared, v.w, sum.w);
         }
-        *reinterpret_cast<float4*>(out + t * width + c) = sum;
+        float4* dst = reinterpret_cast<float4*>(out + t * width + c);
+        if (accumulate) {
+            const float4 old = *dst;
+            sum.x += old.x; sum.y += old.y; sum.z += old.z; sum.w += old.w;
+        }
+        *dst = sum;
     }
 }
 
@@ -340,11 +356,11 @@ extern "C" int xrt_route_experts(const float* logits, long logits_stride, long t
                 "route_experts: %d experts in %d groups of which %d are kept, %d chosen: up to %d experts in equal groups, and no more "
                 "chosen than the kept groups hold", experts, groups, keep, top, XRT_MOST_EXPERTS);
     if (tokens == 0) return 0;
-    if (groups == 1 && !softmax) {
+    if (groups == 1) {
         const long blocks = (tokens + ROUTE_WAVES - 1) / ROUTE_WAVES;
         XRT_REQUIRE(blocks < (1L << 31), "route_experts: too many tokens");
         route_experts_wave_kernel<<<(unsigned)blocks, ROUTE_WAVES * XRT_WAVE, 0, (hipStream_t)stream>>>(logits, logits_stride, tokens, experts, top, floor_, weights,
-                                                                                                     chosen, scale, normalized);
+                                                                                                     chosen, softmax, scale, normalized);
         XRT_LAUNCH_CHECK("route_experts");
         return 0;
     }
@@ -450,7 +466,7 @@ extern "C" int xrt_gather_rows(const void* x, long x_stride, const int* rows, lo
 
 extern "C" int xrt_experts_combine(const float* sorted, const int* places, const int* chosen, const float* weights, long tokens, int top,
                                    int experts, int width, int tile, int parts, float* out, int weigh, const float* shared, int shared_tile,
-                                   int shared_parts, const float* shared_logits, long shared_stride, void* stream) {
+                                   int shared_parts, const float* shared_logits, long shared_stride, int accumulate, void* stream) {
     XRT_REQUIRE(shared == nullptr || (shared_tile > 0 && shared_parts >= 1 && shared_parts <= 2), "experts_combine: %d parts of the shared expert's tiles", shared_parts);
     XRT_REQUIRE((uintptr_t)shared % 16 == 0 && shared_stride >= 0, "experts_combine: the shared expert's rows lie off their sixteen bytes");
     XRT_REQUIRE(parts >= 1 && parts <= 2 && tile > 0, "experts_combine: %d parts of tiles of %d rows", parts, tile);
@@ -458,7 +474,7 @@ extern "C" int xrt_experts_combine(const float* sorted, const int* places, const
                 width % 4 == 0 && (uintptr_t)sorted % 16 == 0 && (uintptr_t)out % 16 == 0, "experts_combine: bad operands");
     experts_combine_kernel<<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(sorted, places, chosen, weights, top, experts, width,
                                                                               tile, parts, out, weigh, shared, shared_tile, shared_parts, shared_logits,
-                                                                              shared_stride);
+                                                                              shared_stride, accumulate);
     XRT_LAUNCH_CHECK("experts_combine");
     return 0;
 }

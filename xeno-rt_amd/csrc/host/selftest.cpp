@@ -34,10 +34,11 @@ int main() {
         REQUIRE(xrt_pool_n_free(pool) == 1 && xrt_pool_is_held(pool, 1) && !xrt_pool_is_held(pool, 3) && xrt_pool_check(pool) == XRT_HOST_OK);
         xrt_pool_delete(pool);
     }
-    for (int window : {0, 100, 64, 1}) {   // block tables: sequences that grow, roll back and end, with and without a window
+    const int windows[][2] = {{0, 0}, {100, 0}, {64, 0}, {1, 0}, {100, 1}, {70, 64}, {1, 65}, {200, 300}, {64, 5000}};
+    for (const auto& [window, keep_first] : windows) {     // block tables: sequences that grow, roll back and end, with and without a window, and with first tokens kept
         const int n_blocks = 24, max_slots = 6, max_blocks = 10, block_tokens = 64;
         std::vector<int32_t> table((size_t)max_slots * max_blocks, -1);
-        xrt_tables* tables = xrt_tables_new(n_blocks, max_slots, max_blocks, window, block_tokens, table.data());
+        xrt_tables* tables = xrt_tables_new(n_blocks, max_slots, max_blocks, window, keep_first, block_tokens, table.data());
         REQUIRE(tables != nullptr);
         std::vector<int> length((size_t)max_slots, -1);         // -1: the slot is free
         std::vector<int> added((size_t)max_blocks);
@@ -64,7 +65,7 @@ int main() {
                 REQUIRE(xrt_tables_release_all(tables, slot) == XRT_HOST_OK);
                 length[(size_t)slot] = -1;
             }
-            // what every sequence holds: exactly the blocks between its window's floor and its end
+            // what every sequence holds: exactly the blocks between its window's floor and its end, and its first ones that are kept
             std::vector<unsigned char> held((size_t)max_slots);
             int in_use = 0;
             for (int s = 0; s < max_slots; ++s) {
@@ -73,7 +74,7 @@ int main() {
                 const int end = (tokens + block_tokens - 1) / block_tokens;
                 for (int logical = 0; logical < max_blocks; ++logical) {
                     const bool has = table[(size_t)s * max_blocks + (size_t)logical] >= 0;
-                    const bool must = logical < end && logical >= xrt_tables_floor(tables, s);
+                    const bool must = logical < end && (logical >= xrt_tables_floor(tables, s) || logical * block_tokens < keep_first);
                     REQUIRE(has == must);
                     in_use += has;
                 }

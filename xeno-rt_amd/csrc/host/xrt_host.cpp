@@ -93,7 +93,7 @@ extern "C" int xrt_pool_check(const xrt_pool* pool) {
 // ---- block tables ---------------------------------------------------------------------------------
 
 struct xrt_tables {
-    int max_slots, max_blocks, window, block_tokens;
+    int max_slots, max_blocks, window, keep_blocks, block_tokens;
     int32_t* table;                      // the caller's
     xrt_pool* pool;
     std::vector<int> end, floor;         // per slot: logical blocks [floor, end) may be held
@@ -133,15 +133,15 @@ int drop(xrt_tables* tables, int slot, const int* logicals, int n) {
 
 }  // namespace
 
-extern "C" xrt_tables* xrt_tables_new(int n_blocks, int max_slots, int max_blocks, int window, int block_tokens, int32_t* table) {
-    if (n_blocks < 0 || max_slots <= 0 || max_blocks <= 0 || window < 0 || block_tokens <= 0 || table == nullptr) {
-        fail(XRT_HOST_ERROR, "block tables: bad sizes (%d blocks, %d slots, %d blocks a sequence, window %d, %d tokens a block)",
-             n_blocks, max_slots, max_blocks, window, block_tokens);
+extern "C" xrt_tables* xrt_tables_new(int n_blocks, int max_slots, int max_blocks, int window, int keep_first, int block_tokens, int32_t* table) {
+    if (n_blocks < 0 || max_slots <= 0 || max_blocks <= 0 || window < 0 || keep_first < 0 || block_tokens <= 0 || table == nullptr) {
+        fail(XRT_HOST_ERROR, "block tables: bad sizes (%d blocks, %d slots, %d blocks a sequence, window %d, the first %d kept, %d tokens a block)",
+             n_blocks, max_slots, max_blocks, window, keep_first, block_tokens);
         return nullptr;
     }
     xrt_pool* pool = xrt_pool_new(n_blocks, "block");
     if (pool == nullptr) return nullptr;
-    return new xrt_tables{max_slots, max_blocks, window, block_tokens, table, pool,
+    return new xrt_tables{max_slots, max_blocks, window, keep_first / block_tokens + (keep_first % block_tokens != 0), block_tokens, table, pool,
                           std::vector<int>((size_t)max_slots, 0), std::vector<int>((size_t)max_slots, 0), 0, 0};
 }
 
@@ -202,7 +202,7 @@ extern "C" int xrt_tables_shrink_to(xrt_tables* tables, int slot, int length) {
     for (int logical = tables->blocks_for(length); logical < end; ++logical)
         if (tables->at(slot, logical) >= 0) gone.push_back(logical);
     const int floor = xrt_tables_first_needed_block(tables, length);
-    for (int logical = tables->floor[(size_t)slot]; logical < std::min(floor, end); ++logical)
+    for (int logical = std::max(tables->floor[(size_t)slot], tables->keep_blocks); logical < std::min(floor, end); ++logical)
         if (tables->at(slot, logical) >= 0) gone.push_back(logical);
     tables->floor[(size_t)slot] = floor;
     return drop(tables, slot, gone.data(), (int)gone.size());

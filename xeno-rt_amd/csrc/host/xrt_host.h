@@ -30,20 +30,22 @@ int xrt_pool_check(const xrt_pool* pool);                  // every item free on
 // ---- the block tables of one group of layer calls: table[slot][logical block] -> physical block, -1 = none.
 // `table` is the caller's memory ([max_slots][max_blocks] int32, all -1 at the start) and stays the caller's:
 // the library writes it, the caller copies changed rows to the device. window 0: a sequence keeps all its
-// blocks; window W: those that a query looking at the W most recent tokens (itself included) can still see.
+// blocks; window W: those that a query looking at the W most recent tokens (itself included) can still see, and those
+// of the sequence's first keep_first tokens.
 typedef struct xrt_tables xrt_tables;
-xrt_tables* xrt_tables_new(int n_blocks, int max_slots, int max_blocks, int window, int block_tokens, int32_t* table);
+xrt_tables* xrt_tables_new(int n_blocks, int max_slots, int max_blocks, int window, int keep_first, int block_tokens, int32_t* table);
 void xrt_tables_delete(xrt_tables* tables);
 xrt_pool* xrt_tables_pool(xrt_tables* tables);             // the group's blocks (owned by the tables)
 // the blocks that tokens up to new_length need; added[0 .. *n_added) are the logical blocks acquired (room:
 // max_blocks). XRT_HOST_FULL leaves the sequence as it was.
 int xrt_tables_grow(xrt_tables* tables, int slot, int new_length, int* added, int* n_added);
 int xrt_tables_drop(xrt_tables* tables, int slot, const int* logicals, int n);
-// releases what a sequence of `length` tokens no longer needs: blocks past its end, blocks out of the window
+// releases what a sequence of `length` tokens no longer needs: blocks past its end, blocks out of the window (those of the
+// first tokens that are kept stay)
 int xrt_tables_shrink_to(xrt_tables* tables, int slot, int length);
 int xrt_tables_release_all(xrt_tables* tables, int slot);
 int xrt_tables_first_needed_block(const xrt_tables* tables, int length);
-int xrt_tables_floor(const xrt_tables* tables, int slot);  // lowest logical block the sequence may still hold
+int xrt_tables_floor(const xrt_tables* tables, int slot);  // lowest logical block the sequence may still hold beside the kept ones
 // rows [*low, *high) have changed since the last call (0, 0: none); the call forgets them
 void xrt_tables_take_changed(xrt_tables* tables, int* low, int* high);
 // no block held by two sequences or by none, free slots (per slot_held[max_slots]) hold nothing

@@ -4,14 +4,15 @@
 // (q_h . (W_h c) = (W_h^T q_h) . c); the sum of the latents under the softmax's weights is turned into the head's output by
 // the head's value matrix afterwards. Both are products with a matrix per head (xrt_linear_heads).
 //   xrt_latent_complete  from the down projection's float32 sums [latent | key part]: the latent divided by its root mean
-//                        square, times a gain; the first rot_dims of the key part turned in pairs of neighbours (2i, 2i + 1) by
-//                        position * frequencies[i]; both into the cache
+//                        square, times a gain; the first rot_dims of the key part turned in pairs of neighbours (2i, 2i + 1) or of
+//                        halves (i, i + rot_dims / 2) by position * frequencies[i], cosines and sines times a magnitude; both into the cache
 //   xrt_latent_queries   from the queries' float32 sums, head by head [plain | part to turn]: the plain parts to rows of
 //                        their own, the turned parts to the tail of the rows that the attention kernel reads
 //   xrt_latent_prepare   both of them in one launch, for layers whose queries come straight from the layer's input
 //   xrt_linear_heads     out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k], float32 sums (bfloat16 with k in whole steps of 32: on the
 //                        matrix cores; else steps of many rows in the order of k, steps of few with the lanes of a wavefront along k);
-//                        with gates (float32 [t][h], any stride) times sigmoid(gates[t][h]) before it is rounded
+//                        with gates (float32 [t][h] or [t][h][n], any stride) times sigmoid(gates[t][h]) or sigmoid(gates[t][h][n]) before
+//                        it is rounded
 // A prompt that starts a sequence can have its scores as a matrix product of its own rows (all heads' queries of a stretch of
 // tokens against the prompt's cached rows, which the step has at hand): then
 //   xrt_causal_softmax   turns the float32 scores [queries x heads][keys] into the softmax's weights over the keys at or before
@@ -27,19 +28,29 @@ __device__ __forceinline__ float small_at(const void* p, int dtype, int i) {
     return dtype == XRT_F32 ? ((const float*)p)[i] : to_float(((const bf16*)p)[i]);
 }
 
-// the element e of a part of `rot_dim` numbers whose first rot_dims turn in pairs of neighbours
-__device__ __forceinline__ float turned(const float* part, int e, int rot_dims, const float* __restrict__ frequencies, int pos) {
-    if (e >= rot_dims) return part[e];
-    float sine, cosine;
-    sincosf((float)pos * frequencies[e / 2], &sine, &cosine);
-    const float mine = part[e], other = part[e ^ 1];
-    return e % 2 == 0 ? mine * cosine - other * sine : mine * cosine + other * sine;
-}
+// How the first `dims` numbers of a part turn: in pairs of neighbours (2i, 2i + 1) or of halves (i, i + dims / 2), by position *
+// frequencies[i], cosines and sines times `magnitude`.
+struct Turn {
+    int dims, neighbours; float magnitude; const float* frequencies;
+    bool is_sound(int part) const { return dims >= 0 && dims % 2 == 0 && dims <= part && (dims == 0 || frequencies != nullptr); }
+    // the element e of a part, turned
+    __device__ __forceinline__ float operator()(const float* part, int e, int pos) const {
+        if (e >= dims) return part[e];
+        const int half = dims / 2;
+        const bool is_first = neighbours ? e % 2 == 0 : e < half;
+        float sine, cosine;
+        sincosf((float)pos * frequencies[neighbours ? e / 2 : is_first ? e : e - half], &sine, &cosine);
+        sine *= magnitude;
+        cosine *= magnitude;
+        const float mine = part[e], other = part[neighbours ? e ^ 1 : is_first ? e + half : e - half];
+        return is_first ? mine * cosine - other * sine : mine * cosine + other * sine;
+    }
+};
 
 // What becomes of a token's float32 row [latent | key part], by the whole workgroup.
 template <typename T>
-__device__ __forceinline__ void complete_row(long t, const float* __restrict__ down, long down_stride, int rank, int rot_dim, int rot_dims,
-                                             const void* __restrict__ gain, int gain_dtype, float eps, const float* __restrict__ frequencies,
+__device__ __forceinline__ void complete_row(long t, const float* __restrict__ down, long down_stride, int rank, int rot_dim, const Turn turn,
+                                             const void* __restrict__ gain, int gain_dtype, float eps,
                                              const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ k_cache,
                                              T* __restrict__ v_cache, const int* __restrict__ block_table, int table_stride, int n_blocks,
                                              T* __restrict__ rows_out) {
@@ -65,7 +76,7 @@ __device__ __forceinline__ void complete_row(long t, const float* __restrict__ d
             values[cache_value_offset(e, place, rank)] = c;
             if (rows_out != nullptr) rows_out[t * head_dim + e] = c;
         } else {
-            const T k = from_float<T>(turned(row + rank, e - rank, rot_dims, frequencies, pos));
+            const T k = from_float<T>(turn(row + rank, e - rank, pos));
             keys[cache_key_offset(place, e, head_dim)] = k;
             if (rows_out != nullptr) rows_out[t * head_dim + e] = k;
         }
@@ -73,34 +84,32 @@ __device__ __forceinline__ void complete_row(long t, const float* __restrict__ d
 }
 
 template <typename T>
-__global__ void __launch_bounds__(256) latent_complete_kernel(const float* __restrict__ down, long down_stride, int rank, int rot_dim, int rot_dims,
-                                                             const void* __restrict__ gain, int gain_dtype, float eps,
-                                                             const float* __restrict__ frequencies, const int* __restrict__ positions,
+__global__ void __launch_bounds__(256) latent_complete_kernel(const float* __restrict__ down, long down_stride, int rank, int rot_dim, const Turn turn,
+                                                             const void* __restrict__ gain, int gain_dtype, float eps, const int* __restrict__ positions,
                                                              const int* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache,
                                                              const int* __restrict__ block_table, int table_stride, int n_blocks,
                                                              T* __restrict__ rows_out) {
-    complete_row(blockIdx.x, down, down_stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies, positions, slots, k_cache, v_cache,
+    complete_row(blockIdx.x, down, down_stride, rank, rot_dim, turn, gain, gain_dtype, eps, positions, slots, k_cache, v_cache,
                  block_table, table_stride, n_blocks, rows_out);
 }
 
 // A head's query of a token, by one wavefront.
 template <typename T>
 __device__ __forceinline__ void query_row(long t, int head, int lane, const float* __restrict__ q, long q_stride, int heads, int dim, int rot_dim,
-                                          int rot_dims, const float* __restrict__ frequencies, const int* __restrict__ positions,
+                                          const Turn turn, const int* __restrict__ positions,
                                           T* __restrict__ plain, T* __restrict__ full, long full_stride, int rank) {
     const int pos = positions[t];
     const float* mine = q + t * q_stride + (long)head * (dim + rot_dim);
     for (int e = lane; e < dim; e += XRT_WAVE) plain[(t * heads + head) * dim + e] = from_float<T>(mine[e]);
     T* tail = full + t * full_stride + (long)head * (rank + rot_dim) + rank;
-    for (int e = lane; e < rot_dim; e += XRT_WAVE) tail[e] = from_float<T>(turned(mine + dim, e, rot_dims, frequencies, pos));
+    for (int e = lane; e < rot_dim; e += XRT_WAVE) tail[e] = from_float<T>(turn(mine + dim, e, pos));
 }
 
 template <typename T>
 __global__ void __launch_bounds__(XRT_WAVE) latent_queries_kernel(const float* __restrict__ q, long q_stride, int heads, int dim, int rot_dim,
-                                                                 int rot_dims, const float* __restrict__ frequencies,
-                                                                 const int* __restrict__ positions, T* __restrict__ plain, T* __restrict__ full,
+                                                                 const Turn turn, const int* __restrict__ positions, T* __restrict__ plain, T* __restrict__ full,
                                                                  long full_stride, int rank) {
-    query_row((long)blockIdx.x / heads, (int)(blockIdx.x % heads), (int)threadIdx.x, q, q_stride, heads, dim, rot_dim, rot_dims, frequencies,
+    query_row((long)blockIdx.x / heads, (int)(blockIdx.x % heads), (int)threadIdx.x, q, q_stride, heads, dim, rot_dim, turn,
               positions, plain, full, full_stride, rank);
 }
 
@@ -109,28 +118,29 @@ constexpr int PREPARE_HEADS = 256 / XRT_WAVE;
 
 template <typename T>
 __global__ void __launch_bounds__(256) latent_prepare_kernel(const float* __restrict__ q, const float* __restrict__ down, long stride, int heads,
-                                                            int dim, int rank, int rot_dim, int rot_dims, const void* __restrict__ gain,
-                                                            int gain_dtype, float eps, const float* __restrict__ frequencies,
+                                                            int dim, int rank, int rot_dim, const Turn turn, const void* __restrict__ gain,
+                                                            int gain_dtype, float eps,
                                                             const int* __restrict__ positions, const int* __restrict__ slots,
                                                             T* __restrict__ k_cache, T* __restrict__ v_cache, const int* __restrict__ block_table,
                                                             int table_stride, int n_blocks, T* __restrict__ plain, T* __restrict__ full,
                                                             long full_stride) {
     if (blockIdx.y == 0) {
-        complete_row<T>(blockIdx.x, down, stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies, positions, slots, k_cache, v_cache,
+        complete_row<T>(blockIdx.x, down, stride, rank, rot_dim, turn, gain, gain_dtype, eps, positions, slots, k_cache, v_cache,
                         block_table, table_stride, n_blocks, nullptr);
         return;
     }
     const int head = ((int)blockIdx.y - 1) * PREPARE_HEADS + (int)threadIdx.x / XRT_WAVE;
     if (head < heads)
-        query_row((long)blockIdx.x, head, (int)threadIdx.x % XRT_WAVE, q, stride, heads, dim, rot_dim, rot_dims, frequencies, positions, plain, full,
+        query_row((long)blockIdx.x, head, (int)threadIdx.x % XRT_WAVE, q, stride, heads, dim, rot_dim, turn, positions, plain, full,
                   full_stride, rank);
 }
 
-// what a head's output is multiplied by: the sigmoid of its gate, or one
+// What a head's outputs are multiplied by: the sigmoid of the head's gate (width 1), or of a gate for each of its outputs (width: as
+// many as a head has outputs), or one.
 struct HeadGates {
-    const float* logits; long stride;
-    __device__ __forceinline__ float operator()(long row, int head) const {
-        return logits == nullptr ? 1.0f : 1.0f / (1.0f + expf(-logits[row * stride + head]));
+    const float* logits; long stride; int width;
+    __device__ __forceinline__ float operator()(long row, int head, int output) const {
+        return logits == nullptr ? 1.0f : 1.0f / (1.0f + expf(-logits[row * stride + (width == 1 ? (long)head : (long)head * width + output)]));
     }
 };
 
@@ -178,7 +188,7 @@ __global__ void __launch_bounds__(256) linear_heads_kernel(const T* __restrict__
         for (int j = 0; j < 4; ++j) {
             const long r = row0 + tr * 4 + i;
             const int c = n0 + tc * 4 + j;
-            if (r < rows && c < n) out[r * out_stride + (long)head * out_head + c] = from_float<T>(acc[i][j] * gates(r, head));
+            if (r < rows && c < n) out[r * out_stride + (long)head * out_head + c] = from_float<T>(acc[i][j] * gates(r, head, c));
         }
 }
 
@@ -270,7 +280,8 @@ __global__ void __launch_bounds__(MFMA_WAVES * XRT_WAVE) linear_heads_mfma_kerne
     for (int t = 0; t < RT; ++t) {
         const long row = row0 + 16 * t + r;
         if (row >= rows) continue;
-        const float gate = gates(row, head);
+        const bool same = gates.width == 1;                    // (one gate for all outputs of the head: worked out once)
+        const float gate = same ? gates(row, head, 0) : 1.f;
         bf16* dst = out + row * out_stride + (long)head * out_head;
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
@@ -278,12 +289,12 @@ __global__ void __launch_bounds__(MFMA_WAVES * XRT_WAVE) linear_heads_mfma_kerne
             if (fours && column + 3 < n) {
                 struct alignas(8) Four { bf16 e[4]; } four;
 #pragma unroll
-                for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(acc[t][j][i] * gate);
+                for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(acc[t][j][i] * (same ? gate : gates(row, head, column + i)));
                 *reinterpret_cast<Four*>(dst + column) = four;
             } else {
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
-                    if (column + i < n) dst[column + i] = (bf16)(acc[t][j][i] * gate);
+                    if (column + i < n) dst[column + i] = (bf16)(acc[t][j][i] * (same ? gate : gates(row, head, column + i)));
             }
         }
     }
@@ -339,7 +350,7 @@ __global__ void __launch_bounds__(FEW_WAVES * XRT_WAVE) linear_heads_few_kernel(
     for (int r = 0; r < HEADS_FEW; ++r) {
         if (r < rows) {
             const float sum = wave_sum(acc[r]);
-            if (lane == 0) out[(long)r * out_stride + (long)head * out_head + column] = from_float<T>(sum * gates(r, head));
+            if (lane == 0) out[(long)r * out_stride + (long)head * out_head + column] = from_float<T>(sum * gates(r, head, column));
         }
     }
 }
@@ -368,52 +379,54 @@ extern "C" int xrt_transpose(const void* src, long src_stride, int dtype, long r
 }
 
 extern "C" int xrt_latent_complete(const float* down, long down_stride, int dtype, long tokens, int rank, int rot_dim, int rot_dims,
-                                   const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions, const int* slots,
-                                   void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks, void* rows_out,
+                                   const void* gain, int gain_dtype, float eps, const float* frequencies, int neighbours, float magnitude,
+                                   const int* positions, const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks, void* rows_out,
                                    void* stream) {
     XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "latent_complete: unknown dtype %d", dtype);
     XRT_REQUIRE(gain_dtype == XRT_F32 || gain_dtype == XRT_BF16, "latent_complete: unknown dtype %d of the gain", gain_dtype);
     XRT_REQUIRE(down && gain && positions && slots && k_cache && v_cache && block_table, "latent_complete: null operand");
     XRT_REQUIRE(tokens >= 0 && tokens < (1L << 31) && rank > 0 && rot_dim >= 0 && down_stride >= rank + rot_dim && table_stride > 0 && n_blocks > 0,
                 "latent_complete: bad sizes");
-    XRT_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= rot_dim && (rot_dims == 0 || frequencies != nullptr),
+    const Turn turn{rot_dims, neighbours, magnitude, frequencies};
+    XRT_REQUIRE(turn.is_sound(rot_dim),
                 "latent_complete: %d dims turn in pairs inside a part of %d", rot_dims, rot_dim);
     if (tokens == 0) return 0;
     if (dtype == XRT_F32)
-        latent_complete_kernel<float><<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(down, down_stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps,
-                                                                                      frequencies, positions, slots, (float*)k_cache, (float*)v_cache,
+        latent_complete_kernel<float><<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(down, down_stride, rank, rot_dim, turn, gain, gain_dtype, eps,
+                                                                                      positions, slots, (float*)k_cache, (float*)v_cache,
                                                                                       block_table, table_stride, n_blocks, (float*)rows_out);
     else
-        latent_complete_kernel<bf16><<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(down, down_stride, rank, rot_dim, rot_dims, gain, gain_dtype, eps,
-                                                                                     frequencies, positions, slots, (bf16*)k_cache, (bf16*)v_cache,
+        latent_complete_kernel<bf16><<<(unsigned)tokens, 256, 0, (hipStream_t)stream>>>(down, down_stride, rank, rot_dim, turn, gain, gain_dtype, eps,
+                                                                                     positions, slots, (bf16*)k_cache, (bf16*)v_cache,
                                                                                      block_table, table_stride, n_blocks, (bf16*)rows_out);
     XRT_LAUNCH_CHECK("latent_complete");
     return 0;
 }
 
 extern "C" int xrt_latent_queries(const float* q, long q_stride, int dtype, long tokens, int heads, int dim, int rot_dim, int rot_dims,
-                                  const float* frequencies, const int* positions, void* plain, void* full, long full_stride, int rank,
-                                  void* stream) {
+                                  const float* frequencies, int neighbours, float magnitude, const int* positions, void* plain, void* full,
+                                  long full_stride, int rank, void* stream) {
     XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "latent_queries: unknown dtype %d", dtype);
     XRT_REQUIRE(q && positions && plain && full, "latent_queries: null operand");
     XRT_REQUIRE(tokens >= 0 && heads > 0 && tokens * heads < (1L << 31) && dim > 0 && rot_dim >= 0 && rank > 0 &&
                 q_stride >= (long)heads * (dim + rot_dim) && full_stride >= (long)heads * (rank + rot_dim), "latent_queries: bad sizes");
-    XRT_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= rot_dim && (rot_dims == 0 || frequencies != nullptr),
+    const Turn turn{rot_dims, neighbours, magnitude, frequencies};
+    XRT_REQUIRE(turn.is_sound(rot_dim),
                 "latent_queries: %d dims turn in pairs inside a part of %d", rot_dims, rot_dim);
     if (tokens == 0) return 0;
     if (dtype == XRT_F32)
-        latent_queries_kernel<float><<<(unsigned)(tokens * heads), XRT_WAVE, 0, (hipStream_t)stream>>>(q, q_stride, heads, dim, rot_dim, rot_dims, frequencies,
+        latent_queries_kernel<float><<<(unsigned)(tokens * heads), XRT_WAVE, 0, (hipStream_t)stream>>>(q, q_stride, heads, dim, rot_dim, turn,
                                                                                                     positions, (float*)plain, (float*)full, full_stride, rank);
     else
-        latent_queries_kernel<bf16><<<(unsigned)(tokens * heads), XRT_WAVE, 0, (hipStream_t)stream>>>(q, q_stride, heads, dim, rot_dim, rot_dims, frequencies,
+        latent_queries_kernel<bf16><<<(unsigned)(tokens * heads), XRT_WAVE, 0, (hipStream_t)stream>>>(q, q_stride, heads, dim, rot_dim, turn,
                                                                                                    positions, (bf16*)plain, (bf16*)full, full_stride, rank);
     XRT_LAUNCH_CHECK("latent_queries");
     return 0;
 }
 
 extern "C" int xrt_latent_prepare(const float* q, const float* down, long stride, int dtype, long tokens, int heads, int dim, int rank, int rot_dim,
-                                  int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions,
-                                  const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
+                                  int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, int neighbours,
+                                  float magnitude, const int* positions, const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
                                   void* plain, void* full, long full_stride, void* stream) {
     XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "latent_prepare: unknown dtype %d", dtype);
     XRT_REQUIRE(gain_dtype == XRT_F32 || gain_dtype == XRT_BF16, "latent_prepare: unknown dtype %d of the gain", gain_dtype);
@@ -421,16 +434,17 @@ extern "C" int xrt_latent_prepare(const float* q, const float* down, long stride
     XRT_REQUIRE(tokens >= 0 && tokens < (1L << 31) && heads > 0 && heads <= 65534 && dim > 0 && rank > 0 && rot_dim >= 0 &&
                 stride >= (long)heads * (dim + rot_dim) && stride >= rank + rot_dim && full_stride >= (long)heads * (rank + rot_dim) &&
                 table_stride > 0 && n_blocks > 0, "latent_prepare: bad sizes");
-    XRT_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= rot_dim && (rot_dims == 0 || frequencies != nullptr),
+    const Turn turn{rot_dims, neighbours, magnitude, frequencies};
+    XRT_REQUIRE(turn.is_sound(rot_dim),
                 "latent_prepare: %d dims turn in pairs inside a part of %d", rot_dims, rot_dim);
     if (tokens == 0) return 0;
     const dim3 grid((unsigned)tokens, 1 + (heads + PREPARE_HEADS - 1) / PREPARE_HEADS);
     if (dtype == XRT_F32)
-        latent_prepare_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies,
+        latent_prepare_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, turn, gain, gain_dtype, eps,
                                                                             positions, slots, (float*)k_cache, (float*)v_cache, block_table, table_stride,
                                                                             n_blocks, (float*)plain, (float*)full, full_stride);
     else
-        latent_prepare_kernel<bf16><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, rot_dims, gain, gain_dtype, eps, frequencies,
+        latent_prepare_kernel<bf16><<<grid, 256, 0, (hipStream_t)stream>>>(q, down, stride, heads, dim, rank, rot_dim, turn, gain, gain_dtype, eps,
                                                                            positions, slots, (bf16*)k_cache, (bf16*)v_cache, block_table, table_stride,
                                                                            n_blocks, (bf16*)plain, (bf16*)full, full_stride);
     XRT_LAUNCH_CHECK("latent_prepare");
@@ -438,9 +452,10 @@ extern "C" int xrt_latent_prepare(const float* q, const float* down, long stride
 }
 
 extern "C" int xrt_linear_heads(const void* a, long a_stride, long a_head, const void* w, int dtype, void* out, long out_stride, long out_head,
-                                long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, void* stream) {
-    XRT_REQUIRE(gate_logits == nullptr || gate_stride >= heads, "linear_heads: rows of gates %ld apart for %d heads", gate_stride, heads);
-    const HeadGates gates{gate_logits, gate_stride};
+                                long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, int gate_width, void* stream) {
+    XRT_REQUIRE(gate_logits == nullptr || ((gate_width == 1 || gate_width == n) && gate_stride >= (long)heads * gate_width),
+                "linear_heads: rows of gates %ld apart, %d a head, for %d heads of %d outputs", gate_stride, gate_width, heads, n);
+    const HeadGates gates{gate_logits, gate_stride, gate_logits == nullptr ? 1 : gate_width};
     XRT_REQUIRE(dtype == XRT_F32 || dtype == XRT_BF16, "linear_heads: unknown dtype %d", dtype);
     XRT_REQUIRE(a && w && out && rows >= 0 && heads > 0 && heads <= 65535 && n > 0 && k > 0, "linear_heads: bad operands");
     XRT_REQUIRE(a_head >= k && a_stride >= (heads - 1) * a_head + k && out_head >= n && out_stride >= (heads - 1) * out_head + n,

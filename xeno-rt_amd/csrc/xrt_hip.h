@@ -35,9 +35,9 @@ int xrt_pack_weight(const void* w, void* packed, int rows, int K, const xrt_pack
 // whether packing pays for a matrix of these sizes (its tiles divide evenly among the compute units)
 int xrt_packing_suits(int rows, int K);
 
-// out[t, :] = table[ids[t], :] as float32
+// out[t, :] = table[ids[t], :] * scale as float32
 int xrt_embed(const void* table, int table_dtype, const xrt_packing* packing, const int* ids, float* out, int tokens,
-              int hidden, int vocab, void* stream);
+              int hidden, int vocab, float scale, void* stream);
 
 // out[i] = element i of the random-weights stream `key`: float(2 * (sum of twelve 10-bit fields of two
 // splitmix64 words) - 12 * 1023) * scale + offset, the same values as the host-side generator gives
@@ -62,6 +62,12 @@ int xrt_add(float* residual, const void* delta, int delta_dtype, long count, voi
 // out[r, :] = rmsnorm(x[rows ? rows[r] : r, :]) * weight ; x float32, out of out_dtype
 int xrt_rmsnorm(const float* x, const void* weight, int weight_dtype, float eps, void* out, int out_dtype,
                 const int* rows, int n_rows, int hidden, void* stream);
+
+// two RMS norms of the same rows that differ in their gains: out_a, out_b [n_rows][hidden]
+int xrt_rmsnorm_two(const float* x, const void* weight_a, const void* weight_b, int weight_dtype, float eps, void* out_a, void* out_b,
+                    int out_dtype, int n_rows, int hidden, void* stream);
+// copy[i] = x[i] in copy_dtype, then x[i] = base[i]
+int xrt_replace_rows(float* x, const float* base, void* copy, int copy_dtype, long count, void* stream);
 
 // xrt_rmsnorm of every row, then xrt_short_conv of the normed rows (plain, or plus the input), for a step in which row r is the
 // one new token of the sequence in slot token_slots[r] (negative: padding, the row becomes zeros): one kernel, the same bits.
@@ -283,12 +289,13 @@ int xrt_kv_store(const void* k, long k_stride, const void* v, long v_stride, int
 // values are read from the cache only). distance_bias: null, or float32 [n_heads][bias_span]: a key d tokens behind the query
 // adds distance_bias[h][min(d, bias_span - 1)] to its scaled score (any bias that is a function of head and distance and
 // stays constant from some distance on). chunk: 0, or the size of the stretches that positions are cut into from a
-// sequence's first token on; a query then sees only the keys of its own stretch (at or before it).
+// sequence's first token on; a query then sees only the keys of its own stretch (at or before it). keep_first: beside those a
+// query sees the sequence's first keep_first keys (at or before it). softcap: 0, or c > 0: a scaled score s becomes c * tanh(s / c), ahead of every bias.
 int xrt_attention_general(const void* qkv, int dtype, int tokens, int n_heads, int n_kv_heads, int head_dim, int value_dim,
                           const void* k_cache, const void* v_cache, const int* block_table, int table_stride, int n_blocks,
                           const int* positions, const int* slots, void* out, float scale, int window,
                           const float* distance_slopes, int sink, const float* sink_scores, long q_stride, const float* distance_bias,
-                          int bias_span, int chunk, void* stream);
+                          int bias_span, int chunk, int keep_first, float softcap, void* stream);
 
 // The matrix-core attention for a step that brings sequences of many tokens, with the queries alone in q (rows q_stride
 // apart; keys and values are in the cache) and, with chunk > 0, queries that see the keys of their own stretch of `chunk`
@@ -431,7 +438,7 @@ int xrt_scale_blocks(void* act, int dtype, const float* weights, long tokens, in
 // xrt_experts_combine: out[t] = sum over the picks of t, in their order, of weights[t][chosen[t][k]] * sorted[places[t][k]] (weigh 0:
 // without the weights), and with shared (float32 rows of `width` for all tokens in
 // their order, in tiles of shared_tile rows and shared_parts parts as xrt_linear_groups leaves them, or null)
-// + sigmoid(shared_logits[t * shared_stride]) * shared[t].
+// + sigmoid(shared_logits[t * shared_stride]) * shared[t] (null logits: shared[t] as it is). accumulate: onto what out holds.
 int xrt_linear_groups_tile_rows(long tokens, int top, int experts);
 long xrt_experts_sort_room(long tokens, int top, int experts);
 int xrt_experts_sort(const int* chosen, long tokens, int top, int experts, int* rows, long room, int* places, int* tile_group, void* stream);
@@ -446,7 +453,7 @@ int xrt_linear_groups(const void* a, int lda, const void* w, long w_stride, int 
                       int tile, long tiles, int n, int k, int coded_mode, const int* tile_group, int parts, void* stream);
 int xrt_experts_combine(const float* sorted, const int* places, const int* chosen, const float* weights, long tokens, int top, int experts,
                         int width, int tile, int parts, float* out, int weigh, const float* shared, int shared_tile, int shared_parts,
-                        const float* shared_logits, long shared_stride, void* stream);
+                        const float* shared_logits, long shared_stride, int accumulate, void* stream);
 
 // ---- a residual stream in several copies (csrc/streams.hip) ------------------------------------------------------------------
 // streams: float32 [tokens][copies][width]. open: every copy is the token's row of x. read: out[r] = norm(sum over the copies s
@@ -464,19 +471,20 @@ int xrt_streams_write(float* streams, int copies, const float* mix, const float*
 // ---- attention through a latent (csrc/latent.hip) ---------------------------------------------------------------------------
 // The cache of such a layer has one key/value head whose keys are [latent (rank) | turned key part (rot_dim)] and whose values
 // are the latent. complete: from float32 rows [latent | key part] (down_stride apart) the latent / rms(latent) * gain and the
-// key part with its first rot_dims turned in pairs of neighbours by position * frequencies[pair], into the cache, and, with
+// key part with its first rot_dims turned, in pairs of neighbours (or, neighbours 0, of halves i and i + rot_dims / 2), by position *
+// frequencies[pair], cosines and sines times magnitude, into the cache, and, with
 // rows_out, once more as rows [tokens][rank + rot_dim] of the cache's element type (zeros for tokens of no sequence).
 // queries: from float32 rows of heads x [plain (dim) | part to turn (rot_dim)] the plain parts to `plain` [tokens][heads][dim]
 // and the turned parts to full[t][h][rank ..], rows full_stride apart, heads rank + rot_dim apart.
 // linear_heads: out[t][h][n] = sum over k of a[t][h][k] * w[h][n][k]; rows of a and out a_stride and out_stride apart, heads
 // a_head and out_head apart; all three of `dtype`, float32 sums (whose order depends on the sizes and, in float32 or with k off the
 // steps of 32, on whether the step has up to 16 rows or more; on nothing else: a row's result never depends on the rows around it); with gate_logits (float32, rows gate_stride apart, or
-// null) times sigmoid(gate_logits[t][h]) before it is rounded.
+// null) times sigmoid(gate_logits[t][h]) before it is rounded, or, gate_width n, sigmoid(gate_logits[t][h * n + output]).
 // prepare: complete and queries in one launch, from float32 rows `stride` apart of which q points at the queries and down at the
 // latents (no rows_out).
 int xrt_latent_complete(const float* down, long down_stride, int dtype, long tokens, int rank, int rot_dim, int rot_dims,
-                        const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions, const int* slots,
-                        void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks, void* rows_out, void* stream);
+                        const void* gain, int gain_dtype, float eps, const float* frequencies, int neighbours, float magnitude,
+                        const int* positions, const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks, void* rows_out, void* stream);
 // causal_softmax: scores float32 [rows][keys], row m being the query at position first_position + m / heads of head m % heads;
 // rounded and rest (bfloat16, same shape) get the weight of every key at or before the query, exp(score * scale) over the sum
 // of those and exp(sinks[head]) (sinks float32 [heads], or null), as the rounded number and what the rounding left; 0 elsewhere.
@@ -485,32 +493,34 @@ int xrt_causal_softmax(const float* scores, long rows, long keys, int heads, int
                        void* rounded, void* rest, void* stream);
 int xrt_transpose(const void* src, long src_stride, int dtype, long rows, int cols, void* dst, void* stream);
 int xrt_latent_queries(const float* q, long q_stride, int dtype, long tokens, int heads, int dim, int rot_dim, int rot_dims,
-                       const float* frequencies, const int* positions, void* plain, void* full, long full_stride, int rank, void* stream);
+                       const float* frequencies, int neighbours, float magnitude, const int* positions, void* plain, void* full,
+                       long full_stride, int rank, void* stream);
 int xrt_latent_prepare(const float* q, const float* down, long stride, int dtype, long tokens, int heads, int dim, int rank, int rot_dim,
-                       int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, const int* positions,
-                       const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
+                       int rot_dims, const void* gain, int gain_dtype, float eps, const float* frequencies, int neighbours, float magnitude,
+                       const int* positions, const int* slots, void* k_cache, void* v_cache, const int* block_table, int table_stride, int n_blocks,
                        void* plain, void* full, long full_stride, void* stream);
 int xrt_linear_heads(const void* a, long a_stride, long a_head, const void* w, int dtype, void* out, long out_stride, long out_head,
-                     long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, void* stream);
+                     long rows, int heads, int n, int k, const float* gate_logits, long gate_stride, int gate_width, void* stream);
 
-// ---- many heads on one key/value head with large keys, on the matrix cores (csrc/attention_latent.hip) ------------------------
-// Causal attention of the step's tokens (queries alone in q, rows q_stride apart, n_heads x head_dim each) over a cache with one
-// key/value head, keys of head_dim and values of value_dim numbers (multiples of 32 up to 640 and 512: `accepts`), bfloat16; a
-// query sees the keys at or before it, of those the `window` newest (0: all); with sink_scores (float32 [n_heads], or null) the
-// softmax's denominator also holds exp(sink_scores[head]). out: rows of n_heads x value_dim. max_context: the longest sequence
-// after this step; the workspace holds `xrt_attention_latent_workspace` floats.
+// ---- heads that share key/value heads, with keys and values of any sizes in whole tiles, on the matrix cores (csrc/attention_latent.hip) ----
+// Causal attention of the step's tokens (queries alone in q, rows q_stride apart, n_heads x head_dim each) over the cache, keys of
+// head_dim and values of value_dim numbers (multiples of 32 up to 640 and 512: `accepts`), bfloat16; head h reads key/value head
+// h / (n_heads / n_kv_heads). A query sees the keys at or before it, of those, with a window, the `window` newest (0: all) and the
+// sequence's first keep_first; softcap 0, or c > 0: a scaled score s becomes c * tanh(s / c); with sink_scores (float32 [n_heads],
+// or null) the softmax's denominator also holds exp(sink_scores[head]). out: rows of n_heads x value_dim. max_context: the longest
+// sequence after this step; the workspace holds `xrt_attention_latent_workspace` floats.
 // prompts: the same for steps that bring sequences many tokens (the step's sequences as in xrt_attention; rows of q lie
 // n_heads * head_dim apart; rows of no sequence are left as they are), scale > 0.
-int xrt_attention_latent_accepts(int dtype, int n_kv_heads, int head_dim, int value_dim);
-long xrt_attention_latent_workspace(long tokens, int n_heads, int value_dim, int max_context, int window);
-int xrt_attention_latent(const void* q, long q_stride, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
+int xrt_attention_latent_accepts(int dtype, int head_dim, int value_dim);
+long xrt_attention_latent_workspace(long tokens, int n_heads, int n_kv_heads, int value_dim, int max_context, int window, int keep_first);
+int xrt_attention_latent(const void* q, long q_stride, long tokens, int n_heads, int n_kv_heads, int head_dim, int value_dim, const void* k_cache,
                          const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* positions,
-                         const int* slots, void* out, float scale, int window, const float* sink_scores, int max_context, float* workspace,
-                         long workspace_floats, void* stream);
-int xrt_attention_latent_prompts(const void* q, long tokens, int n_heads, int head_dim, int value_dim, const void* k_cache,
+                         const int* slots, void* out, float scale, float softcap, int window, int keep_first, const float* sink_scores,
+                         int max_context, float* workspace, long workspace_floats, void* stream);
+int xrt_attention_latent_prompts(const void* q, long tokens, int n_heads, int n_kv_heads, int head_dim, int value_dim, const void* k_cache,
                                  const void* v_cache, const int* block_table, int table_stride, int n_blocks, const int* seq_offsets,
-                                 const int* seq_slots, const int* seq_starts, int n_seqs, void* out, float scale, int window,
-                                 const float* sink_scores, int max_context, void* stream);
+                                 const int* seq_slots, const int* seq_starts, int n_seqs, void* out, float scale, float softcap, int window,
+                                 int keep_first, const float* sink_scores, int max_context, void* stream);
 
 #ifdef __cplusplus
 }

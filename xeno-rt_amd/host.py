@@ -51,7 +51,7 @@ def load_host() -> ctypes.CDLL:
         "xrt_pool_new": (P, [I, ctypes.c_char_p]), "xrt_pool_delete": (None, [P]),
         "xrt_pool_acquire": (I, [P, IP]), "xrt_pool_release": (I, [P, I]), "xrt_pool_size": (I, [P]),
         "xrt_pool_n_free": (I, [P]), "xrt_pool_is_held": (I, [P, I]), "xrt_pool_check": (I, [P]),
-        "xrt_tables_new": (P, [I, I, I, I, I, P]), "xrt_tables_delete": (None, [P]), "xrt_tables_pool": (P, [P]),
+        "xrt_tables_new": (P, [I, I, I, I, I, I, P]), "xrt_tables_delete": (None, [P]), "xrt_tables_pool": (P, [P]),
         "xrt_tables_grow": (I, [P, I, I, P, IP]), "xrt_tables_drop": (I, [P, I, P, I]),
         "xrt_tables_shrink_to": (I, [P, I, I]), "xrt_tables_release_all": (I, [P, I]),
         "xrt_tables_first_needed_block": (I, [P, I]), "xrt_tables_floor": (I, [P, I]),

@@ -3,7 +3,8 @@ of layer calls, final norm, output head.
 
 The schedule is a list. An entry names a layer and may name it again (the same
 weights run twice, each call with a cache entry of its own), or may read the
-cache entry of an earlier call instead of owning one.
+cache entry of an earlier call instead of owning one. Before an entry the stream may be made anew
+from what it holds and what it began with (the beginning of a pass of layers that run several times).
 """
 from __future__ import annotations
 
@@ -19,9 +20,11 @@ from ..parts.embedding import Embedding, OutputHead
 @dataclass(frozen=True)
 class LayerCall:
     """One entry of the schedule: run `layer`; keep its keys/values/state in the
-    cache entry of this call, or read (not write) the entry of call `reads_cache_of`."""
+    cache entry of this call, or read (not write) the entry of call `reads_cache_of`. enters: a pass begins with this
+    call, and the model's `entry` comes before it."""
     layer: int
     reads_cache_of: Optional[int] = None
+    enters: bool = False
 
 
 @dataclass
@@ -33,11 +36,16 @@ class ModelSpec:
     head: OutputHead
     schedule: Optional[List[LayerCall]] = None
     streams: Optional[object] = None        # a residual stream in several copies (parts/block.py: ResidualStreams), or None for one
+    entry: Optional[object] = None          # what comes before the calls that begin a pass (parts/block.py: PassEntry)
 
     def __post_init__(self):
         if self.schedule is None:
             self.schedule = [LayerCall(i) for i in range(len(self.layers))]
+        if self.entry is not None and self.streams is not None:
+            raise ValueError("passes are entered on one residual stream, not on copies of it")
         for index, call in enumerate(self.schedule):
+            if call.enters and self.entry is None:
+                raise ValueError(f"schedule entry {index} begins a pass, and the model has no entry for it")
             if not 0 <= call.layer < len(self.layers):
                 raise ValueError(f"schedule entry {index} names layer {call.layer} of {len(self.layers)}")
             if call.reads_cache_of is not None:
@@ -54,7 +62,8 @@ class ModelSpec:
                                      "whose layer keeps something else")
 
     def parts(self):
-        return [self.embedding, *self.layers, self.final_norm, self.head] + ([self.streams] if self.streams is not None else [])
+        return [self.embedding, *self.layers, self.final_norm, self.head] + ([self.streams] if self.streams is not None else []) + (
+            [self.entry] if self.entry is not None else [])
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
         specs: Dict[str, WeightSpec] = {}
@@ -105,7 +114,7 @@ class DecoderModel:
         spec = self.spec
         first = spec.layers[spec.schedule[0].layer]
         reads = first.first_norm() if getattr(first, "passes_norms", False) else None
-        return (getattr(reads, "reads_stream", False) and spec.streams is None and self.runtime.dtype != torch.float32
+        return (getattr(reads, "reads_stream", False) and spec.streams is None and not spec.schedule[0].enters and self.runtime.dtype != torch.float32
                 and getattr(spec.embedding, "norm_name", None) is not None)
 
     def forward(self, batch, cache) -> torch.Tensor:
@@ -121,13 +130,17 @@ class DecoderModel:
             x = spec.embedding.forward(batch.token_ids, batch.positions)
         if spec.streams is not None:                             # the blocks then work on the copies [tokens, copies, hidden]
             x = spec.streams.open(x)
+        opened = spec.entry.open(x) if spec.entry is not None else None      # (before any layer: the stream still is what the embedding left)
         for index, call in enumerate(spec.schedule):
             block = spec.layers[call.layer]
+            if call.enters:
+                spec.entry.forward(x, opened)
             if not getattr(block, "passes_norms", False):
                 block.forward(x, batch, cache.layer_cache(index))
                 h = None
                 continue
-            after = spec.layers[spec.schedule[index + 1].layer] if index + 1 < len(spec.schedule) else None
+            last = index + 1 == len(spec.schedule) or spec.schedule[index + 1].enters      # (what follows does not read the stream as this block leaves it)
+            after = None if last else spec.layers[spec.schedule[index + 1].layer]
             then = after.first_norm() if after is not None and getattr(after, "passes_norms", False) else None
             h = block.forward(x, batch, cache.layer_cache(index), h=h, then=then)
         if batch.n_logit_rows == 0:

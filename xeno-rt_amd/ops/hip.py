@@ -208,7 +208,7 @@ class HipOps:
                      "xrt_experts_sort", "xrt_gather_rows", "xrt_linear_groups", "xrt_linear_groups_accepts", "xrt_experts_combine",
                      "xrt_linear_groups_tile_rows", "xrt_linear_groups_parts", "xrt_streams_open", "xrt_streams_read", "xrt_streams_write",
                      "xrt_latent_complete", "xrt_latent_queries", "xrt_linear_heads", "xrt_causal_softmax", "xrt_transpose", "xrt_attention_latent",
-                     "xrt_attention_latent_accepts", "xrt_attention_latent_prompts", "xrt_latent_prepare", "xrt_glu_experts", "xrt_embed_normed"):
+                     "xrt_attention_latent_accepts", "xrt_attention_latent_prompts", "xrt_latent_prepare", "xrt_glu_experts", "xrt_embed_normed", "xrt_rmsnorm_two", "xrt_replace_rows"):
             getattr(self.lib, name).restype = ctypes.c_int
         from ..cache.allocator import BLOCK_TOKENS
         if int(self.lib.xrt_block_tokens()) != BLOCK_TOKENS:
@@ -248,7 +248,8 @@ class HipOps:
             raise KernelError(f"{what}: shape {tuple(tensor.shape)}, expected {tuple(shape)}")
 
     # -- operations ----------------------------------------------------------
-    def embed(self, table, ids, out):
+    def embed(self, table, ids, out, scale=1.0):
+        """out[t] = table[ids[t]] * scale, float32."""
         vocab, hidden = table.shape
         tokens = ids.shape[0]
         data, packing = _matrix(table)
@@ -256,7 +257,7 @@ class HipOps:
         self._require(ids, "embed ids", torch.int32, (tokens,), data)
         self._require(out, "embed out", torch.float32, (tokens, hidden), data)
         self._check(self.lib.xrt_embed(_ptr(data), _code(data), packing, _ptr(ids), _ptr(out), tokens, hidden, vocab,
-                                       self._stream(out)))
+                                       ctypes.c_float(scale), self._stream(out)))
 
     def packing_suits(self, rows: int, cols: int) -> bool:
         """Whether a bfloat16 matrix of these sizes is better kept packed."""
@@ -318,6 +319,23 @@ class HipOps:
             self._require(rows, "rmsnorm rows", torch.int32, (n_rows,), x)
         self._check(self.lib.xrt_rmsnorm(_ptr(x), _ptr(weight), _code(weight), ctypes.c_float(eps), _ptr(out),
                                          _code(out), _ptr(rows), n_rows, hidden, self._stream(x)))
+
+    def rmsnorm_two(self, x, weights, eps, outs):
+        """Two RMS norms of the rows of x (float32) that differ in their weights: outs[i] = x / sqrt(mean(x^2) + eps) * weights[i]."""
+        rows, hidden = x.shape
+        self._require(x, "rmsnorm_two x", torch.float32)
+        for weight, out in zip(weights, outs):
+            self._require(weight, "rmsnorm_two weight", weights[0].dtype, (hidden,), x)
+            self._require(out, "rmsnorm_two out", outs[0].dtype, (rows, hidden), x)
+        self._check(self.lib.xrt_rmsnorm_two(_ptr(x), _ptr(weights[0]), _ptr(weights[1]), _code(weights[0]), ctypes.c_float(eps), _ptr(outs[0]), _ptr(outs[1]),
+                                             _code(outs[0]), rows, hidden, self._stream(x)))
+
+    def replace_rows(self, x, base, copy):
+        """copy = x in copy's element type, then x = base (x and base float32, in one pass)."""
+        self._require(x, "replace_rows x", torch.float32)
+        self._require(base, "replace_rows base", torch.float32, x.shape, x)
+        self._require(copy, "replace_rows copy", None, x.shape, x)
+        self._check(self.lib.xrt_replace_rows(_ptr(x), _ptr(base), _ptr(copy), _code(copy), ctypes.c_long(x.numel()), self._stream(x)))
 
     def _linear(self, a, w, out, coded_mode, n, then_norm=None):
         mode = coded_mode & 255                 # what rides above is a gated product's activation
@@ -496,28 +514,34 @@ class HipOps:
 
     def attention(self, qkv, n_heads, n_kv_heads, head_dim, kv, batch, out, scale, window=None, distance_slopes=None,
                   finish: Optional[QkvFinish] = None, value_dim: Optional[int] = None, sink=False,
-                  distance_bias: Optional[torch.Tensor] = None, queries_alone: bool = False, chunk: Optional[int] = None):
+                  distance_bias: Optional[torch.Tensor] = None, queries_alone: bool = False, chunk: Optional[int] = None,
+                  keep_first: int = 0, softcap: Optional[float] = None):
         """Causal attention of the step's tokens over the cache. chunk: positions are cut into stretches of this many from a
         sequence's first token on, and a query sees the keys of its own stretch only. distance_slopes: float32 [n_heads], or None; a key at
         position j adds slope * (j - P) to the scaled score of the query at position P. distance_bias: float32
         [n_heads, span], or None; a key d tokens behind the query adds distance_bias[h, min(d, span - 1)]. queries_alone: the
         rows of `qkv` hold the queries only (keys and values are in the cache already). sink: True, or float32 [n_heads]: the softmax's
-        denominator has one more term, exp(0) or exp of the head's number. finish: what is still to do to
+        denominator has one more term, exp(0) or exp of the head's number. keep_first: beside its window a query sees the sequence's
+        first keep_first keys (those at or before it). softcap c: a scaled score s becomes c * tanh(s / c). finish: what is still to do to
         q, k and v (only where `attention_finishes_qkv` says so); the cache must be writable then."""
         from ..cache import BLOCK_TOKENS
+        keep_first = int(keep_first) if window else 0           # (without a window every key is seen anyway)
+        if softcap is not None and not softcap > 0:
+            raise KernelError(f"attention: a softcap must be positive, found {softcap}")
         if finish is not None:
             return self._attention_finishing(qkv, n_heads, n_kv_heads, head_dim, kv, batch, out, scale, finish)
-        if (queries_alone and sink is not True and distance_slopes is None and not window
+        if (queries_alone and sink is not True and distance_slopes is None and not window and softcap is None
                 and self._attention_stretches(qkv, n_heads, n_kv_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, chunk,
                                               distance_bias, sink if isinstance(sink, torch.Tensor) else None)):
             return None
-        if (queries_alone and n_kv_heads == 1 and sink is not True and distance_bias is None and distance_slopes is None and not chunk
-                and self._attention_one_kv_head(qkv, n_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, window,
-                                                sink if isinstance(sink, torch.Tensor) else None)):
+        if (queries_alone and sink is not True and distance_bias is None and distance_slopes is None and not chunk
+                and self._attention_tiles(qkv, n_heads, n_kv_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, window,
+                                          sink if isinstance(sink, torch.Tensor) else None, keep_first, softcap)):
             return None
-        if sink is not False or (value_dim is not None and value_dim != head_dim) or distance_bias is not None or queries_alone or chunk:
+        if (sink is not False or (value_dim is not None and value_dim != head_dim) or distance_bias is not None or queries_alone or chunk or keep_first
+                or softcap is not None):
             return self._attention_general(qkv, n_heads, n_kv_heads, head_dim, value_dim or head_dim, kv, batch, out, scale, window,
-                                           distance_slopes, sink, distance_bias, queries_alone, chunk)
+                                           distance_slopes, sink, distance_bias, queries_alone, chunk, keep_first, softcap)
         tokens = qkv.shape[0]
         width = (n_heads + 2 * n_kv_heads) * head_dim
         self._require(qkv, "qkv", None, (tokens, width))
@@ -552,18 +576,19 @@ class HipOps:
             max_count, max_context, _ptr(workspace), ctypes.c_long(workspace_floats), self._stream(qkv)))
 
     def attention_takes_latent(self, dtype, head_dim, value_dim) -> bool:
-        """Whether `attention` has matrix-core kernels for many query heads on one key/value head of these sizes."""
-        return dtype in _CODES and bool(self.lib.xrt_attention_latent_accepts(_CODES[dtype], 1, int(head_dim), int(value_dim)))
+        """Whether `attention` has matrix-core kernels for queries alone on key/value heads of these sizes."""
+        return dtype in _CODES and bool(self.lib.xrt_attention_latent_accepts(_CODES[dtype], int(head_dim), int(value_dim)))
 
     PROMPTS_FROM = 16           # new tokens of some sequence from which a step takes the kernel for prompts
 
-    def _attention_one_kv_head(self, q, n_heads, head_dim, value_dim, kv, batch, out, scale, window, sink_scores) -> bool:
-        """The matrix-core kernels for many query heads on one key/value head (the queries alone in `q`; bfloat16, key and value
+    def _attention_tiles(self, q, n_heads, n_kv_heads, head_dim, value_dim, kv, batch, out, scale, window, sink_scores, keep_first=0,
+                         softcap=None) -> bool:
+        """The matrix-core kernels for heads that share key/value heads (the queries alone in `q`; bfloat16, key and value
         sizes that are multiples of 32 up to 640 and 512): one for steps of few tokens a sequence, one for prompts. False: not
         served here, and nothing was done."""
         tokens = q.shape[0]
         max_context = int(getattr(batch, "max_context", 0) or 0)
-        if max_context <= 0 or not self.lib.xrt_attention_latent_accepts(_code(q), 1, head_dim, value_dim):
+        if max_context <= 0 or not self.lib.xrt_attention_latent_accepts(_code(q), head_dim, value_dim):
             return False
         offsets, seq_slots = getattr(batch, "sequence_offsets", None), getattr(batch, "sequence_slots", None)
         starts, counts = getattr(batch, "sequence_starts", None), getattr(batch, "host_counts", None)
@@ -575,7 +600,7 @@ class HipOps:
         if q_stride % 8 != 0 or q.data_ptr() % 16 != 0:
             return False
         self._require(out, "attention out", q.dtype, (tokens, n_heads * value_dim), q)
-        k_cache, v_cache, table, stride, n_blocks = self._kv(kv, q, 1, head_dim, value_dim)
+        k_cache, v_cache, table, stride, n_blocks = self._kv(kv, q, n_kv_heads, head_dim, value_dim)
         if sink_scores is not None:
             self._require(sink_scores, "attention sink", torch.float32, (n_heads,), q)
         if prompts:
@@ -586,18 +611,18 @@ class HipOps:
             if counts is None or sum(counts) < tokens:
                 out.zero_()                       # padding rows: written by no one, read by the product that follows
             self._check(self.lib.xrt_attention_latent_prompts(
-                _ptr(q), ctypes.c_long(tokens), n_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride, n_blocks, _ptr(offsets),
-                _ptr(seq_slots), _ptr(starts), n_seqs, _ptr(out), ctypes.c_float(scale), int(window or 0), _ptr(sink_scores), max_context,
-                self._stream(q)))
+                _ptr(q), ctypes.c_long(tokens), n_heads, n_kv_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride, n_blocks, _ptr(offsets),
+                _ptr(seq_slots), _ptr(starts), n_seqs, _ptr(out), ctypes.c_float(scale), ctypes.c_float(softcap or 0.0), int(window or 0),
+                int(keep_first), _ptr(sink_scores), max_context, self._stream(q)))
             return True
         self._require(batch.positions, "positions", torch.int32, (tokens,), q)
         self._require(batch.slots, "slots", torch.int32, (tokens,), q)
-        need = int(self.lib.xrt_attention_latent_workspace(ctypes.c_long(tokens), n_heads, value_dim, max_context, int(window or 0)))
+        need = int(self.lib.xrt_attention_latent_workspace(ctypes.c_long(tokens), n_heads, n_kv_heads, value_dim, max_context, int(window or 0), int(keep_first)))
         workspace = self._empty(need, torch.float32, q.device)
         self._check(self.lib.xrt_attention_latent(
-            _ptr(q), ctypes.c_long(q_stride), ctypes.c_long(tokens), n_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride,
-            n_blocks, _ptr(batch.positions), _ptr(batch.slots), _ptr(out), ctypes.c_float(scale), int(window or 0), _ptr(sink_scores), max_context,
-            _ptr(workspace), ctypes.c_long(need), self._stream(q)))
+            _ptr(q), ctypes.c_long(q_stride), ctypes.c_long(tokens), n_heads, n_kv_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride,
+            n_blocks, _ptr(batch.positions), _ptr(batch.slots), _ptr(out), ctypes.c_float(scale), ctypes.c_float(softcap or 0.0),
+            int(window or 0), int(keep_first), _ptr(sink_scores), max_context, _ptr(workspace), ctypes.c_long(need), self._stream(q)))
         return True
 
     def _attention_stretches(self, q, n_heads, n_kv_heads, head_dim, value_dim, kv, batch, out, scale, chunk, distance_bias=None,
@@ -641,7 +666,7 @@ class HipOps:
         return True
 
     def _attention_general(self, qkv, n_heads, n_kv_heads, head_dim, value_dim, kv, batch, out, scale, window, distance_slopes, sink,
-                           distance_bias=None, queries_alone=False, chunk=None):
+                           distance_bias=None, queries_alone=False, chunk=None, keep_first=0, softcap=None):
         """Rows of qkv are [n_heads x head_dim | n_kv_heads x head_dim | n_kv_heads x value_dim] (or the queries alone), rows of
         out n_heads x value_dim. sink: the softmax's denominator has one more (a key without a value whose score is 0 or, if sink is
         a tensor float32 [n_heads], the head's number there)."""
@@ -668,7 +693,7 @@ class HipOps:
             _ptr(qkv), _code(qkv), tokens, n_heads, n_kv_heads, head_dim, value_dim, _ptr(k_cache), _ptr(v_cache), _ptr(table), stride,
             n_blocks, _ptr(batch.positions), _ptr(batch.slots), _ptr(out), ctypes.c_float(scale), int(window or 0),
             _ptr(distance_slopes), int(sink is not False and sink is not None), _ptr(sink_scores), ctypes.c_long(q_stride), _ptr(distance_bias), int(span), int(chunk or 0),
-            self._stream(qkv)))
+            int(keep_first), ctypes.c_float(softcap or 0.0), self._stream(qkv)))
 
     def attention_sigmoid(self, q, n_heads, n_kv_heads, head_dim, value_dim, kv, batch, out, scale, window=None, head_mix=None,
                           head_bias=None, gate=None):
@@ -1167,10 +1192,10 @@ class HipOps:
                                                0 if out is None else _code(out), self._stream(streams)))
 
     # -- attention through a latent -----------------------------------------------------------------------
-    def latent_complete(self, down, rank, rot_dim, gain, eps, frequencies, rot_dims, kv, batch, like, rows_out=None):
+    def latent_complete(self, down, rank, rot_dim, gain, eps, frequencies, rot_dims, kv, batch, like, rows_out=None, neighbours=True, magnitude=1.0):
         """From the float32 rows `down` [latent (rank) | key part (rot_dim)] (columns of a wider matrix will do): the latent divided
-        by its root mean square, times gain, and the key part with its first rot_dims turned in pairs of neighbours by
-        position * frequencies[pair], into the cache `kv` of one key/value head (keys rank + rot_dim wide, values rank wide), whose
+        by its root mean square, times gain, and the key part with its first rot_dims turned, in pairs of neighbours (or of halves), by
+        position * frequencies[pair], cosines and sines times magnitude, into the cache `kv` of one key/value head (keys rank + rot_dim wide, values rank wide), whose
         element type is that of `like`. rows_out ([tokens, rank + rot_dim] of that type, or None) takes the same rows once more."""
         tokens = down.shape[0]
         stride = self._rows(down, "latent_complete down", rank + rot_dim, torch.float32)
@@ -1183,8 +1208,8 @@ class HipOps:
         self._require(batch.slots, "slots", torch.int32, (tokens,), down)
         k_cache, v_cache, table, table_stride, n_blocks = self._kv(kv, like, 1, rank + rot_dim, rank)
         self._check(self.lib.xrt_latent_complete(_ptr(down), ctypes.c_long(stride), _code(like), ctypes.c_long(tokens), rank, rot_dim, int(rot_dims),
-                                                 _ptr(gain), _code(gain), ctypes.c_float(eps), _ptr(frequencies), _ptr(batch.positions),
-                                                 _ptr(batch.slots), _ptr(k_cache), _ptr(v_cache), _ptr(table), table_stride, n_blocks,
+                                                 _ptr(gain), _code(gain), ctypes.c_float(eps), _ptr(frequencies), int(bool(neighbours)), ctypes.c_float(magnitude),
+                                                 _ptr(batch.positions), _ptr(batch.slots), _ptr(k_cache), _ptr(v_cache), _ptr(table), table_stride, n_blocks,
                                                  _ptr(rows_out), self._stream(down)))
 
     def causal_softmax(self, scores, heads, first_position, scale, sinks, rounded, rest):
@@ -1208,7 +1233,7 @@ class HipOps:
         self._require(out, "transpose out", src.dtype, (cols, rows), src)
         self._check(self.lib.xrt_transpose(_ptr(src), ctypes.c_long(stride), _code(src), ctypes.c_long(rows), cols, _ptr(out), self._stream(src)))
 
-    def latent_queries(self, q, heads, dim, rot_dim, frequencies, rot_dims, batch, plain, full, rank):
+    def latent_queries(self, q, heads, dim, rot_dim, frequencies, rot_dims, batch, plain, full, rank, neighbours=True, magnitude=1.0):
         """From the float32 rows q of heads x [plain (dim) | part to turn (rot_dim)]: the plain parts to `plain` [tokens, heads * dim],
         the turned parts to the last rot_dim columns of every head of `full` [tokens, heads * (rank + rot_dim)]."""
         tokens = q.shape[0]
@@ -1219,10 +1244,11 @@ class HipOps:
             self._require(frequencies, "latent_queries frequencies", torch.float32, (rot_dims // 2,), q)
         self._require(batch.positions, "positions", torch.int32, (tokens,), q)
         self._check(self.lib.xrt_latent_queries(_ptr(q), ctypes.c_long(stride), _code(plain), ctypes.c_long(tokens), heads, dim, rot_dim,
-                                                int(rot_dims), _ptr(frequencies), _ptr(batch.positions), _ptr(plain), _ptr(full),
+                                                int(rot_dims), _ptr(frequencies), int(bool(neighbours)), ctypes.c_float(magnitude), _ptr(batch.positions), _ptr(plain), _ptr(full),
                                                 ctypes.c_long(heads * (rank + rot_dim)), rank, self._stream(q)))
 
-    def latent_prepare(self, q, down, heads, dim, rank, rot_dim, gain, eps, frequencies, rot_dims, kv, batch, plain, full):
+    def latent_prepare(self, q, down, heads, dim, rank, rot_dim, gain, eps, frequencies, rot_dims, kv, batch, plain, full, neighbours=True,
+                       magnitude=1.0):
         """`latent_complete` of `down` and `latent_queries` of `q` in one launch: both float32 columns of one matrix, or of two whose
         rows lie equally far apart."""
         tokens = q.shape[0]
@@ -1241,28 +1267,30 @@ class HipOps:
         self._require(batch.slots, "slots", torch.int32, (tokens,), q)
         k_cache, v_cache, table, table_stride, n_blocks = self._kv(kv, plain, 1, rank + rot_dim, rank)
         self._check(self.lib.xrt_latent_prepare(_ptr(q), _ptr(down), ctypes.c_long(stride), _code(plain), ctypes.c_long(tokens), heads, dim, rank, rot_dim,
-                                                int(rot_dims), _ptr(gain), _code(gain), ctypes.c_float(eps), _ptr(frequencies), _ptr(batch.positions),
-                                                _ptr(batch.slots), _ptr(k_cache), _ptr(v_cache), _ptr(table), table_stride, n_blocks, _ptr(plain),
+                                                int(rot_dims), _ptr(gain), _code(gain), ctypes.c_float(eps), _ptr(frequencies), int(bool(neighbours)), ctypes.c_float(magnitude),
+                                                _ptr(batch.positions), _ptr(batch.slots), _ptr(k_cache), _ptr(v_cache), _ptr(table), table_stride, n_blocks, _ptr(plain),
                                                 _ptr(full), ctypes.c_long(heads * (rank + rot_dim)), self._stream(q)))
 
     def linear_heads(self, a, w, out, out_head=None, gate_logits=None):
         """out[t, h, :n] = w[h] a[t, h]: a [tokens, heads * k], w [heads, n, k], out [tokens, heads * out_head] with the head's
         n outputs at the beginning of its out_head columns (out_head None: n). One element type, float32 sums in the order of k.
-        gate_logits (float32 [tokens, heads], columns of a wider matrix will do): times sigmoid(gate_logits[t, h]) before the rounding."""
+        gate_logits (float32 [tokens, heads], columns of a wider matrix will do): times sigmoid(gate_logits[t, h]) before the rounding, or, with
+        heads * n columns, every output times the sigmoid of its own."""
         heads, n, k = w.shape
         tokens = a.shape[0]
         out_head = n if out_head is None else int(out_head)
         self._require(a, "linear_heads a", None, (tokens, heads * k))
         self._require(w, "linear_heads w", a.dtype, None, a)
         self._require(out, "linear_heads out", a.dtype, (tokens, heads * out_head), a)
-        gate_stride = 0
+        gate_stride, gate_width = 0, 1
         if gate_logits is not None:
-            gate_stride = self._rows(gate_logits, "linear_heads gate_logits", heads, torch.float32, a)
+            gate_width = n if gate_logits.dim() == 2 and gate_logits.shape[1] != heads else 1
+            gate_stride = self._rows(gate_logits, "linear_heads gate_logits", heads * gate_width, torch.float32, a)
             if gate_logits.shape[0] != tokens:
                 raise KernelError(f"linear_heads gate_logits: {gate_logits.shape[0]} rows for {tokens} tokens")
         self._check(self.lib.xrt_linear_heads(_ptr(a), ctypes.c_long(heads * k), ctypes.c_long(k), _ptr(w), _code(a), _ptr(out),
                                               ctypes.c_long(heads * out_head), ctypes.c_long(out_head), ctypes.c_long(tokens), heads, n, k,
-                                              _ptr(gate_logits), ctypes.c_long(gate_stride), self._stream(a)))
+                                              _ptr(gate_logits), ctypes.c_long(gate_stride), gate_width, self._stream(a)))
 
     # -- experts that multiply only the tokens that chose them
     def _expert_matrices(self, w_gate_up, w_down, experts, width, stacked=False, shared_width=0):
@@ -1343,7 +1371,7 @@ class HipOps:
         return out, parts
 
     def experts_sorted(self, h, w_gate_up, w_down, weights, chosen, width, out, activation: str = "silu", clamp=None, weigh_input=False,
-                       shared_width=0, shared_logits=None):
+                       shared_width=0, shared_logits=None, accumulate=False):
         """out[t] (float32) = sum over the experts e that token t chose, in the order of `chosen`, of weights[t, e] *
         W_down_e (act(W_gate_e h_t) * (W_up_e h_t)): the picks are sorted by expert, every expert multiplies its own rows, and
         the outputs go back to their tokens. A token's result does not depend on what else the step holds.
@@ -1351,7 +1379,7 @@ class HipOps:
         expert in a plain matrix; their product keeps float32 sums, and the clamps and the activation are a pass of their own.
         weigh_input: the weight multiplies the row that the expert reads instead of its output. shared_width: both matrices hold a
         shared expert's rows and columns behind the others'; every token's output of it joins the sum, times sigmoid(shared_logits[t])
-        if those are given."""
+        if those are given. accumulate: onto what `out` holds."""
         tokens, hidden = h.shape
         experts, top = weights.shape[1], chosen.shape[1]
         matrices = self._expert_matrices(w_gate_up, w_down, experts, width, stacked=clamp is not None, shared_width=shared_width)
@@ -1395,7 +1423,7 @@ class HipOps:
             shared, shared_parts = self._shared_expert(h, w_gate_up, matrices[1], experts * width, shared_width, activation)
         self._check(self.lib.xrt_experts_combine(_ptr(sorted_out), _ptr(places), _ptr(chosen), _ptr(weights), ctypes.c_long(tokens), top, experts,
                                                  hidden, tile, parts, _ptr(out), int(not weigh_input), _ptr(shared), self.SHARED_TILE, shared_parts,
-                                                 logits, ctypes.c_long(logits_stride), stream))
+                                                 logits, ctypes.c_long(logits_stride), int(bool(accumulate)), stream))
 
     def scale_blocks(self, act, weights, width):
         """act[t, e * width + c] *= weights[t, e], in place."""

@@ -9,7 +9,7 @@ from .latent import LatentAttention
 from .recurrent import GatedLinearAttention, LightningAttention, Retention, SelectiveStateSpace, StateSpaceDuality, TimeMixWKV
 from .parallel import ParallelMixer, WeightedPair
 from .feedforward import ClampedGLU, DenseMLP, ExpertsMLP, GatedMLP
-from .block import HyperConnectionBlock, ParallelBlock, PostNormBlock, PreNormBlock, ResidualStreams, SandwichBlock
+from .block import HyperConnectionBlock, ParallelBlock, PassEntry, PostNormBlock, PreNormBlock, ResidualStreams, SandwichBlock
 from .embedding import Embedding, HashedPairEmbedding, OutputHead, PositionedEmbedding, TokenSideInput, TokenSideTable
 
 __all__ = [
@@ -20,5 +20,5 @@ __all__ = [
     "ParallelMixer", "DenseMLP", "PositionedEmbedding", "LayerNorm", "DistanceBuckets", "PairRotation", "SharedValues",
     "SandwichBlock", "OffsetRMSNorm", "SelectiveStateSpace", "StateSpaceDuality", "WeightedPair", "ClampedGLU", "ExpertsMLP",
     "ParallelBlock", "HashedPairEmbedding", "TokenSideInput", "TokenSideTable", "HyperConnectionBlock", "ResidualStreams",
-    "LatentAttention", "LightningAttention", "PostNormBlock",
+    "LatentAttention", "LightningAttention", "PostNormBlock", "PassEntry",
 ]

@@ -34,7 +34,9 @@ asks for this path outright (float32 sums of the projection, whatever else the l
 and v but not on the output (`biases="qkv"`); head norms without weights (`qk_norm="plain"`: every head of q and k divided by
 its root mean square); a query temperature (`query_temperature=(coef, every)`: the queries at position p times
 1 + coef * ln(floor((p + 1) / every) + 1)); a sink with a learnt score per head (`sink="name"` of the tensor [n_heads]: the
-softmax's denominator also holds exp of it, neither scaled nor biased); and a layer without keys and values of its own
+softmax's denominator also holds exp of it, neither scaled, capped nor biased); a cap on the scores (`softcap=c`: a scaled score s becomes
+c * tanh(s / c)); a window that keeps a sequence's first tokens in sight (`keep_first=n`: a query sees its window and the first n
+keys, at or before it, which the cache then never lets go of); and a layer without keys and values of its own
 (`keys_from_another=True`: no k and v tensors; its schedule entry reads the cache entry of the layer whose keys and values it uses).
 """
 from __future__ import annotations
@@ -77,7 +79,7 @@ class Attention(Mixer):
                  convolution=None, names: Optional[Dict[str, str]] = None, biases: bool = False, weights: str = "softmax",
                  head_mix: Optional[str] = None, score_bias: Optional[str] = None, output_gate: Optional[str] = None,
                  values=None, unread=(), chunk: Optional[int] = None, completed: bool = False, query_temperature=None,
-                 keys_from_another: bool = False):
+                 keys_from_another: bool = False, softcap: Optional[float] = None, keep_first: int = 0):
         if n_heads <= 0 or n_kv_heads <= 0 or n_heads % n_kv_heads != 0:
             raise ValueError(f"head counts {n_heads}/{n_kv_heads}: the first must be a multiple of the second")
         if weights not in ("softmax", "sigmoid"):
@@ -98,6 +100,12 @@ class Attention(Mixer):
         if self.query_temperature is not None and self.query_temperature[1] <= 0:
             raise ValueError(f"a query temperature grows every so many positions, found {query_temperature!r}")
         self.keys_from_another = bool(keys_from_another)
+        self.softcap = None if softcap is None else float(softcap)
+        self.keep_first = int(keep_first) if window is not None else 0      # (without a window every key is in sight anyway)
+        if (self.softcap is not None and self.softcap <= 0) or keep_first < 0:
+            raise ValueError(f"a cap on the scores is positive and first tokens are counted from 0, found {softcap!r} and {keep_first!r}")
+        if weights != "softmax" and (self.softcap is not None or self.keep_first):
+            raise ValueError("a cap on the scores and kept first tokens are served for softmax weights")
         self.head_mix_name, self.score_bias_name, self.gate_name = head_mix, score_bias, output_gate
         self.values = values
         self.unread = tuple(unread)         # tensors under the prefix that a checkpoint may carry and this layer does not read
@@ -106,7 +114,8 @@ class Attention(Mixer):
             raise ValueError("stretches of positions have a positive size and are served for softmax weights")
         self.completed = (bool(completed) or self.biases or weights == "sigmoid" or output_gate is not None or values is not None or self.chunk is not None
                           or hasattr(position, "pair_rotation") or hasattr(position, "score_bias_table") or self.sink_name is not None
-                          or self.plain_norm or self.query_temperature is not None or self.keys_from_another)
+                          or self.plain_norm or self.query_temperature is not None or self.keys_from_another
+                          or self.softcap is not None or self.keep_first > 0)
         if self.completed and convolution is not None:
             raise ValueError("the completed path of attention has no convolution")
         if self.sink and weights != "softmax":
@@ -184,7 +193,7 @@ class Attention(Mixer):
 
     def cache_needs(self) -> CacheNeeds:
         needs = CacheNeeds(kv=KVSpec(self.n_kv_heads, self.head_dim, self.window,
-                                     None if self.value_dim == self.head_dim else self.value_dim))
+                                     None if self.value_dim == self.head_dim else self.value_dim, self.keep_first))
         return needs if self.convolution is None else needs.merged(self.convolution.cache_needs())
 
     def bind(self, tensors, runtime: Runtime) -> None:
@@ -287,7 +296,7 @@ class Attention(Mixer):
         slopes = None if self.position is None else self.position.score_slopes()
         ops.attention(q, self.n_heads, self.n_kv_heads, self.head_dim, cache.kv, batch, out, scale=self.scale, window=self.window,
                       distance_slopes=slopes, value_dim=self.value_dim, distance_bias=table, queries_alone=True, chunk=self.chunk,
-                      sink=self.sink_scores if self.sink_scores is not None else self.sink)
+                      sink=self.sink_scores if self.sink_scores is not None else self.sink, keep_first=self.keep_first, softcap=self.softcap)
         return out
 
     def forward_into(self, h, batch, cache, out: torch.Tensor, bias_later: bool = False):
@@ -309,6 +318,9 @@ class Attention(Mixer):
         return None
 
     def forward(self, h, batch, cache, residual: torch.Tensor, then=None):
+        if self.completed and self.bias_o is None:
+            self.runtime.ops.linear(self._attend_completed(h, batch, cache), self.w_o, residual, accumulate=True)
+            return None
         if self.completed:
             out = self.runtime.empty(residual.shape, torch.float32)
             self.forward_into(h, batch, cache, out)

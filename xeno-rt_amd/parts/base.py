@@ -40,12 +40,14 @@ class KVSpec:
     as wide as the keys unless given).
 
     window = None keeps all tokens; window = W keeps what a query can still see
-    when it looks at the W most recent tokens (itself included).
+    when it looks at the W most recent tokens (itself included). keep_first: a window
+    lets go of none of a sequence's first keep_first tokens.
     """
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     value_dim: Optional[int] = None
+    keep_first: int = 0
 
     @property
     def value_width(self) -> int:

@@ -236,17 +236,24 @@ class ParallelBlock(Block):
     write their float32 outputs aside and one pass adds them to the stream; a mixer that is itself a weighted sum of
     mixers (`forward_terms`) has its terms added in that same pass. `after`, if given, is a part that then adds what the
     step's tokens bring to the stream of their own (`forward(x, batch, reads=)`, reads being x in the compute dtype if the
-    block has it at hand)."""
+    block has it at hand). With `feed_forward_norm` the feed-forward reads a norm of its own, of the same x:
+    x += a * mixer(norm(x)) + b * feed_forward(feed_forward_norm(x)); two plain RMS norms of equal eps are one pass. Without a and b
+    each sublayer then adds its own output to the stream, in turn: what both read was made before. `unread`: tensors that
+    a checkpoint may carry for the block and that it does not read."""
 
-    def __init__(self, norm, mixer, feed_forward=None, hidden=None, mixer_scale=None, feed_forward_scale=None, after=None):
+    def __init__(self, norm, mixer, feed_forward=None, hidden=None, mixer_scale=None, feed_forward_scale=None, after=None, feed_forward_norm=None,
+                 unread=()):
+        if feed_forward_norm is not None and feed_forward is None:
+            raise ValueError("a feed-forward's norm without a feed-forward")
         self.norm, self.mixer, self.feed_forward, self.after = norm, mixer, feed_forward, after
+        self.feed_forward_norm = feed_forward_norm
         self.hidden = int(hidden if hidden is not None else norm.dim)
         self.scale_names = (mixer_scale, feed_forward_scale if feed_forward is not None else None)
-        self.unread = [feed_forward_scale] if feed_forward is None and feed_forward_scale is not None else []
+        self.unread = list(unread) + ([feed_forward_scale] if feed_forward is None and feed_forward_scale is not None else [])
         self.scales = [None, None]
 
     def parts(self):
-        return tuple(part for part in (self.norm, self.mixer, self.feed_forward, self.after) if part is not None)
+        return tuple(part for part in (self.norm, self.mixer, self.feed_forward_norm, self.feed_forward, self.after) if part is not None)
 
     @property
     def capturable(self) -> bool:
@@ -275,9 +282,26 @@ class ParallelBlock(Block):
     def first_norm(self):
         return self.norm
 
+    def _reads(self, x):
+        """What the mixer and what the feed-forward reads."""
+        if self.feed_forward_norm is None:
+            h = self.norm.forward(x)
+            return h, h
+        rt = self.runtime
+        scales = [norm.row_scale() for norm in (self.norm, self.feed_forward_norm)]
+        if any(scale is None for scale in scales) or scales[0][1] != scales[1][1] or scales[0][0].dtype != scales[1][0].dtype:
+            return self.norm.forward(x), self.feed_forward_norm.forward(x)
+        outs = rt.empty(x.shape), rt.empty(x.shape)
+        rt.ops.rmsnorm_two(x, [gain for gain, _ in scales], scales[0][1], outs)
+        return outs
+
     def forward(self, x, batch, cache) -> None:
         rt = self.runtime
-        h = self.norm.forward(x)
+        h, h_of_feed_forward = self._reads(x)
+        if self.feed_forward_norm is not None and self.scale_names == (None, None) and self.after is None and not hasattr(self.mixer, "forward_terms"):
+            self.mixer.forward(h, batch, cache, x)
+            self.feed_forward.forward(h_of_feed_forward, batch, x)
+            return
         if hasattr(self.mixer, "forward_terms"):
             terms = [(y, self.scales[0], scale) for y, scale in self.mixer.forward_terms(h, batch, cache, x)]
         else:
@@ -286,13 +310,49 @@ class ParallelBlock(Block):
             terms = [(y, self.scales[0], 1.0)]
         if self.feed_forward is not None:
             y = rt.empty(x.shape, torch.float32)
-            self.feed_forward.forward_into(h, batch, y)
+            self.feed_forward.forward_into(h_of_feed_forward, batch, y)
             terms.append((y, self.scales[1], 1.0))
         # what follows reads the updated stream in the compute dtype: written in the same pass
         reads = rt.empty(x.shape) if self.after is not None and rt.dtype != torch.float32 else None
         rt.ops.add_weighted(x, terms, copy=reads)
         if self.after is not None:
             self.after.forward(x, batch, reads=reads)
+
+
+class PassEntry(Part):
+    """What comes before every pass of layers that run several times in a row: x <- W [x; o], o being the stream as the embedding left
+    it. `name` is the tensor [width, 2 width] that holds W = [A | B]. B o is the same for all passes of a step and made once (`open`);
+    a pass then puts it in x's place and adds A times what x was."""
+    capturable = True
+
+    def __init__(self, name: str, hidden: int):
+        self.name, self.hidden = name, int(hidden)
+        self.of_stream = self.of_origin = None
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        return {self.name: WeightSpec((self.hidden, 2 * self.hidden))}
+
+    def bind(self, tensors, runtime: Runtime) -> None:
+        super().bind(tensors, runtime)
+        w = tensors[self.name]
+        self.of_stream, self.of_origin = runtime.weight(w[:, :self.hidden]), runtime.weight(w[:, self.hidden:])
+
+    def open(self, x: torch.Tensor) -> torch.Tensor:
+        """B o (float32) for the stream x as the embedding left it."""
+        rt = self.runtime
+        read = x
+        if rt.dtype != torch.float32:
+            read = rt.empty(x.shape)
+            rt.ops.cast(x, read)
+        out = rt.empty(x.shape, torch.float32)
+        rt.ops.linear(read, self.of_origin, out)
+        return out
+
+    def forward(self, x: torch.Tensor, opened: torch.Tensor) -> None:
+        rt = self.runtime
+        read = rt.empty(x.shape)
+        rt.ops.replace_rows(x, opened, read)
+        rt.ops.linear(read, self.of_stream, x, accumulate=True)
 
 
 class ResidualStreams(Part):

@@ -1,6 +1,7 @@
 """Token embedding and output head.
 
-Embedding: x = E[token_id, :], no scaling (crates/xrt-models/src/llama.rs:1042-1055).
+Embedding: x = E[token_id, :], no scaling (crates/xrt-models/src/llama.rs:1042-1055) unless one is given (`scale`; a head that
+is tied to the table reads it without).
 Head: logits = W y in float32, W = lm_head.weight, or the embedding table when
 the model ties them (llama.rs:299-305, 604-613).
 """
@@ -16,8 +17,9 @@ from .base import CacheNeeds, Part, Runtime, StateSpec, WeightSpec
 class Embedding(Part):
     capturable = True
 
-    def __init__(self, prefix: str, vocab: int, hidden: int, name: Optional[str] = None):
+    def __init__(self, prefix: str, vocab: int, hidden: int, name: Optional[str] = None, scale: float = 1.0):
         self.prefix = prefix
+        self.row_scale = float(scale)
         self.name = name if name is not None else prefix + "weight"       # the table's tensor
         self.vocab = vocab
         self.hidden = hidden
@@ -37,7 +39,7 @@ class Embedding(Part):
         """float32 residual stream [tokens, hidden] for int32 token ids (an embedding that knows nothing of positions
         does not look at them)."""
         x = self.runtime.empty((token_ids.shape[0], self.hidden), torch.float32)
-        self.runtime.ops.embed(self.table, token_ids, x)
+        self.runtime.ops.embed(self.table, token_ids, x, **({} if self.row_scale == 1.0 else {"scale": self.row_scale}))
         return x
 
 

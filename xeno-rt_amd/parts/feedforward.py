@@ -166,7 +166,7 @@ class ExpertsMLP(FeedForward):
     matrix whose product keeps float32 sums, which the clamps and the activation read and round once.
     `normalized=False` takes the chosen scores as weights as they are; `weigh_input=True` multiplies what a chosen expert reads
     by the weight instead of its output; `shared=n` adds a shared expert of width n (`shared.gate|up|down`, same form) that every
-    token uses, times sigmoid(`shared.sg` h), one number a token. With either of the last two a step of few tokens keeps the float32
+    token uses, times sigmoid(`shared.sg` h), one number a token (`shared_gate=None`: its output as it is). With either of the last two a step of few tokens keeps the float32
     sums of the gate/up product, and one kernel makes every expert's stretch of the activations from them, weights and
     shared gate included: the shared expert's rows and columns lie behind the others' in the same two matrices, and its
     gate's row below the router's."""
@@ -177,7 +177,7 @@ class ExpertsMLP(FeedForward):
     def __init__(self, prefix: str, hidden: int, intermediate: int, experts: int, top: int, groups=None, keep=None,
                  router: str = "router", expert: str = "e{}.", gate: str = "gate", up: str = "up", down: str = "down",
                  scores: str = "sigmoid", group_top: Optional[int] = None, scale: float = 1.0, clamp=None, normalized: bool = True,
-                 weigh_input: bool = False, shared: Optional[int] = None, shared_expert: str = "shared.", shared_gate: str = "sg"):
+                 weigh_input: bool = False, shared: Optional[int] = None, shared_expert: str = "shared.", shared_gate: Optional[str] = "sg"):
         if experts <= 0 or not 0 < top <= experts:
             raise ValueError(f"{top} of {experts} experts")
         if scores not in ("sigmoid", "softmax"):
@@ -201,7 +201,7 @@ class ExpertsMLP(FeedForward):
         self.router_name = prefix + router
         self.expert_names = [tuple(prefix + expert.format(n) + name for name in (gate, up, down)) for n in range(self.experts)]
         self.shared_names = None if shared is None else tuple(prefix + shared_expert + name for name in (gate, up, down))
-        self.shared_gate_name = None if shared is None else prefix + shared_expert + shared_gate
+        self.shared_gate_name = None if shared is None or shared_gate is None else prefix + shared_expert + shared_gate
         self.w_router = self.w_gate_up = self.w_down = None
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
@@ -209,8 +209,9 @@ class ExpertsMLP(FeedForward):
         specs = {self.router_name: WeightSpec((self.experts, h))}
         if self.shared is not None:
             gate, up, down = self.shared_names
-            specs.update({gate: WeightSpec((self.shared, h)), up: WeightSpec((self.shared, h)), down: WeightSpec((h, self.shared)),
-                          self.shared_gate_name: WeightSpec((1, h))})
+            specs.update({gate: WeightSpec((self.shared, h)), up: WeightSpec((self.shared, h)), down: WeightSpec((h, self.shared))})
+            if self.shared_gate_name is not None:
+                specs[self.shared_gate_name] = WeightSpec((1, h))
         for gate, up, down in self.expert_names:
             specs.update({gate: WeightSpec((i, h)), up: WeightSpec((i, h)), down: WeightSpec((h, i))})
         return specs
@@ -218,7 +219,7 @@ class ExpertsMLP(FeedForward):
     def bind(self, tensors, runtime: Runtime) -> None:
         super().bind(tensors, runtime)
         shared = self.shared or 0
-        self.w_router = (runtime.matrix(tensors[self.router_name]) if not shared else
+        self.w_router = (runtime.matrix(tensors[self.router_name]) if self.shared_gate_name is None else
                          runtime.stacked([tensors[self.router_name], tensors[self.shared_gate_name]]))
         names_of_all = self.expert_names + ([self.shared_names] if shared else [])
         total = self.experts * self.intermediate + shared
@@ -239,16 +240,19 @@ class ExpertsMLP(FeedForward):
         self.w_down = runtime.weight(down)
 
     def _weights(self, h, chosen=None):
-        """(weights [tokens, experts], the shared expert's gate logits [tokens] or None)."""
+        """(weights [tokens, experts], the shared expert's gate logits [tokens], or None if it has no gate)."""
         rt = self.runtime
         logits = rt.empty((h.shape[0], self.w_router.shape[0]), torch.float32)
         rt.ops.linear(h, self.w_router, logits)
         weights = rt.empty((h.shape[0], self.experts), torch.float32)
         rt.ops.route_experts(logits[:, :self.experts], weights, self.top, self.groups, self.keep, self.group_top, self.WEIGHT_FLOOR, chosen=chosen,
                              scores=self.scores, scale=self.scale, **({} if self.normalized else {"normalized": False}))
-        return weights, (None if self.shared is None else logits[:, self.experts])
+        return weights, (None if self.shared_gate_name is None else logits[:, self.experts])
 
     def forward_into(self, h, batch, out: torch.Tensor) -> None:
+        self._run(h, out, False)
+
+    def _run(self, h, out: torch.Tensor, accumulate: bool) -> None:
         rt = self.runtime
         # A step of many tokens of which each uses few of the experts: the picks sorted by expert, every expert multiplies the
         # tokens that chose it. (Where the kernels have no such product, or it would not pay, every token meets every expert.)
@@ -262,6 +266,8 @@ class ExpertsMLP(FeedForward):
             extra = {"activation": "silu"} if self.clamp is None else {"clamp": self.clamp}
             if self.keeps_sums:
                 extra.update(weigh_input=self.weigh_input, shared_width=self.shared or 0, shared_logits=shared_logits)
+            if accumulate:
+                extra["accumulate"] = True
             rt.ops.experts_sorted(h, self.w_gate_up, self.w_down, weights, chosen, self.intermediate, out, **extra)
             return
         weights, shared_logits = self._weights(h)
@@ -280,12 +286,10 @@ class ExpertsMLP(FeedForward):
         else:
             rt.ops.linear_glu(h, self.w_gate_up, act, activation="silu")
             rt.ops.scale_blocks(act, weights, self.intermediate)
-        rt.ops.linear(act, self.w_down, out)
+        rt.ops.linear(act, self.w_down, out, accumulate=accumulate)
 
     def forward(self, h, batch, residual: torch.Tensor) -> None:
-        out = self.runtime.empty(residual.shape, torch.float32)
-        self.forward_into(h, batch, out)
-        self.runtime.ops.add(residual, out)
+        self._run(h, residual, True)
 
 
 register_part("feed_forward", "gated_mlp", GatedMLP)

@@ -5,13 +5,15 @@ With h the mixer's input, H heads, per head d plain and r turned query/key dims 
   latent    W_dkv h = [kv_rank | r]: c = RMSnorm of the first kv_rank (gain `dkv.norm`); the last r are one key part for all
             heads, turned like the queries' parts and not normed
   per head  plain key W_uk,h c, value W_uv,h c; score = (q_plain . k_plain + q_turned . k_turned) * scale
-  rotation  the first `rot_dims` of a part of r turn in pairs of neighbours (2i, 2i + 1) by position * base^(-2i / rot_dims)
+  rotation  the first `rot_dims` of a part of r turn in pairs of neighbours (2i, 2i + 1) by position * base^(-2i / rot_dims), or as the
+            `position` that is handed over says (a PairRotation: pairs of halves, stretched frequencies, a magnitude)
   softmax   over the keys at or before the query, with one more term exp(sink_h) in the denominator (a learnt number per head)
   output    W_o on the heads' outputs side by side
 
 Options: `q_rank=None` makes the queries straight from the input, q = W_q h (no c_q); `sink=None` leaves the denominator to the keys
 alone; `window=W` lets a query see only the W newest of the keys up to its own, which is one of them, and the cache
-then keeps what a window still sees; `output_gate="g"` multiplies head i's output by sigmoid(W_g h)_i before W_o.
+then keeps what a window still sees; `output_gate="g"` multiplies head i's output by sigmoid(W_g h)_i before W_o, and with
+`gate_per="output"` W_g has a row for each of the heads' outputs, which are multiplied by their own sigmoids.
 
 What is cached per token is one row [c | turned key part] as the key of a single key/value head, and c as its value. The
 per-head keys never exist: q_plain . (W_uk,h c) = (W_uk,h^T q_plain) . c, so the plain part of a query is multiplied by its
@@ -47,16 +49,21 @@ class LatentAttention(Mixer):
 
     def __init__(self, prefix: str, hidden: int, n_heads: int, dim: int, rot_dim: int, value_dim: int, kv_rank: int, q_rank: Optional[int],
                  scale: float, eps: float, rot_dims: int, rot_base: float, sink: Optional[str] = "sink", window: Optional[int] = None,
-                 output_gate: Optional[str] = None):
+                 output_gate: Optional[str] = None, gate_per: str = "head", position: Optional[PairRotation] = None):
         if min(n_heads, dim, value_dim, kv_rank) <= 0 or rot_dim < 0 or (q_rank is not None and q_rank <= 0) or (window is not None and window <= 0):
             raise ValueError("latent attention: sizes must be positive")
         if rot_dims < 0 or rot_dims % 2 != 0 or rot_dims > rot_dim:
             raise ValueError(f"latent attention: {rot_dims} dims turn in pairs inside a part of {rot_dim}")
         self.prefix, self.hidden, self.n_heads, self.dim, self.rot_dim = prefix, hidden, int(n_heads), int(dim), int(rot_dim)
         self.value_dim, self.kv_rank, self.q_rank = int(value_dim), int(kv_rank), None if q_rank is None else int(q_rank)
+        if gate_per not in ("head", "output"):
+            raise ValueError(f"a gate stands for a head or for each of its outputs, found {gate_per!r}")
+        if position is not None and position.rope_dim != rot_dims:
+            raise ValueError(f"a rotation of {position.rope_dim} dims for a part of which {rot_dims} turn")
         self.window, self.gate_name = None if window is None else int(window), output_gate
+        self.gate_rows = self.n_heads * (self.value_dim if gate_per == "output" else 1)
         self.scale, self.eps, self.sink_name = float(scale), float(eps), sink
-        self.position = PairRotation(rot_dims, rot_base, neighbours=True) if rot_dims > 0 else None
+        self.position = position if position is not None else PairRotation(rot_dims, rot_base, neighbours=True) if rot_dims > 0 else None
         self.rot_dims = int(rot_dims)
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
@@ -72,7 +79,7 @@ class LatentAttention(Mixer):
         if self.sink_name is not None:
             specs[p + self.sink_name] = WeightSpec((heads,), init="zeros", kind="vector")
         if self.gate_name is not None:
-            specs[p + self.gate_name] = WeightSpec((heads, w))
+            specs[p + self.gate_name] = WeightSpec((self.gate_rows, w))
         specs[p + "o"] = WeightSpec((w, heads * self.value_dim))
         return specs
 
@@ -149,29 +156,30 @@ class LatentAttention(Mixer):
         rt = self.runtime
         ops = rt.ops
         tokens, heads, rank, rot = h.shape[0], self.n_heads, self.kv_rank, self.rot_dim
-        frequencies = None if self.position is None else self.position.pair_rotation()[0]
+        frequencies, _, neighbours, magnitude = (None, 0, True, 1.0) if self.position is None else self.position.pair_rotation()
+        turn = dict(neighbours=neighbours, magnitude=magnitude)
         prompts = self._prompts_alone(h, batch, cache)
         rows = rt.empty((tokens, rank + rot)) if prompts else None
         plain = rt.empty((tokens, heads * self.dim))
         full = rt.empty((tokens, heads * (rank + rot)))
         gates = None
         if self.q_rank is None:
-            cuts = [heads * (self.dim + rot), rank + rot] + ([heads] if self.gate_name is not None else [])
+            cuts = [heads * (self.dim + rot), rank + rot] + ([self.gate_rows] if self.gate_name is not None else [])
             sums = rt.empty((tokens, sum(cuts)), torch.float32)
             ops.linear(h, self.w_in, sums)
             q, down, *rest = sums.split(cuts, dim=1)
             gates = rest[0] if rest else None
             if cache.writable and not prompts:
-                ops.latent_prepare(q, down, heads, self.dim, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, plain, full)
+                ops.latent_prepare(q, down, heads, self.dim, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, plain, full, **turn)
             else:
                 if cache.writable:
-                    ops.latent_complete(down, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, like=h, rows_out=rows)
-                ops.latent_queries(q, heads, self.dim, rot, frequencies, self.rot_dims, batch, plain, full, rank)
+                    ops.latent_complete(down, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, like=h, rows_out=rows, **turn)
+                ops.latent_queries(q, heads, self.dim, rot, frequencies, self.rot_dims, batch, plain, full, rank, **turn)
         else:
             if cache.writable:
                 down = rt.empty((tokens, rank + rot), torch.float32)
                 ops.linear(h, self.w_dkv, down)
-                ops.latent_complete(down, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, like=h, rows_out=rows)
+                ops.latent_complete(down, rank, rot, self.kv_gain, self.eps, frequencies, self.rot_dims, cache.kv, batch, like=h, rows_out=rows, **turn)
             low = rt.empty((tokens, self.q_rank), torch.float32)
             ops.linear(h, self.w_dq, low)
             c_q = rt.empty((tokens, self.q_rank))
@@ -179,9 +187,9 @@ class LatentAttention(Mixer):
             q = rt.empty((tokens, heads * (self.dim + rot)), torch.float32)
             ops.linear(c_q, self.w_uq, q)
             if self.w_gate is not None:
-                gates = rt.empty((tokens, heads), torch.float32)
+                gates = rt.empty((tokens, self.gate_rows), torch.float32)
                 ops.linear(h, self.w_gate, gates)
-            ops.latent_queries(q, heads, self.dim, rot, frequencies, self.rot_dims, batch, plain, full, rank)
+            ops.latent_queries(q, heads, self.dim, rot, frequencies, self.rot_dims, batch, plain, full, rank, **turn)
         ops.linear_heads(plain, self.w_uk_t, full, out_head=rank + rot)
         summed = rt.empty((tokens, heads * rank))
         if prompts:
