@@ -51,6 +51,13 @@ the same for the Mitunex decoder (attention through a cached latent under a wind
 sublayers; the first layer's feed-forward dense, behind the others eight experts of which a token uses two and a shared one;
 every fourth layer runs the weights of the one before it once more), beside the Renapel decoder, the library's closest
 (attention through a latent, experts), and Llama.
+
+    python bench.py --design fisopel [--size small|medium|large] [--layers N]
+
+the same for the Fisopel decoder (attention through a cached latent with a gate per output, and grouped attention with head norms, capped
+scores and a learnt sink under a window of 512 keys that keeps the first four, in turn, each beside eight experts of which a token
+uses two and a shared one; one pass through the layers), beside the Mitunex decoder, the library's closest (attention through a latent,
+experts beside a shared one), and Llama.
 """
 import argparse
 import json
@@ -214,9 +221,23 @@ def mitunex_config(size, layers, max_positions):
             "logit_scale": 0.5, "logit_softcap": 50.0, "layers": out}
 
 
+def fisopel_config(size, layers, max_positions):
+    w, d, ff = size["width"], size["head"], size["ff"]
+    heads = w // d
+    latent = {"heads": heads, "dim": d, "rot_dim": d // 2, "vdim": d, "kv_rank": 3 * d, "scale": (3 * d // 2) ** -0.5,
+              "rot": {"dims": d // 2, "base": 500000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 16.0, "slow": 2.0}}}
+    windowed = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": d, "vdim": d, "mask": {"size": 512, "keep_first": 4}, "scale": d ** -0.5,
+                "softcap": 30.0}
+    experts = {"kind": "moe", "expert": {"ff": ff // 2}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 2}}
+    kinds = [("latent_attention", latent), ("attention", windowed)]
+    return {"architecture": "Fisopel", "vocab": size["vocab"], "width": w, "norm": {"eps": 1e-6}, "embedding": {"scale": w ** 0.5},
+            "loop": {"start": 0, "stop": max(1, layers), "times": 1},
+            "layers": [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": experts} for i in range(layers)]}
+
+
 DESIGN_CONFIGS = {"sozopel": sozopel_config, "ledudra": ledudra_config, "depunex": depunex_config, "renapel": renapel_config,
-                  "mitunex": mitunex_config}
-DESIGN_BESIDE = {"depunex": ("sozopel", "llama"), "renapel": ("depunex", "llama"), "mitunex": ("renapel", "llama")}          # the models a design is measured beside (Llama alone unless named)
+                  "mitunex": mitunex_config, "fisopel": fisopel_config}
+DESIGN_BESIDE = {"depunex": ("sozopel", "llama"), "renapel": ("depunex", "llama"), "mitunex": ("renapel", "llama"), "fisopel": ("mitunex", "llama")}          # the models a design is measured beside (Llama alone unless named)
 
 
 def llama_config(size, layers, max_positions):

@@ -16,13 +16,11 @@
 // head's sink to the denominator (a learnt score without a value, or none) and writes the result.
 //
 // Steps that bring sequences many tokens (xrt_attention_latent_prompts). The heads of a key/value head read the same keys in all
-// tokens, so its (token, head) pairs of a sequence are simply rows, one after another, and a wavefront takes sixteen of them (or, with
-// keys and values of up to 128 dims, two sets of sixteen, which share every tile read from LDS) as the columns of
+// tokens, so its (token, head) pairs of a sequence are simply rows, one after another, and a wavefront takes sixteen of them as the columns of
 // its products: with many heads its rows are one token's or a few tokens', with few heads many tokens'. A workgroup of eight
-// wavefronts walks the groups of 32 keys that some row of it sees; a group's tiles of keys and values (a contiguous
+// wavefronts (or four) walks the groups of 32 keys that some row of it sees; a group's tiles of keys and values (a contiguous
 // stretch each) travel straight into LDS while the group before it is multiplied. The softmax keeps its exponent until a score
-// exceeds it by 8 (in log2), so that the sums are rarely rescaled. (Two sets of sixteen columns of larger keys and values need more
-// registers than there are: the compiler keeps the sums twice around the rescaling.)
+// exceeds it by 8 (in log2), so that the sums are rarely rescaled.
 #include "cache_layout.h"
 #include "xrt_hip.h"
 
@@ -207,7 +205,8 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_chunks_kernel(const bf16* __r
     }
 }
 
-// A workgroup a (token, head): the chunks' parts in their order, the sink, the quotient.
+// A workgroup a (token, head): the chunks' parts in their order, the sink, the quotient. OWNED: value dims a lane has (value size / 64 at least).
+template <int OWNED>
 __global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __restrict__ partial, const Shape shape, int chunk_groups, int chunks, const int* __restrict__ positions,
                                                                const int* __restrict__ slots, const float* __restrict__ sinks, bf16* __restrict__ out) {
     const long token = blockIdx.x;
@@ -221,7 +220,7 @@ __global__ void __launch_bounds__(XRT_WAVE) latent_merge_kernel(const float* __r
     const int pos = positions[token];
     const int mine = (Seen(pos, shape.window, shape.keep_first).groups(pos) - 1) / chunk_groups + 1;      // this query's chunks
     const float* parts = partial + ((token * groups + group) * chunks) * partial_floats(value_dim) + (long)(in_group % HEADS_A_WAVE) * head_floats(value_dim);
-    constexpr int OWNED = LATENT_MOST / XRT_WAVE, MERGED = 8;
+    constexpr int MERGED = 8;
     float acc[OWNED], top = -INFINITY, sum = 0.f;
 #pragma unroll
     for (int i = 0; i < OWNED; ++i) acc[i] = 0.f;
@@ -280,19 +279,19 @@ int chunks_for(int max_context, int window, int keep_first) {
 
 // ---- steps that bring sequences many tokens -------------------------------------------------------------------------------
 
-constexpr int PROMPT_WAVES = 8;
-constexpr int SET_ROWS = 16;                     // columns of a product
+constexpr int WAVE_ROWS = 16;                    // rows of a wavefront: the columns of its products
 constexpr int AHEAD = 2;                         // pairs of tiles that are read from LDS ahead of their products
 constexpr int TILE_BYTES = 1024;                 // an operand tile of the cache, in the order of the lanes
 
 // KS, VT: the steps of 32 key dims and tiles of 16 value dims that this instantiation multiplies, whatever the sizes leave of them.
-// SETS: sets of sixteen rows a wavefront has. CAP: with a softcap.
-template <int KS, int VT, int SETS, bool CAP>
-__global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel(
+// WAVES: wavefronts of a workgroup. CAP: with a softcap. (Tried and no faster: two sets of sixteen rows a wavefront, which share the tiles
+// read from LDS, and three groups of keys in LDS instead of two.)
+template <int KS, int VT, int WAVES, bool CAP>
+__global__ void __launch_bounds__(WAVES * XRT_WAVE) latent_prompts_kernel(
     const bf16* __restrict__ q, const Shape shape, const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache,
     const int* __restrict__ block_table, int table_stride, int n_blocks, const int* __restrict__ seq_offsets, const int* __restrict__ seq_slots,
     const int* __restrict__ seq_starts, int n_seqs, float scale, float softcap, const float* __restrict__ sinks, bf16* __restrict__ out) {
-    constexpr int WAVE_ROWS = SETS * SET_ROWS, TILE_ROWS = PROMPT_WAVES * WAVE_ROWS;
+    constexpr int TILE_ROWS = WAVES * WAVE_ROWS;
     extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
     const int lane = threadIdx.x % XRT_WAVE, column = lane % 16, quarter = lane / 16;
     const int wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x / XRT_WAVE);
@@ -331,41 +330,28 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
     const int groups = kept_groups + group_high - group_low + 1;
     auto group_at = [&](int counted) { return counted < kept_groups ? counted : group_low + counted - kept_groups; };
 
-    // this wavefront's rows, a column of a set each
+    // this wavefront's rows, a column each
     const int wave_row = tile * TILE_ROWS + wave * WAVE_ROWS;
     const bool awake = wave_row < rows;
     const int wave_low = start + min(wave_row, rows - 1) / group_size, wave_high = start + min(wave_row + WAVE_ROWS - 1, rows - 1) / group_size;
     const int wave_all = Seen(wave_high, window, keep_first).first;      // the first key that the windows of all rows of the wavefront hold
-    int row[SETS], pos[SETS], head[SETS];
-    bf16x8 queries[SETS][KS];
+    const int row = wave_row + column, clamped = min(row, rows - 1);
+    const int pos = start + clamped / group_size, head = kv_head * group_size + clamped % group_size;
+    const bf16* of_row = q + at(clamped) * head_dim + quarter * 8;
+    bf16x8 queries[KS];
 #pragma unroll
-    for (int w = 0; w < SETS; ++w) {
-        row[w] = wave_row + w * SET_ROWS + column;
-        const int clamped = min(row[w], rows - 1);
-        pos[w] = start + clamped / group_size;
-        head[w] = kv_head * group_size + clamped % group_size;
-        const bf16* of_row = q + at(clamped) * head_dim + quarter * 8;
+    for (int s = 0; s < KS; ++s) {
 #pragma unroll
-        for (int s = 0; s < KS; ++s) {
-#pragma unroll
-            for (int e = 0; e < 8; ++e) queries[w][s][e] = (bf16)0.f;
-            if (s < key_steps) queries[w][s] = *reinterpret_cast<const bf16x8*>(of_row + s * 32);
-        }
+        for (int e = 0; e < 8; ++e) queries[s][e] = (bf16)0.f;
+        if (s < key_steps) queries[s] = *reinterpret_cast<const bf16x8*>(of_row + s * 32);
     }
     // (awaited here: left to their first use the wait would stand inside the loop and hold up the tiles on their way to LDS)
 #pragma unroll
-    for (int w = 0; w < SETS; ++w)
+    for (int s = 0; s < KS; ++s) asm volatile("" : "+v"(queries[s]));
+    floatx4 o[VT];
 #pragma unroll
-        for (int s = 0; s < KS; ++s) asm volatile("" : "+v"(queries[w][s]));
-    floatx4 o[SETS][VT];
-    float m[SETS], l[SETS];                                    // m is shared by the row's four lanes, l is this lane's share
-#pragma unroll
-    for (int w = 0; w < SETS; ++w) {
-#pragma unroll
-        for (int u = 0; u < VT; ++u) o[w][u] = floatx4{0.f, 0.f, 0.f, 0.f};
-        m[w] = -INFINITY;
-        l[w] = 0.f;
-    }
+    for (int u = 0; u < VT; ++u) o[u] = floatx4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;                              // m is shared by the row's four lanes, l is this lane's share
 
     // scores are kept in units of log2: scaled as they are used, or, with a softcap, scaled and capped at once
     const float scale2 = CAP ? 1.0f : scale * LOG2E;
@@ -383,7 +369,7 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
         const long of_head = ((long)block * shape.n_kv_heads + kv_head) * XRT_BLOCK_TOKENS;
         const char* keys = reinterpret_cast<const char*>(k_cache + of_head * head_dim) + (long)(g % 2) * key_tiles * TILE_BYTES;
         const char* values = reinterpret_cast<const char*>(v_cache + of_head * value_dim) + (long)(g % 2) * value_tiles * TILE_BYTES;
-        for (int t = wave; t < tiles_a_group; t += PROMPT_WAVES) {
+        for (int t = wave; t < tiles_a_group; t += WAVES) {
             const bool is_key = t < key_tiles;
             const int place = !is_key ? 2 * KS + t - key_tiles : t < key_steps ? t : KS + t - key_steps;
             load_to_lds(is_key ? keys : values, (unsigned)((is_key ? t : t - key_tiles) * TILE_BYTES + lane * 16),
@@ -392,22 +378,21 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
     };
 
     // places that the sizes at hand leave empty hold zeros (the code multiplies them all, without a branch)
-    for (int t = wave; t < 2 * PLACES; t += PROMPT_WAVES) {
+    for (int t = wave; t < 2 * PLACES; t += WAVES) {
         const int place = t % PLACES;
         if (place < 2 * KS ? place % KS >= key_steps : place - 2 * KS >= value_tiles)
             *reinterpret_cast<uint4*>(lds_raw + (size_t)t * TILE_BYTES + lane * 16) = make_uint4(0u, 0u, 0u, 0u);
     }
     fetch(group_at(0), 0);
-    wait_loads_and_barrier<0>();
     for (int counted = 0; counted < groups; ++counted) {
+        // this group has arrived from every wavefront, and the one before it has been read by all: its buffer takes the next one
+        wait_loads_and_barrier<0>();
         const int buffer = counted & 1;
-        if (counted + 1 < groups) fetch(group_at(counted + 1), buffer ^ 1);      // (read for the last time ahead of the last barrier)
+        if (counted + 1 < groups) fetch(group_at(counted + 1), buffer ^ 1);
         const int k0 = group_at(counted) * GROUP;
         const unsigned char* tiles = lds_raw + (size_t)buffer * buffer_bytes + lane * 16;
         auto tile_at = [&](int t) { return *reinterpret_cast<const bf16x8*>(tiles + (size_t)t * TILE_BYTES); };
-        floatx4 s[SETS][2];
-#pragma unroll
-        for (int w = 0; w < SETS; ++w) s[w][0] = s[w][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+        floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
         // A tile is read AHEAD steps before it is multiplied. (The fences between the steps keep the compiler from reading
         // all of them at once.)
         bf16x8 ahead[AHEAD][2];
@@ -418,11 +403,8 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
             __builtin_amdgcn_sched_barrier(0);
             const bf16x8 first = ahead[step % AHEAD][0], second = ahead[step % AHEAD][1];
             if (step + AHEAD < KS) { ahead[step % AHEAD][0] = tile_at(step + AHEAD); ahead[step % AHEAD][1] = tile_at(KS + step + AHEAD); }
-#pragma unroll
-            for (int w = 0; w < SETS; ++w) {
-                s[w][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(first, queries[w][step], s[w][0], 0, 0, 0);
-                s[w][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(second, queries[w][step], s[w][1], 0, 0, 0);
-            }
+            s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(first, queries[step], s[0], 0, 0, 0);
+            s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(second, queries[step], s[1], 0, 0, 0);
         }
         // the first values are on their way while the softmax is done
 #pragma unroll
@@ -430,45 +412,42 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
         __builtin_amdgcn_sched_barrier(0);
         // register i of tile t is the key k0 + 8 quarter + 4 t + i, for the row of this lane's column
         const bool masked = k0 + GROUP - 1 > wave_low || k0 < wave_all;
-        bf16x8 rounded[SETS], rest[SETS];
+        if constexpr (CAP) {
 #pragma unroll
-        for (int w = 0; w < SETS; ++w) {
-            if constexpr (CAP) {
+            for (int e = 0; e < 8; ++e) s[e / 4][e % 4] = capped(s[e / 4][e % 4], to_power, cap2);
+        }
+        if (masked) {
+            const Seen seen(pos, window, keep_first);
 #pragma unroll
-                for (int e = 0; e < 8; ++e) s[w][e / 4][e % 4] = capped(s[w][e / 4][e % 4], to_power, cap2);
-            }
-            if (masked) {
-                const Seen seen(pos[w], window, keep_first);
+            for (int e = 0; e < 8; ++e)
+                if (!seen.sees(k0 + quarter * 8 + e, pos)) s[e / 4][e % 4] = -INFINITY;
+        }
+        float top = s[0][0];
 #pragma unroll
-                for (int e = 0; e < 8; ++e)
-                    if (!seen.sees(k0 + quarter * 8 + e, pos[w])) s[w][e / 4][e % 4] = -INFINITY;
-            }
-            float top = s[w][0][0];
+        for (int e = 1; e < 8; ++e) top = fmaxf(top, s[e / 4][e % 4]);
+        top *= scale2;                                     // (the scale is positive: checked on the host)
+        // m is the exponent that the sums are relative to; it moves only when some row meets a score more than 8 above it (in
+        // log2), until when the weights stay below 2^8 and the quotient in the end is the same.
+        if (__builtin_amdgcn_ballot_w64(top > m + 8.0f) != 0) {
+            float here = fmaxf(top, __shfl_xor(top, 16, XRT_WAVE));
+            here = fmaxf(here, __shfl_xor(here, 32, XRT_WAVE));
+            const float m_new = fmaxf(m, here);
+            const float correction = __builtin_amdgcn_exp2f(m - (m_new == -INFINITY ? 0.f : m_new));
+            m = m_new;
+            l *= correction;
 #pragma unroll
-            for (int e = 1; e < 8; ++e) top = fmaxf(top, s[w][e / 4][e % 4]);
-            top *= scale2;                                     // (the scale is positive: checked on the host)
-            // m is the exponent that the sums are relative to; it moves only when some row meets a score more than 8 above it (in
-            // log2), until when the weights stay below 2^8 and the quotient in the end is the same.
-            if (__builtin_amdgcn_ballot_w64(top > m[w] + 8.0f) != 0) {
-                float here = fmaxf(top, __shfl_xor(top, 16, XRT_WAVE));
-                here = fmaxf(here, __shfl_xor(here, 32, XRT_WAVE));
-                const float m_new = fmaxf(m[w], here);
-                const float correction = __builtin_amdgcn_exp2f(m[w] - (m_new == -INFINITY ? 0.f : m_new));
-                m[w] = m_new;
-                l[w] *= correction;
+            for (int u = 0; u < VT; ++u)
 #pragma unroll
-                for (int u = 0; u < VT; ++u)
+                for (int j = 0; j < 4; ++j) o[u][j] *= correction;
+        }
+        bf16x8 rounded, rest;
+        const float m_safe = m == -INFINITY ? 0.f : m;       // a row that has seen no key yet
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) o[w][u][j] *= correction;
-            }
-            const float m_safe = m[w] == -INFINITY ? 0.f : m[w];       // a row that has seen no key yet
-#pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const float weight = __builtin_amdgcn_exp2f(fmaf(s[w][e / 4][e % 4], scale2, -m_safe));
-                l[w] += weight;
-                rounded[w][e] = (bf16)weight;
-                rest[w][e] = (bf16)(weight - (float)rounded[w][e]);
-            }
+        for (int e = 0; e < 8; ++e) {
+            const float weight = __builtin_amdgcn_exp2f(fmaf(s[e / 4][e % 4], scale2, -m_safe));
+            l += weight;
+            rounded[e] = (bf16)weight;
+            rest[e] = (bf16)(weight - (float)rounded[e]);
         }
         const bool edge = k0 + GROUP - 1 > pos_high;       // what lies behind the last key may be anything: kept away from the weights' zeros
 #pragma unroll
@@ -487,57 +466,49 @@ __global__ void __launch_bounds__(PROMPT_WAVES * XRT_WAVE) latent_prompts_kernel
                         if (k0 + quarter * 8 + e > pos_high) value[i][e] = (bf16)0.f;
             }
 #pragma unroll
-            for (int w = 0; w < SETS; ++w)
+            for (int i = 0; i < 2; ++i)
+                o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rounded, o[u0 + i], 0, 0, 0);
 #pragma unroll
-                for (int i = 0; i < 2; ++i)
-                    o[w][u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rounded[w], o[w][u0 + i], 0, 0, 0);
-#pragma unroll
-            for (int w = 0; w < SETS; ++w)
-#pragma unroll
-                for (int i = 0; i < 2; ++i)
-                    o[w][u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rest[w], o[w][u0 + i], 0, 0, 0);
+            for (int i = 0; i < 2; ++i)
+                o[u0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value[i], rest, o[u0 + i], 0, 0, 0);
         }
-        wait_loads_and_barrier<0>();                       // the next group has arrived from every wavefront, this one has been read by all
     }
     if (!awake) return;
+    float sum = l;
+    sum += __shfl_xor(sum, 16, XRT_WAVE);
+    sum += __shfl_xor(sum, 32, XRT_WAVE);
+    if (sinks != nullptr) sum += __builtin_amdgcn_exp2f(fmaf(sinks[head], LOG2E, -(m == -INFINITY ? 0.f : m)));    // (relative to the same exponent)
+    const float inv = sum > 0.f ? 1.0f / sum : 0.f;
+    if (row < rows) {
+        // register i of tile u is dim 16 u + 4 quarter + i of this lane's row
+        bf16* dst = out + at(row) * value_dim + quarter * 4;
 #pragma unroll
-    for (int w = 0; w < SETS; ++w) {
-        float sum = l[w];
-        sum += __shfl_xor(sum, 16, XRT_WAVE);
-        sum += __shfl_xor(sum, 32, XRT_WAVE);
-        if (sinks != nullptr) sum += __builtin_amdgcn_exp2f(fmaf(sinks[head[w]], LOG2E, -(m[w] == -INFINITY ? 0.f : m[w])));    // (relative to the same exponent)
-        const float inv = sum > 0.f ? 1.0f / sum : 0.f;
-        if (row[w] < rows) {
-            // register i of tile u is dim 16 u + 4 quarter + i of this lane's row
-            bf16* dst = out + at(row[w]) * value_dim + quarter * 4;
+        for (int u = 0; u < VT; ++u) {
+            if (u < value_tiles) {
+                struct alignas(8) Four { bf16 e[4]; } four;
 #pragma unroll
-            for (int u = 0; u < VT; ++u) {
-                if (u < value_tiles) {
-                    struct alignas(8) Four { bf16 e[4]; } four;
-#pragma unroll
-                    for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(o[w][u][i] * inv);
-                    *reinterpret_cast<Four*>(dst + u * 16) = four;
-                }
+                for (int i = 0; i < 4; ++i) four.e[i] = (bf16)(o[u][i] * inv);
+                *reinterpret_cast<Four*>(dst + u * 16) = four;
             }
         }
     }
 }
 
-template <int KS, int VT, int SETS, bool CAP>
+template <int KS, int VT, int WAVES, bool CAP>
 int launch_prompts(const bf16* q, long tokens, const Shape& shape, const bf16* k_cache, const bf16* v_cache, const int* block_table, int table_stride,
                    int n_blocks, const int* seq_offsets, const int* seq_slots, const int* seq_starts, int n_seqs, float scale, float softcap,
                    const float* sinks, bf16* out, hipStream_t s) {
-    constexpr int TILE_ROWS = PROMPT_WAVES * SETS * SET_ROWS;
+    constexpr int TILE_ROWS = WAVES * WAVE_ROWS;
     const long tiles = tokens * shape.group() / TILE_ROWS + n_seqs;     // every sequence's last tile may be partly filled
     XRT_REQUIRE(tiles < (1L << 31), "attention (latent, prompts): too many rows");
     constexpr size_t lds = (size_t)2 * (2 * KS + VT) * TILE_BYTES;
     static bool configured = false;                            // per instantiation
     if (!configured) {
-        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_prompts_kernel<KS, VT, SETS, CAP>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_prompts_kernel<KS, VT, WAVES, CAP>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         XRT_REQUIRE(e == hipSuccess, "attention (latent, prompts): cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(e));
         configured = true;
     }
-    latent_prompts_kernel<KS, VT, SETS, CAP><<<dim3((unsigned)tiles, shape.n_kv_heads), PROMPT_WAVES * XRT_WAVE, lds, s>>>(
+    latent_prompts_kernel<KS, VT, WAVES, CAP><<<dim3((unsigned)tiles, shape.n_kv_heads), WAVES * XRT_WAVE, lds, s>>>(
         q, shape, k_cache, v_cache, block_table, table_stride, n_blocks, seq_offsets, seq_slots, seq_starts, n_seqs, scale, softcap, sinks, out);
     XRT_LAUNCH_CHECK("attention (latent, prompts)");
     return 0;
@@ -587,8 +558,11 @@ extern "C" int xrt_attention_latent(const void* q, long q_stride, long tokens, i
     else XRT_CHUNKS(KEY_STEPS, VALUE_TILES, false);
 #undef XRT_CHUNKS
     XRT_LAUNCH_CHECK("attention (latent, chunks)");
-    latent_merge_kernel<<<dim3((unsigned)tokens, n_heads), XRT_WAVE, 0, (hipStream_t)stream>>>(workspace, shape, chunk_groups, chunks, positions, slots, sink_scores,
-                                                                                              (bf16*)out);
+#define XRT_MERGE(OWNED_)                                                                                                                               \
+    latent_merge_kernel<OWNED_><<<dim3((unsigned)tokens, n_heads), XRT_WAVE, 0, (hipStream_t)stream>>>(workspace, shape, chunk_groups, chunks, positions, \
+                                                                                                      slots, sink_scores, (bf16*)out)
+    if (value_dim <= 2 * XRT_WAVE) XRT_MERGE(2); else XRT_MERGE(LATENT_MOST / XRT_WAVE);
+#undef XRT_MERGE
     XRT_LAUNCH_CHECK("attention (latent, merge)");
     return 0;
 }
@@ -610,15 +584,16 @@ extern "C" int xrt_attention_latent_prompts(const void* q, long tokens, int n_he
         return launcher((const bf16*)q, tokens, shape, (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, n_blocks, seq_offsets, seq_slots,
                         seq_starts, n_seqs, scale, softcap, sink_scores, (bf16*)out, (hipStream_t)stream);
     };
-    // the instantiation that holds the sizes with the least to spare
-#define XRT_PROMPTS(KS_, VT_, SETS_) (softcap > 0.f ? run(launch_prompts<KS_, VT_, SETS_, true>) : run(launch_prompts<KS_, VT_, SETS_, false>))
-    if (head_dim <= 64 && value_dim <= 64) return XRT_PROMPTS(2, 4, 2);
-    if (head_dim <= 128 && value_dim <= 128) return XRT_PROMPTS(4, 8, 2);
-    if (head_dim <= 192 && value_dim <= 128) return XRT_PROMPTS(6, 8, 1);
-    if (head_dim <= 256 && value_dim <= 192) return XRT_PROMPTS(8, 12, 1);
-    if (head_dim <= 320 && value_dim <= 256) return XRT_PROMPTS(10, 16, 1);
-    if (head_dim <= 448 && value_dim <= 384) return XRT_PROMPTS(14, 24, 1);
-    if (head_dim <= 576) return XRT_PROMPTS(18, 32, 1);
-    return XRT_PROMPTS(20, 32, 1);
+    // the instantiation that holds the sizes with the least to spare (the largest ones in workgroups of four wavefronts, which may have
+    // twice the registers each)
+#define XRT_PROMPTS(KS_, VT_, WAVES_) (softcap > 0.f ? run(launch_prompts<KS_, VT_, WAVES_, true>) : run(launch_prompts<KS_, VT_, WAVES_, false>))
+    if (head_dim <= 64 && value_dim <= 64) return XRT_PROMPTS(2, 4, 8);
+    if (head_dim <= 128 && value_dim <= 128) return XRT_PROMPTS(4, 8, 8);
+    if (head_dim <= 192 && value_dim <= 128) return XRT_PROMPTS(6, 8, 8);
+    if (head_dim <= 256 && value_dim <= 192) return XRT_PROMPTS(8, 12, 8);
+    if (head_dim <= 320 && value_dim <= 256) return XRT_PROMPTS(10, 16, 8);
+    if (head_dim <= 448 && value_dim <= 384) return XRT_PROMPTS(14, 24, 8);
+    if (head_dim <= 576) return XRT_PROMPTS(18, 32, 4);
+    return XRT_PROMPTS(20, 32, 4);
 #undef XRT_PROMPTS
 }
