@@ -185,3 +185,38 @@ def test_random_traffic_keeps_the_books(seed=0):
         cache.free_slot(slot)
     cache.check()
     assert cache.held_blocks() == 0 and cache.slots.n_free == 5
+
+
+def test_a_window_may_keep_a_sequences_first_tokens():
+    needs = [CacheNeeds(kv=KVSpec(2, 16, window=100, keep_first=70)), CacheNeeds(kv=KVSpec(2, 16, window=100)), CacheNeeds(kv=KVSpec(2, 16, window=100, keep_first=64))]
+    cache = SequenceCache(needs, [0, 1, 2], 2048, 2, 1024, torch.float32, "cpu")
+    assert len(cache.groups) == 3                          # what a window keeps is part of what a layer call needs
+    two, none, one = (next(g for g in cache.groups if g.spec.keep_first == n) for n in (70, 0, 64))
+    a = cache.alloc_slot()
+    cache.reserve(a, 600); cache.commit(a, 600)            # a query at 600 sees keys 501..: blocks 7, 8, 9, and the first 70 keys: 0 and 1
+    blocks = lambda group: [i for i, x in enumerate(group.table[a].tolist()) if x >= 0]
+    assert blocks(two) == [0, 1, 7, 8, 9] and blocks(none) == [7, 8, 9] and blocks(one) == [0, 7, 8, 9]
+    for length in range(601, 700):
+        cache.reserve(a, length); cache.commit(a, length)
+    assert blocks(two) == [0, 1, 9, 10] and blocks(one) == [0, 9, 10]
+    cache.check()
+    b = cache.alloc_slot()
+    cache.reserve(b, 65); cache.commit(b, 65)
+    cache.truncate(b, 3)                                   # nothing that a shorter sequence sees is gone
+    cache.check()
+    with pytest.raises(CacheError, match="released"):
+        cache.truncate(a, 300)
+    cache.free_slot(a)
+    cache.free_slot(b)
+    assert all(group.pool.n_held == 0 for group in cache.groups)
+    cache.check()
+
+
+def test_a_window_that_has_let_go_of_nothing_but_kept_tokens_can_be_rolled_back():
+    cache = SequenceCache([CacheNeeds(kv=KVSpec(1, 16, window=10, keep_first=128))], [0], 1024, 1, 1024, torch.float32, "cpu")
+    a = cache.alloc_slot()
+    cache.reserve(a, 130); cache.commit(a, 130)
+    cache.truncate(a, 20)
+    cache.reserve(a, 90); cache.commit(a, 90)
+    cache.check()
+    assert cache.groups[0].pool.n_held == 2
