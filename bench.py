@@ -56,7 +56,7 @@ every fourth layer runs the weights of the one before it once more), beside the 
 
 the same for the Fisopel decoder (attention through a cached latent with a gate per output, and grouped attention with head norms, capped
 scores and a learnt sink under a window of 512 keys that keeps the first four, in turn, each beside eight experts of which a token
-uses two and a shared one; one pass through the layers), beside the Mitunex decoder, the library's closest (attention through a latent,
+uses two and a shared one; the first two layers run twice in a row), beside the Mitunex decoder, the library's closest (attention through a latent,
 experts beside a shared one), and Llama.
 """
 import argparse
@@ -231,8 +231,8 @@ def fisopel_config(size, layers, max_positions):
     experts = {"kind": "moe", "expert": {"ff": ff // 2}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 2}}
     kinds = [("latent_attention", latent), ("attention", windowed)]
     return {"architecture": "Fisopel", "vocab": size["vocab"], "width": w, "norm": {"eps": 1e-6}, "embedding": {"scale": w ** 0.5},
-            "loop": {"start": 0, "stop": max(1, layers), "times": 1},
-            "layers": [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": experts} for i in range(layers)]}
+            "loop": {"start": 0, "stop": 2, "times": 2} if layers >= 4 else None,           # (the first two layers' second run counts among the layers)
+            "layers": [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": experts} for i in range(layers - 2 if layers >= 4 else layers)]}
 
 
 DESIGN_CONFIGS = {"sozopel": sozopel_config, "ledudra": ledudra_config, "depunex": depunex_config, "renapel": renapel_config,
