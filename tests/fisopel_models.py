@@ -57,7 +57,7 @@ TILES = _model(130, 64, 1e-6, 0.5, [
     _latent(5, 24, 32, 48, 96, 0.2, 5000.0, _moe(128, 6, 3, 64), scaling=(8.0, 32, 4.0, 1.0)),
     _attention(20, 1, 32, 32, 0.5, _moe(64, 8, 2), size=33, keep_first=34),
     _attention(3, 3, 128, 64, 0.2, _moe(64, 3, 2, 192), softcap=5.0),
-], loop=(0, 2, 3))
+], loop=(0, 1, 3))
 
 # edges: a window of one token, everything chosen, a loop over all layers that is gone through once, nothing capped, a scale of one
 EDGES = _model(64, 32, 1e-3, 1.0, [

@@ -332,7 +332,7 @@ def attend(ops, q, k, v, cuts, dtype, n_heads, n_kv_heads, dim, vdim, ahead=0, w
 
 # heads, key/value heads, key size, value size: in whole tiles (the matrix-core kernels in bfloat16), and not
 TILES = [(8, 2, 64, 96), (16, 16, 32, 32), (20, 1, 128, 64), (4, 2, 128, 128), (34, 2, 64, 64), (6, 3, 192, 160), (2, 1, 448, 384), (3, 1, 576, 512), (5, 5, 64, 128)]
-OTHERS = [(6, 3, 64, 80), (4, 1, 40, 24), (5, 5, 7, 3), (12, 2, 100, 130), (2, 2, 33, 32)]
+OTHERS = [(9, 3, 64, 72), (4, 1, 40, 24), (5, 5, 7, 3), (12, 2, 100, 130), (2, 2, 33, 32)]
 
 
 @pytest.mark.parametrize("dtype,sizes", [(torch.bfloat16, s) for s in TILES + OTHERS] + [(torch.float32, s) for s in OTHERS + TILES[:2] + TILES[6:7]])
@@ -387,14 +387,14 @@ def test_one_key_far_back_is_found_under_a_cap(dtype, n_heads, n_kv_heads, dim, 
         assert float((got[-20:] - 7.0).abs().max()) < 0.1, f"key {key}, cuts {cuts[:2]}"
 
 
-@pytest.mark.parametrize("dtype,dim,vdim", [(torch.float32, 24, 16), (torch.bfloat16, 64, 64), (torch.bfloat16, 64, 80)])
+@pytest.mark.parametrize("dtype,dim,vdim", [(torch.float32, 24, 16), (torch.bfloat16, 64, 64), (torch.bfloat16, 64, 72)])
 def test_a_cap_flattens_scores_far_above_it_and_leaves_small_ones(dtype, dim, vdim, ops):
     """Scores of some hundreds under a cap of two: all that are large have nearly the same weight; and scores of thousandths, which the
     cap must leave as they are."""
     n_heads, length = 4, 140
     generator = torch.Generator().manual_seed(2)
     q, k, v = (torch.randn(length, width, generator=generator).bfloat16().float() for width in (n_heads * dim, 2 * dim, 2 * vdim))
-    for scale, cap in ((40.0, 2.0), (1e-3, 50.0), (3.0, 30.0), (500.0, 0.01)):
+    for scale, cap in ((40.0, 2.0), (1e-3, 60.0), (3.0, 30.0), (500.0, 0.01)):
         want = plain_attention(q, k, v, n_heads, 2, scale, 50, 3, cap, torch.full((n_heads,), -1.0))
         for cuts in ([length], [length - 6] + [1] * 6):
             got = attend(ops, q, k, v, cuts, dtype, n_heads, 2, dim, vdim, scale=scale, window=50, keep_first=3, softcap=cap, sink=torch.full((n_heads,), -1.0).cuda())
